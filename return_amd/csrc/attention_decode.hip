@@ -71,15 +71,35 @@ __device__ __forceinline__ DecodeRange decode_range(int pos_q, int start, int wi
     return r;
 }
 
-// The optional extras (XT): head_scale[h] multiplies the scale of query head h; softcap c turns a score s
-// into c tanh(s / c); keep_first as above; sink adds one to the softmax's denominator (a key of score 0
-// that has no value), where the splits are merged.
+// The optional extras (XT 1 or 2): head_scale[h] multiplies the scale of query head h; softcap c turns a score s
+// into c tanh(s / c); keep_first as above; sink adds exp(sink_logit[h]) to the softmax's denominator (one, a key
+// of score 0, where sink_logit is null), a key that has no value, where the splits are merged; out_scale multiplies
+// the result before it is stored; out's rows are ld_out elements apart (0: the heads of a token and nothing else).
+// With fine_weights (XT 2) the weights go into the product with the values as two bfloat16 halves.
 struct DecodeExtras {
     const float* head_scale;
     float softcap;
     int keep_first;
     int sink;
+    const float* sink_logit;
+    float out_scale;
+    long long ld_out;
+    int fine_weights;
 };
+#define DEC_NO_EXTRAS {nullptr, 0.f, 0, 0, nullptr, 1.f, 0, 0}
+
+// The sink's part of a merge: given the maximum mx (base-2 exponents), the sum l and the head's sink, what the sums
+// are multiplied by after the sink has entered (their scale, the result's factor and 1 / denominator).
+__device__ __forceinline__ float decode_finish(float mx, float l, const DecodeExtras& ex, int head) {
+    float rescale = 1.f;
+    if (ex.sink) {
+        const float sl = ex.sink_logit != nullptr ? ex.sink_logit[head] * 1.44269504088896340736f : 0.f;
+        const float top = fmaxf(mx, sl);
+        rescale = __builtin_amdgcn_exp2f(mx - top);
+        l = fmaf(l, rescale, __builtin_amdgcn_exp2f(sl - top));
+    }
+    return l > 0.f ? rescale * ex.out_scale / l : 0.f;
+}
 
 // What the kernel needs to prepare the new token's q, k and v itself (the work of the q/k/v
 // preparation kernel: per-head RMSNorm of q and k, rotation, k and v into the cache;
@@ -219,7 +239,7 @@ __host__ __device__ constexpr int dec_region_bytes(int D) {
 // per (request, kv head), wave w takes split w, and the waves' sums are merged through LDS here
 // (the same sums in the same order as the merge kernel), so that nothing goes through memory and
 // no second kernel runs; for requests whose splits fit one workgroup.
-template <int D16, bool FUSED, bool XT>
+template <int D16, bool FUSED, int XT>
 __global__ __launch_bounds__(D16 <= 8 ? 512 : 256) __attribute__((amdgpu_waves_per_eu(D16 <= 8 ? 2 : 1)))
 void attn_decode_kernel(
     const bf16* __restrict__ q, float* __restrict__ part_acc, float* __restrict__ part_ml,
@@ -260,7 +280,7 @@ void attn_decode_kernel(
     // A merging workgroup cuts its own request into merge_waves even splits (counted from
     // position 0), whatever the longest request of the step is.
     if (merge_waves > 1) split_tokens = max(1, (pos_q + DEC_CHUNK * merge_waves) / (DEC_CHUNK * merge_waves)) * DEC_CHUNK;
-    const DecodeRange rg = decode_range(pos_q, start, window, split_tokens, sp, XT ? ex.keep_first : 0);
+    const DecodeRange rg = decode_range(pos_q, start, window, split_tokens, sp, XT != 0 ? ex.keep_first : 0);
     const bool empty = rg.lo > rg.hi;            // a split beyond the request's keys
     if (empty && merge_waves == 1) return;       // (in a merging workgroup the wave stays for the barrier, with no keys)
     const int* pt = page_table + first_page;
@@ -377,8 +397,8 @@ void attn_decode_kernel(
     const float scale2 = scale * 1.44269504088896340736f;      // scores in the base-2 domain
     // XT: this lane's head has a factor of its own on the scale, and the score is capped before it enters the softmax
     [[maybe_unused]] const float head_scale =
-        XT ? scale * ((ex.head_scale != nullptr && n < G) ? ex.head_scale[h0 + n] : 1.f) : 0.f;
-    [[maybe_unused]] const float inv_cap = (XT && ex.softcap > 0.f) ? 1.0f / ex.softcap : 0.f;
+        XT != 0 ? scale * ((ex.head_scale != nullptr && n < G) ? ex.head_scale[h0 + n] : 1.f) : 0.f;
+    [[maybe_unused]] const float inv_cap = (XT != 0 && ex.softcap > 0.f) ? 1.0f / ex.softcap : 0.f;
     float m_run = -INFINITY, l_run = 0.f;
     float4_t acc[D16];                           // acc[dt][i] = O^T[d = 16dt + 4g + i][head n]
 #pragma unroll
@@ -429,7 +449,7 @@ void attn_decode_kernel(
             for (int i = 0; i < 4; ++i) {
                 const int kp_abs = c0 + st * 16 + 4 * g + i;
                 const bool ok = kp_abs >= rg.lo && kp_abs <= key_hi;
-                if constexpr (XT) {
+                if constexpr (XT != 0) {
                     float t = cs[st][i] * head_scale;
                     if (ex.softcap > 0.f) {                 // c tanh(t / c) = c (1 - 2 / (1 + e^(2t/c)))
                         const float e2 = __builtin_amdgcn_exp2f(t * inv_cap * 2.88539008177792681472f);
@@ -473,6 +493,16 @@ void attn_decode_kernel(
             const uint4_t pw = {pack2(s[2 * b][0], s[2 * b][1]), pack2(s[2 * b][2], s[2 * b][3]),
                                 pack2(s[2 * b + 1][0], s[2 * b + 1][1]), pack2(s[2 * b + 1][2], s[2 * b + 1][3])};
             const bf16x8_t pb = __builtin_bit_cast(bf16x8_t, pw);
+            [[maybe_unused]] bf16x8_t pl = z8;       // XT 2: what the weights lack in bf16
+            if constexpr (XT == 2) {
+                uint4_t lw;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const int st = 2 * b + (j >> 1), i = 2 * (j & 1);
+                    lw[j] = pack2(s[st][i] - __uint_as_float(pw[j] << 16), s[st][i + 1] - __uint_as_float(pw[j] & 0xffff0000u));
+                }
+                pl = __builtin_bit_cast(bf16x8_t, lw);
+            }
             // this lane's address as lane l' = n of its group: key 32b + 4g + n/4, columns 4(n%4)..+3
             const uint16_t* vr = &v_s[(32 * b + 4 * g + (n >> 2)) * VS + 4 * (n & 3)];
 #pragma unroll
@@ -481,6 +511,8 @@ void attn_decode_kernel(
                 const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4_ptr)(vr + 16 * VS + dt * 16));
                 const short8_t both = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
                 acc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, both), pb, acc[dt], 0, 0, 0);
+                if constexpr (XT == 2)
+                    acc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, both), pl, acc[dt], 0, 0, 0);
             }
         }
     }
@@ -550,12 +582,16 @@ void attn_decode_kernel(
                 o[2] = fmaf(a[2], e, o[2]); o[3] = fmaf(a[3], e, o[3]);
                 l += other[16 * D + 2 * hn + 1] * e;
             }
-            if constexpr (XT) {
-                if (ex.sink) l += __builtin_amdgcn_exp2f(-mx);       // the key of score 0 without a value
+            float inv;
+            size_t row = (size_t)t * Hq * D;
+            if constexpr (XT != 0) {
+                inv = decode_finish(mx, l, ex, h0 + hn);
+                if (ex.ld_out) row = (size_t)t * ex.ld_out;
+            } else {
+                inv = l > 0.f ? 1.0f / l : 0.f;
             }
-            const float inv = l > 0.f ? 1.0f / l : 0.f;
             const uint2 packed = {pack2(o[0] * inv, o[1] * inv), pack2(o[2] * inv, o[3] * inv)};
-            *reinterpret_cast<uint2*>(out + ((size_t)t * Hq + h0 + hn) * D + 4 * d4) = packed;
+            *reinterpret_cast<uint2*>(out + row + (size_t)(h0 + hn) * D + 4 * d4) = packed;
         }
         return;
     }
@@ -576,7 +612,7 @@ void attn_decode_kernel(
 #define DEC_CAT2(a, b) a##b
 #define DEC_CAT(a, b) DEC_CAT2(a, b)
 // head sizes 16*(4*DEC_PART+1) .. 16*(4*DEC_PART+4)
-template <int N, bool FUSED, bool XT>
+template <int N, bool FUSED, int XT>
 static int dec_launch_one(dim3 grid, hipStream_t st, const bf16* q, float* pa, float* pm, const bf16* kp,
                           const bf16* vp, const int* pt, const int* cup, const int* kvs, const int* cuq,
                           const int* qs, const int* segs, int Hq, int Hkv, int P, float scale, int window,
@@ -607,14 +643,16 @@ extern "C" int DEC_CAT(ra_dec_part_, DEC_PART)(int D16, dim3 grid, hipStream_t s
                                               DecodeExtras ex) {
 #define DEC_ARGS grid, st, q, pa, pm, kp, vp, pt, cup, kvs, cuq, qs, segs, Hq, Hkv, P, scale, window, \
                  split_tokens, max_splits, fz, merge_waves, out, ex
-    const bool extras = ex.head_scale != nullptr || ex.softcap > 0.f || ex.keep_first > 0 || ex.sink != 0;
+    const bool extras = ex.head_scale != nullptr || ex.softcap > 0.f || ex.keep_first > 0 || ex.sink != 0 ||
+                        ex.out_scale != 1.f || ex.ld_out != 0;
     if (fz.qkv != nullptr) {                      // head sizes 64, 128, 192, 256: one of them in each part
-        if (D16 != 4 * DEC_PART + 4 || extras) return RA_ERR_ARG;
-        return dec_launch_one<4 * DEC_PART + 4, true, false>(DEC_ARGS);
+        if (D16 != 4 * DEC_PART + 4 || extras || ex.fine_weights) return RA_ERR_ARG;
+        return dec_launch_one<4 * DEC_PART + 4, true, 0>(DEC_ARGS);
     }
 #define DEC_CASE(N_)                                                                  \
     case N_:                                                                          \
-        return extras ? dec_launch_one<N_, false, true>(DEC_ARGS) : dec_launch_one<N_, false, false>(DEC_ARGS);
+        return ex.fine_weights ? dec_launch_one<N_, false, 2>(DEC_ARGS)               \
+               : extras ? dec_launch_one<N_, false, 1>(DEC_ARGS) : dec_launch_one<N_, false, 0>(DEC_ARGS);
     switch (D16) {
         DEC_CASE(4 * DEC_PART + 1)
         DEC_CASE(4 * DEC_PART + 2)
@@ -658,7 +696,7 @@ __global__ __launch_bounds__(128 * GROUPS) void attn_decode_combine_kernel(
     const float* __restrict__ part_acc, const float* __restrict__ part_ml, bf16* __restrict__ out,
     const int* __restrict__ kv_start, const int* __restrict__ cu_q, const int* __restrict__ q_start,
     const int* __restrict__ seg_ids, int Hq, int D, int window, int split_tokens, int max_splits,
-    int keep_first, int sink) {
+    DecodeExtras ex) {
     const int di = blockIdx.x, head = blockIdx.y, tid = threadIdx.x & 127, grp = threadIdx.x >> 7;
     // this group's run of splits: [first, first + per)
     const int per = GROUPS == 1 ? max_splits : (max_splits + GROUPS - 1) / GROUPS;
@@ -681,7 +719,7 @@ __global__ __launch_bounds__(128 * GROUPS) void attn_decode_combine_kernel(
     }
     const int seg = seg_ids ? seg_ids[di] : di;
     const int t = cu_q ? cu_q[seg] : seg;
-    const DecodeRange rg = decode_range(q_start[seg], kv_start[seg], window, split_tokens, 0, keep_first);
+    const DecodeRange rg = decode_range(q_start[seg], kv_start[seg], window, split_tokens, 0, ex.keep_first);
     const int ns_all = min(rg.n_splits, max_splits);
     const int ns = max(0, min(ns_all - first, per));        // splits of this group that hold keys
     float m = -INFINITY;                                   // (the maxima are base-2 exponents)
@@ -726,9 +764,8 @@ __global__ __launch_bounds__(128 * GROUPS) void attn_decode_combine_kernel(
         }
         m = mx;
     }
-    if (sink) l += __builtin_amdgcn_exp2f(-m);             // the key of score 0 without a value (base-2 exponents)
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
-    bf16* o = out + ((size_t)t * Hq + head) * D;
+    const float inv = decode_finish(m, l, ex, head);
+    bf16* o = out + (size_t)t * (ex.ld_out ? (size_t)ex.ld_out : (size_t)Hq * D) + (size_t)head * D;
     if (tid < D) o[tid] = from_f<bf16>(o0 * inv);
     if (tid + 128 < D) o[tid + 128] = from_f<bf16>(o1 * inv);
 }
@@ -752,7 +789,7 @@ static int decode_launch(const bf16* qq, void* out, float* pa, float* pm, const 
                          const int* page_table, const int* cu_pages, const int* kv_start, const int* cu_q,
                          const int* q_start, const int* seg_ids, int n_dec, int Hq, int Hkv, int D, int P,
                          float scale, int window, int split_tokens, int max_splits, DecodeFused fz,
-                         int merge, hipStream_t st, DecodeExtras ex = DecodeExtras{nullptr, 0.f, 0, 0}) {
+                         int merge, hipStream_t st, DecodeExtras ex = DecodeExtras DEC_NO_EXTRAS) {
     if (n_dec <= 0) return RA_OK;
     if (D % 16 != 0 || D < 16 || D > 256 || Hkv <= 0 || Hq % Hkv != 0 ||
         split_tokens <= 0 || split_tokens % DEC_CHUNK != 0 || max_splits <= 0 || max_splits > 65535 || P <= 0)
@@ -779,8 +816,7 @@ static int decode_launch(const bf16* qq, void* out, float* pa, float* pm, const 
     if (hipGetLastError() != hipSuccess) return RA_ERR_LAUNCH;
     if (merge) return RA_OK;
 #define DEC_COMBINE(G) hipLaunchKernelGGL(attn_decode_combine_kernel<G>, dim3(n_dec, Hq), dim3(128 * G), 0, st, pa, pm, \
-                                          (bf16*)out, kv_start, cu_q, q_start, seg_ids, Hq, D, window, split_tokens, max_splits, \
-                                          ex.keep_first, ex.sink)
+                                          (bf16*)out, kv_start, cu_q, q_start, seg_ids, Hq, D, window, split_tokens, max_splits, ex)
     const int groups = (max_splits + COMBINE_AHEAD - 1) / COMBINE_AHEAD;
     if (groups <= 1) DEC_COMBINE(1);
     else if (groups <= 2) DEC_COMBINE(2);
@@ -804,7 +840,8 @@ extern "C" int ra_attention_decode_bf16(const void* q, void* out, void* part_acc
 }
 
 // The same with the optional extras: head_scale (fp32 [Hq] or null), softcap (0: none), keep_first (the
-// keys below it are one more split where the window has moved past them: max_splits counts it), sink.
+// keys below it are one more split where the window has moved past them: max_splits counts it), sink with
+// sink_logit (fp32 [Hq] or null), out_scale, ld_out (elements from one token's row of out to the next), fine_weights.
 extern "C" int ra_attention_decode_extras_bf16(const void* q, void* out, void* part_acc, void* part_ml,
                                                const void* k_pool, const void* v_pool,
                                                const int* page_table, const int* cu_pages,
@@ -812,10 +849,13 @@ extern "C" int ra_attention_decode_extras_bf16(const void* q, void* out, void* p
                                                const int* seg_ids, int n_dec, int Hq, int Hkv, int D, int P,
                                                float scale, int window, int split_tokens, int max_splits,
                                                int merge, const float* head_scale, float softcap, int keep_first,
-                                               int sink, void* stream) {
+                                               int sink, const float* sink_logit, float out_scale, long long ld_out,
+                                               int fine_weights, void* stream) {
     DecodeFused none = {};
-    if (softcap < 0.f || keep_first < 0) return RA_ERR_ARG;
-    const DecodeExtras ex = {head_scale, softcap, window > 0 ? keep_first : 0, sink};
+    if (softcap < 0.f || keep_first < 0 || ld_out < (long long)Hq * D || ld_out % 4 != 0 || ((uintptr_t)out & 7) != 0)
+        return RA_ERR_ARG;
+    const DecodeExtras ex = {head_scale, softcap, window > 0 ? keep_first : 0, sink, sink_logit, out_scale,
+                             ld_out == (long long)Hq * D ? 0 : ld_out, fine_weights};
     return decode_launch((const bf16*)q, out, (float*)part_acc, (float*)part_ml, (const bf16*)k_pool,
                          (const bf16*)v_pool, page_table, cu_pages, kv_start, cu_q, q_start, seg_ids, n_dec, Hq,
                          Hkv, D, P, scale, window, split_tokens, max_splits, none, merge, (hipStream_t)stream, ex);

@@ -23,8 +23,9 @@
 //
 // Optional, each off at 0 / null: head_scale[h] multiplies the scale of query head h; softcap c
 // turns a score s into c tanh(s / c); keep_first n lets every query also read the keys at positions
-// below n, whatever the window; sink adds one to the softmax's denominator (a key of score 0 that
-// has no value).
+// below n, whatever the window; sink adds exp(sink_logit[h]) to the softmax's denominator (one, a key of
+// score 0, where sink_logit is null), a key that has no value; out_scale multiplies the result before it
+// is stored; out's rows are ld_out elements apart (a token's heads side by side in each).
 #include "common.h"
 
 #define PLAIN_MAX_ACC 8     // D <= 64 * 8
@@ -48,7 +49,8 @@ __global__ __launch_bounds__(WAVES * 64) void attn_plain_kernel(
     const int* __restrict__ cu_pages, const int* __restrict__ kv_start,
     const int* __restrict__ cu_q, const int* __restrict__ q_start,
     const int* __restrict__ tok_ids, int n_seqs, int T_tokens, int Hq, int Hkv, int D, int P, float scale,
-    int window, const float* __restrict__ head_scale, float softcap, int keep_first, int sink) {
+    int window, const float* __restrict__ head_scale, float softcap, int keep_first, int sink,
+    const float* __restrict__ sink_logit, float out_scale, long long ld_out) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     float* q_s = smem;                                   // [QR][D]
     float* p_s = q_s + QR * D;                           // [WAVES][QR][64]
@@ -256,8 +258,13 @@ __global__ __launch_bounds__(WAVES * 64) void attn_plain_kernel(
                 num = fmaf(acc_s[(w * QR + r) * D + e], ew, num);
                 den = fmaf(ml_s[(w * QR + r) * 2 + 1], ew, den);
             }
-            if (sink) den += expf(-mm);                  // one more key of score 0 that has no value
-            out[((size_t)t_row * Hq + head) * D + e] = from_f<T>(den > 0.f ? num / den : 0.f);
+            if (sink) {                                  // one more key that has no value
+                const float sl = sink_logit != nullptr ? sink_logit[head] : 0.f;
+                const float top = fmaxf(mm, sl), ew = (mm == -INFINITY) ? 0.f : expf(mm - top);
+                num *= ew;
+                den = fmaf(den, ew, expf(sl - top));
+            }
+            out[(size_t)t_row * ld_out + (size_t)head * D + e] = from_f<T>(den > 0.f ? num / den * out_scale : 0.f);
         }
         __syncthreads();                                 // before the next pass writes q_s and the merge buffers
     }
@@ -268,22 +275,24 @@ static void plain_launch(hipStream_t st, const void* q, void* out, const void* k
                          const int* page_table, const int* cu_pages, const int* kv_start, const int* cu_q,
                          const int* q_start, const int* tok_ids, int n_seqs, int T_tokens, int Hq, int Hkv,
                          int D, int P, float scale, int window, const float* head_scale, float softcap,
-                         int keep_first, int sink) {
+                         int keep_first, int sink, const float* sink_logit, float out_scale, long long ld_out) {
     const size_t floats = (size_t)QR * D + (size_t)WAVES * QR * 64 + WAVES * 64 + WAVES * QR * 2 +
                           (size_t)WAVES * QR * D;
     dim3 grid((T_tokens + QR - 1) / QR, Hq), block(WAVES * 64);
     hipLaunchKernelGGL((attn_plain_kernel<T, QR, WAVES>), grid, block, floats * sizeof(float), st, (const T*)q,
                        (T*)out, (const T*)k_pool, (const T*)v_pool, page_table, cu_pages, kv_start, cu_q,
                        q_start, tok_ids, n_seqs, T_tokens, Hq, Hkv, D, P, scale, window, head_scale, softcap,
-                       keep_first, sink);
+                       keep_first, sink, sink_logit, out_scale, ld_out);
 }
 
 extern "C" int ra_attention_plain(const void* q, void* out, const void* k_pool, const void* v_pool,
                                   const int* page_table, const int* cu_pages, const int* kv_start,
                                   const int* cu_q, const int* q_start, const int* tok_ids,
                                   int n_seqs, int T_tokens, int Hq, int Hkv, int D, int P, float scale, int window, int dtype,
-                                  const float* head_scale, float softcap, int keep_first, int sink, void* stream) {
+                                  const float* head_scale, float softcap, int keep_first, int sink,
+                                  const float* sink_logit, float out_scale, long long ld_out, void* stream) {
     if (T_tokens <= 0 || n_seqs <= 0) return RA_OK;
+    if (ld_out < (long long)Hq * D) return RA_ERR_ARG;
     if (D > 64 * PLAIN_MAX_ACC || D <= 0 || Hkv <= 0 || Hq % Hkv != 0 || P <= 0 || Hq > 65535) return RA_ERR_ARG;
     if (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16) return RA_ERR_ARG;
     hipStream_t st = (hipStream_t)stream;
@@ -293,7 +302,7 @@ extern "C" int ra_attention_plain(const void* q, void* out, const void* k_pool, 
 #define PLAIN_GO(T_, QR_, W_)                                                                              \
     plain_launch<T_, QR_, W_>(st, q, out, k_pool, v_pool, page_table, cu_pages, kv_start, cu_q, q_start,   \
                               tok_ids, n_seqs, T_tokens, Hq, Hkv, D, P, scale, window, head_scale, softcap,   \
-                              keep_first, sink)
+                              keep_first, sink, sink_logit, out_scale, ld_out)
     if (dtype == RA_DTYPE_F32) {
         if (single) PLAIN_GO(float, 1, 8); else PLAIN_GO(float, 4, 4);
     } else {

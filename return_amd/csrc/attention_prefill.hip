@@ -52,11 +52,13 @@ typedef uint32_t uint4_t __attribute__((ext_vector_type(4)));
 
 typedef short4_t __attribute__((address_space(3))) * lds_short4_ptr;
 
-// XT: the optional extras. head_scale[h] multiplies the scale of query head h; softcap c turns a score s
+// XT: 1 or 2, the optional extras. head_scale[h] multiplies the scale of query head h; softcap c turns a score s
 // into c tanh(s / c); keys at positions below keep_first stay readable whatever the window (their tiles
-// are walked first, then the tiles from the window's first key on); sink adds one to the softmax's
-// denominator (a key of score 0 that has no value).
-template <int D16, int QG, int KSPLIT, bool XT>
+// are walked first, then the tiles from the window's first key on); sink adds exp(sink_logit[h]) to the softmax's
+// denominator (one, a key of score 0, where sink_logit is null), a key that has no value; out_scale multiplies the
+// result before it is stored; out's rows are ld_out elements apart. With XT 2 the weights go into the product with
+// the values as two bfloat16 halves (16 bits of mantissa) in place of one.
+template <int D16, int QG, int KSPLIT, int XT>
 __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2))) void attn_prefill_kernel(
     const bf16* __restrict__ q, bf16* __restrict__ out, const bf16* __restrict__ k_pool,
     const bf16* __restrict__ v_pool, const int* __restrict__ page_table,
@@ -64,7 +66,8 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
     const int* __restrict__ cu_q, const int* __restrict__ q_start,
     const int* __restrict__ tiles,       // [n_tiles][2]: request number, first row of the tile within it
     int n_tiles, int Hq, int Hkv, int P, float scale, int window,
-    const float* __restrict__ head_scale, float softcap, int keep_first, int sink) {
+    const float* __restrict__ head_scale, float softcap, int keep_first, int sink,
+    const float* __restrict__ sink_logit, float out_scale, long long ld_out) {
     constexpr int D = 16 * D16;
     constexpr int D32 = D / 32;
     constexpr bool TAIL16 = (D % 32) != 0;
@@ -149,7 +152,7 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
     // tile on; with them the tiles below keep_end come first and the walk then jumps over the gap.
     int keep_end = 0, gap = 0, u_first = (first_key / BN) * BN;
     int low_key = first_key;                             // the earliest key that a row of this tile may read
-    if constexpr (XT) {
+    if constexpr (XT != 0) {
         if (keep_first > 0 && window > 0 && first_key > start) {
             low_key = start;
             keep_end = ((min(keep_first, tile_last_pos + 1) + BN - 1) / BN) * BN;
@@ -163,10 +166,10 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
     }
 #define POS_OF(u_) ((u_) + ((u_) >= keep_end ? gap : 0))
 
-    const float score_scale = XT ? scale * (head_scale != nullptr ? head_scale[head] : 1.f) : 1.f;
-    const float inv_cap = (XT && softcap > 0.f) ? 1.0f / softcap : 0.f;
+    const float score_scale = XT != 0 ? scale * (head_scale != nullptr ? head_scale[head] : 1.f) : 1.f;
+    const float inv_cap = (XT != 0 && softcap > 0.f) ? 1.0f / softcap : 0.f;
     // (with the extras the scores are finished before the maximum is taken; else the scale comes in with the exponent)
-    const float scale2 = (XT ? 1.f : scale) * 1.44269504088896340736f;
+    const float scale2 = (XT != 0 ? 1.f : scale) * 1.44269504088896340736f;
     // positions of the first and last row of this wave (wave-uniform, for skipping the mask)
     const int wave_first_pos = pos0 + q_off + wave * QG * 16;
     const int wave_last_pos = wave_first_pos + QG * 16 - 1;
@@ -271,7 +274,7 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
         // a tile that lies wholly below every row of the wave and inside every window needs no mask
         bool need_mask = (c0 + BN - 1 > wave_first_pos) || (c0 < first_key) ||
                          (window > 0 && c0 <= wave_last_pos - window);
-        if constexpr (XT) {
+        if constexpr (XT != 0) {
             // a tile of kept keys only, below every row of the wave, needs none either
             if (keep_first > 0 && c0 >= low_key && c0 + BN <= keep_first && c0 + BN - 1 <= wave_first_pos) need_mask = false;
             // the scores as they enter the softmax: scale and the head's factor, then the soft cap
@@ -291,6 +294,7 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
                     }
         }
         uint4_t pw[QG][BN / 32];                         // P as bf16, in the order the B operand wants
+        [[maybe_unused]] uint4_t pl[QG][BN / 32];        // XT 2: what P lacks in bf16
 #pragma unroll
         for (int qg = 0; qg < QG; ++qg) {
             float s[BN / 16][4];
@@ -302,7 +306,7 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
                     for (int i = 0; i < 4; ++i) {
                         const int kpos = c0 + st * 16 + 4 * g + i;
                         bool ok = kpos >= low_key && kpos <= pos_q[qg];
-                        if constexpr (XT) {
+                        if constexpr (XT != 0) {
                             if (window > 0) ok = ok && (kpos > pos_q[qg] - window || kpos < keep_first);
                         } else {
                             if (window > 0) ok = ok && kpos > pos_q[qg] - window;
@@ -351,6 +355,17 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
             for (int b = 0; b < BN / 32; ++b)
                 pw[qg][b] = uint4_t{pack2(s[2 * b][0], s[2 * b][1]), pack2(s[2 * b][2], s[2 * b][3]),
                                     pack2(s[2 * b + 1][0], s[2 * b + 1][1]), pack2(s[2 * b + 1][2], s[2 * b + 1][3])};
+            if constexpr (XT == 2) {
+#pragma unroll
+                for (int b = 0; b < BN / 32; ++b)
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        const int st = 2 * b + (j >> 1), i = 2 * (j & 1);
+                        const uint32_t hi = pw[qg][b][j];
+                        pl[qg][b][j] = pack2(s[st][i] - __uint_as_float(hi << 16),
+                                             s[st][i + 1] - __uint_as_float(hi & 0xffff0000u));
+                    }
+            }
         }
 
         // ---- O^T += V^T P^T, 32 keys per MFMA; V^T through the transposing LDS read, once for every group
@@ -364,9 +379,13 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
                 const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4_ptr)(vr + 16 * VS + dt * 16));
                 const short8_t both = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
-                for (int qg = 0; qg < QG; ++qg)
+                for (int qg = 0; qg < QG; ++qg) {
                     acc[qg][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
                         __builtin_bit_cast(bf16x8_t, both), __builtin_bit_cast(bf16x8_t, pw[qg][b]), acc[qg][dt], 0, 0, 0);
+                    if constexpr (XT == 2)
+                        acc[qg][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                            __builtin_bit_cast(bf16x8_t, both), __builtin_bit_cast(bf16x8_t, pl[qg][b]), acc[qg][dt], 0, 0, 0);
+                }
             }
         }
         }
@@ -417,11 +436,20 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
 #pragma unroll
     for (int qg = 0; qg < QG; ++qg) {
         if (!q_ok[qg]) continue;
-        if constexpr (XT) {
-            if (sink) l_run[qg] += __builtin_amdgcn_exp2f(-m_run[qg] * scale2);      // the key of score 0 without a value
+        float inv;
+        if constexpr (XT != 0) {
+            float rescale = 1.f;
+            if (sink) {                                  // the key without a value
+                const float sl = sink_logit != nullptr ? sink_logit[head] : 0.f;
+                const float top = fmaxf(m_run[qg], sl);
+                rescale = __builtin_amdgcn_exp2f((m_run[qg] - top) * scale2);
+                l_run[qg] = fmaf(l_run[qg], rescale, __builtin_amdgcn_exp2f((sl - top) * scale2));
+            }
+            inv = l_run[qg] > 0.f ? rescale * out_scale / l_run[qg] : 0.f;
+        } else {
+            inv = l_run[qg] > 0.f ? 1.0f / l_run[qg] : 0.f;
         }
-        const float inv = l_run[qg] > 0.f ? 1.0f / l_run[qg] : 0.f;
-        bf16* op = out + ((size_t)(cu_q[seg] + pos_q[qg] - pos0) * Hq + head) * D;
+        bf16* op = out + (size_t)(cu_q[seg] + pos_q[qg] - pos0) * ld_out + (size_t)head * D;
 #pragma unroll
         for (int dt = 0; dt < D16; ++dt) {
             uint2 w;
@@ -440,18 +468,18 @@ extern "C" int PRE_CAT(ra_pre_part_, PRE_PART)(int D16, int tile_rows, int key_s
                                               const int* cup, const int* kvs, const int* cuq,
                                               const int* qs, const int* tiles, int n_tiles, int Hq,
                                               int Hkv, int P, float scale, int window, const float* head_scale,
-                                              float softcap, int keep_first, int sink) {
-    const bool extras = head_scale != nullptr || softcap > 0.f || keep_first > 0 || sink != 0;
+                                              float softcap, int keep_first, int sink, const float* sink_logit,
+                                              float out_scale, long long ld_out, int fine_weights) {
+    const bool extras = head_scale != nullptr || softcap > 0.f || keep_first > 0 || sink != 0 || out_scale != 1.f;
+#define PRE_ONE(N, QG_, KS_, XT_)                                                                  \
+    hipLaunchKernelGGL((attn_prefill_kernel<N, QG_, KS_, XT_>), grid, dim3(256 * KS_), 0, st, q, out, kp, vp, pt, cup, \
+                       kvs, cuq, qs, tiles, n_tiles, Hq, Hkv, P, scale, window, head_scale, softcap, keep_first, sink, \
+                       sink_logit, out_scale, ld_out)
 #define PRE_LAUNCH(N, QG_, KS_)                                                                    \
     do {                                                                                           \
-        if (extras)                                                                                \
-            hipLaunchKernelGGL((attn_prefill_kernel<N, QG_, KS_, true>), grid, dim3(256 * KS_), 0, st, q, out, kp, vp, pt, \
-                               cup, kvs, cuq, qs, tiles, n_tiles, Hq, Hkv, P, scale, window, head_scale, softcap,     \
-                               keep_first, sink);                                                  \
-        else                                                                                       \
-            hipLaunchKernelGGL((attn_prefill_kernel<N, QG_, KS_, false>), grid, dim3(256 * KS_), 0, st, q, out, kp, vp, pt, \
-                               cup, kvs, cuq, qs, tiles, n_tiles, Hq, Hkv, P, scale, window, head_scale, softcap,     \
-                               keep_first, sink);                                                  \
+        if (fine_weights) PRE_ONE(N, QG_, KS_, 2);                                                 \
+        else if (extras) PRE_ONE(N, QG_, KS_, 1);                                                  \
+        else PRE_ONE(N, QG_, KS_, 0);                                                              \
     } while (0)
 #define PRE_CASE(N)                                                                               \
     case N:                                                                                       \
@@ -470,6 +498,7 @@ extern "C" int PRE_CAT(ra_pre_part_, PRE_PART)(int D16, int tile_rows, int key_s
     }
 #undef PRE_CASE
 #undef PRE_LAUNCH
+#undef PRE_ONE
 }
 #endif  // PRE_PART
 
@@ -477,7 +506,7 @@ extern "C" int PRE_CAT(ra_pre_part_, PRE_PART)(int D16, int tile_rows, int key_s
 #define PRE_PART_ARGS int D16, int tile_rows, int key_split, dim3 grid, hipStream_t st, const bf16* q, bf16* out, const bf16* kp,    \
     const bf16* vp, const int* pt, const int* cup, const int* kvs, const int* cuq, const int* qs,    \
     const int* tiles, int n_tiles, int Hq, int Hkv, int P, float scale, int window, const float* head_scale,   \
-    float softcap, int keep_first, int sink
+    float softcap, int keep_first, int sink, const float* sink_logit, float out_scale, long long ld_out, int fine_weights
 extern "C" int ra_pre_part_0(PRE_PART_ARGS);
 extern "C" int ra_pre_part_1(PRE_PART_ARGS);
 extern "C" int ra_pre_part_2(PRE_PART_ARGS);
@@ -496,8 +525,10 @@ extern "C" int ra_attention_prefill_bf16(const void* q, void* out, const void* k
                                          const int* q_start, const int* tiles, int n_tiles,
                                          int tile_rows, int key_split, int Hq, int Hkv, int D, int P,
                                          float scale, int window, const float* head_scale, float softcap,
-                                         int keep_first, int sink, void* stream) {
+                                         int keep_first, int sink, const float* sink_logit, float out_scale,
+                                         long long ld_out, int fine_weights, void* stream) {
     if (n_tiles <= 0) return RA_OK;
+    if (ld_out < (long long)Hq * D || ld_out % 4 != 0 || ((uintptr_t)out & 7) != 0) return RA_ERR_ARG;
     if (D % 16 != 0 || D < 16 || D > 256 || Hkv <= 0 || Hq % Hkv != 0 || P <= 0 ||
         (long long)n_tiles * Hq > 0x7fffffffLL || (tile_rows != ra_attention_prefill_tile_rows(D) && tile_rows != 64))
         return RA_ERR_ARG;
@@ -513,7 +544,8 @@ extern "C" int ra_attention_prefill_bf16(const void* q, void* out, const void* k
 #define GO(k)                                                                                      \
     rc = ra_pre_part_##k(d16, tile_rows, key_split, grid, st, (const bf16*)q, (bf16*)out, (const bf16*)k_pool,           \
                          (const bf16*)v_pool, page_table, cu_pages, kv_start, cu_q, q_start, tiles, \
-                         n_tiles, Hq, Hkv, P, scale, window, head_scale, softcap, keep_first, sink)
+                         n_tiles, Hq, Hkv, P, scale, window, head_scale, softcap, keep_first, sink, sink_logit,     \
+                         out_scale, ld_out, fine_weights)
     switch ((d16 - 1) / 4) {
         case 0: GO(0); break;
         case 1: GO(1); break;

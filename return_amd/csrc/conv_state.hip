@@ -6,6 +6,9 @@
 //                                                          before the request's first row; b null: no bias)
 //   out_t  = act(y_t)  or  act(x_t + y_t)                 (flags: 1 adds the input, 2 applies SiLU)
 //
+// With an input bias every input is x + in_bias, rounded to the storage type (what a stored x + in_bias would be), in
+// the rows as in the tail; the zeros before the request's first row stay zeros.
+//
 // x: rows of ld_x elements of which C are read (a column slice of a wider projection is fine),
 // out: rows of ld_out elements. Request s brings rows cu_q[s]..cu_q[s+1]-1 and owns tail row
 // slot_ids[s]. All sums in 32-bit; the result and the tail are rounded to the storage type.
@@ -23,7 +26,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void causal_conv_kernel(
     const T* __restrict__ x, long long ld_x, const float* __restrict__ w, T* __restrict__ tail,
     const int* __restrict__ cu_q, const int* __restrict__ slot_ids, T* __restrict__ out, long long ld_out,
-    int C, int taps, int flags, const float* __restrict__ bias) {
+    int C, int taps, int flags, const float* __restrict__ bias, const float* __restrict__ in_bias) {
     const int s = blockIdx.y;
     const int base = cu_q[s];
     const int q_len = cu_q[s + 1] - base;
@@ -36,6 +39,11 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
     T* my_tail = tail + ((size_t)slot_ids[s] * back) * C + c;
 
     const float b0 = bias != nullptr ? bias[c] : 0.f;
+    const float bi = in_bias != nullptr ? in_bias[c] : 0.f;
+    auto input = [&](int li) {
+        const float v = to_f(x[(size_t)(base + li) * ld_x + c]);
+        return in_bias != nullptr ? round_to<T>(v + bi) : v;
+    };
     float wt[CONV_MAX_TAPS], win[CONV_MAX_TAPS], old[CONV_MAX_TAPS];
 #pragma unroll
     for (int j = 0; j < CONV_MAX_TAPS; ++j) {
@@ -43,12 +51,12 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
         win[j] = old[j] = 0.f;
         if (j < back) {
             const int li = first - back + j;                 // the input that far back, among this step's rows or before
-            win[j] = li >= 0 ? to_f(x[(size_t)(base + li) * ld_x + c]) : to_f(my_tail[(size_t)(back + li) * C]);
+            win[j] = li >= 0 ? input(li) : to_f(my_tail[(size_t)(back + li) * C]);
             old[j] = win[j];
         }
     }
     for (int li = first; li < last; ++li) {
-        const float cur = to_f(x[(size_t)(base + li) * ld_x + c]);
+        const float cur = input(li);
         float y = b0;
 #pragma unroll
         for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
@@ -73,7 +81,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
             if (j < back) {
                 const int li = q_len - back + j;
                 float v = 0.f;
-                if (li >= 0) v = to_f(x[(size_t)(base + li) * ld_x + c]);
+                if (li >= 0) v = input(li);
                 else {
 #pragma unroll
                     for (int k = 0; k < CONV_MAX_TAPS - 1; ++k)
@@ -86,7 +94,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
 }
 
 // x [T rows], w fp32 [C, taps], tail [slots, taps-1, C], out [T rows]; max_q_len: the longest request of the step.
-static int causal_conv_run(const void* x, long long ld_x, const float* w, const float* bias, void* tail, const int* cu_q,
+static int causal_conv_run(const void* x, long long ld_x, const float* in_bias, const float* w, const float* bias, void* tail, const int* cu_q,
                            const int* slot_ids, void* out, long long ld_out, int n_seqs, int max_q_len,
                            int C, int taps, int flags, int dtype, void* stream) {
     if (n_seqs <= 0 || max_q_len <= 0) return RA_OK;
@@ -96,24 +104,25 @@ static int causal_conv_run(const void* x, long long ld_x, const float* w, const 
     dim3 grid((max_q_len + CONV_SEG - 1) / CONV_SEG, n_seqs, (C + 255) / 256), block(256);
     if (dtype == RA_DTYPE_F32)
         hipLaunchKernelGGL(causal_conv_kernel<float>, grid, block, 0, (hipStream_t)stream, (const float*)x, ld_x, w,
-                           (float*)tail, cu_q, slot_ids, (float*)out, ld_out, C, taps, flags, bias);
+                           (float*)tail, cu_q, slot_ids, (float*)out, ld_out, C, taps, flags, bias, in_bias);
     else
         hipLaunchKernelGGL(causal_conv_kernel<bf16>, grid, block, 0, (hipStream_t)stream, (const bf16*)x, ld_x, w,
-                           (bf16*)tail, cu_q, slot_ids, (bf16*)out, ld_out, C, taps, flags, bias);
+                           (bf16*)tail, cu_q, slot_ids, (bf16*)out, ld_out, C, taps, flags, bias, in_bias);
     return ra_launch_status();
 }
 
 extern "C" int ra_causal_conv(const void* x, long long ld_x, const float* w, void* tail, const int* cu_q,
                               const int* slot_ids, void* out, long long ld_out, int n_seqs, int max_q_len,
                               int C, int taps, int flags, int dtype, void* stream) {
-    return causal_conv_run(x, ld_x, w, nullptr, tail, cu_q, slot_ids, out, ld_out, n_seqs, max_q_len, C, taps, flags,
+    return causal_conv_run(x, ld_x, nullptr, w, nullptr, tail, cu_q, slot_ids, out, ld_out, n_seqs, max_q_len, C, taps, flags,
                            dtype, stream);
 }
 
-// the same with a bias per channel (fp32 [C]) added to the filter's sum before the activation
-extern "C" int ra_causal_conv_bias(const void* x, long long ld_x, const float* w, const float* bias, void* tail,
+// the same with a bias per channel (fp32 [C]) added to the filter's sum before the activation, and one added to the
+// inputs (each may be null)
+extern "C" int ra_causal_conv_bias(const void* x, long long ld_x, const float* in_bias, const float* w, const float* bias, void* tail,
                                    const int* cu_q, const int* slot_ids, void* out, long long ld_out, int n_seqs,
                                    int max_q_len, int C, int taps, int flags, int dtype, void* stream) {
-    return causal_conv_run(x, ld_x, w, bias, tail, cu_q, slot_ids, out, ld_out, n_seqs, max_q_len, C, taps, flags,
+    return causal_conv_run(x, ld_x, in_bias, w, bias, tail, cu_q, slot_ids, out, ld_out, n_seqs, max_q_len, C, taps, flags,
                            dtype, stream);
 }

@@ -33,6 +33,10 @@
 // per row by the exact routines (delta multiplies what is written, so its relative error counts where it is tiny);
 // delta takes beta's place, the decay fills the row's decays. The read-out goes to a kernel of its own, which adds
 // skip[h] v_t, gates and norms in equal parts of the row.
+//
+// A fourth rule (rule 3, "head"): the delta rule itself (unit vectors, beta, the correction term) with one decay per
+// head and token, g = exp(-exp(A_log[h]) softplus(a_t[h] + dt_bias[h])), formed once per row by the exact routines,
+// and the output gate silu(c).
 #include "common.h"
 
 #define DR_TC_MAX 32      // rows of a chunk; fewer where a head's rows would not fit the LDS
@@ -120,7 +124,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
         // (rule 2: the row's step before its softplus, which the wave that takes the row turns into delta)
         if (tid < nt)
             beta_s[tid] = rule == 2 ? to_f(ag[(size_t)(base + c0 + tid) * ld_ag + h]) + dt_bias[h]
-                          : rule ? 1.f : dr_sigmoid(to_f(b[(size_t)(base + c0 + tid) * ld_b + h]));
+                          : rule == 1 ? 1.f : dr_sigmoid(to_f(b[(size_t)(base + c0 + tid) * ld_b + h]));
+        // (rule 3: the row's step before its softplus waits in the first place of the row's padding)
+        if (rule == 3 && tid < nt) g_s[tid * DP + DPT] = to_f(ag[(size_t)(base + c0 + tid) * ld_ag + h]) + dt_bias[h];
         for (int idx = tid; idx < nt * VB; idx += NT) {
             const int tt = idx / VB, jj = idx - tt * VB;
             v_s[idx] = j0 + jj < V ? to_f(qkv[(size_t)(base + c0 + tt) * ld_qkv + 2 * G * D + h * V + j0 + jj]) : 0.f;
@@ -138,7 +144,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
                     const T* row = qkv + (size_t)(base + c0 + tt) * ld_qkv;
                     qq[x] = to_f(row[kvh * D + i]);
                     kk[x] = to_f(row[G * D + kvh * D + i]);
-                    if (rule != 2)
+                    if (rule < 2)
                         aa[x] = a_sign * (to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h * D + i]) + dt_bias[h * D + i]);
                 }
             }
@@ -150,7 +156,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
                 const int at = tt * DP + (i / DPT) * PS + (i % DPT);
                 k_s[at] = kk[x];
                 q_s[at] = qq[x];
-                g_s[at] = (i < D && rule != 2) ? dr_decay(neg_a, aa[x]) : 1.f;
+                g_s[at] = (i < D && rule < 2) ? dr_decay(neg_a, aa[x]) : 1.f;
             }
         }
         __syncthreads();
@@ -170,12 +176,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
                 sk = fmaf(k_s[at], k_s[at], sk);
                 sq = fmaf(q_s[at], q_s[at], sq);
             }
-            sk = rule ? 1.f : 1.0f / sqrtf(wave_sum(sk) + 1e-6f);
-            sq = rule ? q_scale : q_scale / sqrtf(wave_sum(sq) + 1e-6f);
+            sk = rule == 1 ? 1.f : 1.0f / sqrtf(wave_sum(sk) + 1e-6f);
+            sq = rule == 1 ? q_scale : q_scale / sqrtf(wave_sum(sq) + 1e-6f);
+            const float dec = rule == 3 ? expf(neg_a * dr_softplus_exact(g_s[tt * DP + DPT])) : 1.f;
             for (int i = lane; i < D; i += 64) {
                 const int at = tt * DP + (i / DPT) * PS + (i % DPT);
                 k_s[at] *= sk;
                 q_s[at] *= sq;
+                if (rule == 3) g_s[at] = dec;
             }
         }
         __syncthreads();
@@ -211,7 +219,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
                 a3 = fmaf(st[ii + 3], kreg[ii + 3], a3);
             }
             // (the outer-product rule has no correction term: what is written is the value itself)
-            const float acc = rule ? 0.f : dr_group_sum((a0 + a1) + (a2 + a3), RS);
+            const float acc = (rule == 1 || rule == 2) ? 0.f : dr_group_sum((a0 + a1) + (a2 + a3), RS);
             const float u = beta * (vv - acc);
             float o0 = 0.f, o1 = 0.f, o2 = 0.f, o3 = 0.f;
 #pragma unroll
@@ -303,7 +311,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
         const int nt = min(TC, q_len - c0);
         // the chunk's values and betas (every feeder thread has a share, whether or not its wave has rows)
         auto feed_values = [&]() {
-            float bv = (ft < nt && !rule) ? to_f(b[(size_t)(base + c0 + ft) * ld_b + h]) : 0.f;
+            float bv = (ft < nt && (rule == 0 || rule == 3)) ? to_f(b[(size_t)(base + c0 + ft) * ld_b + h]) : 0.f;
             if (ft < nt && rule == 2) bv = to_f(ag[(size_t)(base + c0 + ft) * ld_ag + h]) + dt_bias[h];
             for (int idx0 = ft; idx0 < nt * VB; idx0 += 4 * DR_FEEDERS) {
                 float vv[4];
@@ -318,7 +326,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                 for (int x = 0; x < 4; ++x)
                     if (idx0 + x * DR_FEEDERS < nt * VB) v_s[idx0 + x * DR_FEEDERS] = vv[x];
             }
-            if (ft < nt) beta_s[ft] = rule == 2 ? dr_softplus_exact(bv) : rule ? 1.f : dr_sigmoid(bv);
+            if (ft < nt) beta_s[ft] = rule == 2 ? dr_softplus_exact(bv) : rule == 1 ? 1.f : dr_sigmoid(bv);
         };
         bool values_done = false;
         constexpr int EPL = (8 * DPT + 63) / 64;            // elements of a row per lane (RS <= 8)
@@ -336,7 +344,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                         const T* row = qkv + (size_t)(base + c0 + tt) * ld_qkv;
                         fq[m][e] = to_f(row[kvh * D + i]);
                         fk[m][e] = to_f(row[G * D + kvh * D + i]);
-                        fa[m][e] = rule == 2 ? to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h]) + dt_bias[h]
+                        fa[m][e] = rule >= 2 ? to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h]) + dt_bias[h]
                                    : a_sign * (to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h * D + i]) + dt_bias[h * D + i]);
                     }
                 }
@@ -355,10 +363,10 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                     sk = fmaf(fk[m][e], fk[m][e], sk);
                     sq = fmaf(fq[m][e], fq[m][e], sq);
                 }
-                sk = rule ? 1.f : 1.0f / sqrtf(dr_wave_sum(sk) + 1e-6f);
-                sq = rule ? q_scale : q_scale / sqrtf(dr_wave_sum(sq) + 1e-6f);
-                // (rule 2: one decay for the whole row; lanes with an element of the row hold its step in fa[m][0])
-                const float row_decay = (rule == 2 && lane < D) ? expf(neg_a * dr_softplus_exact(fa[m][0])) : 1.f;
+                sk = (rule == 1 || rule == 2) ? 1.f : 1.0f / sqrtf(dr_wave_sum(sk) + 1e-6f);
+                sq = (rule == 1 || rule == 2) ? q_scale : q_scale / sqrtf(dr_wave_sum(sq) + 1e-6f);
+                // (rules 2 and 3: one decay for the whole row; lanes with an element of the row hold its step in fa[m][0])
+                const float row_decay = (rule >= 2 && lane < D) ? expf(neg_a * dr_softplus_exact(fa[m][0])) : 1.f;
 #pragma unroll
                 for (int e = 0; e < EPL; ++e) {
                     const int i = lane + 64 * e;
@@ -366,7 +374,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                         const int at = tt * DP + (i / DPT) * PS + (i % DPT);
                         k_s[at] = fk[m][e] * sk;
                         q_s[at] = fq[m][e] * sq;
-                        g_s[at] = i >= D ? 1.f : rule == 2 ? row_decay : dr_decay(neg_a, fa[m][e]);
+                        g_s[at] = i >= D ? 1.f : rule >= 2 ? row_decay : dr_decay(neg_a, fa[m][e]);
                     }
                 }
             }
@@ -431,7 +439,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                     a2 = fmaf(st[ii + 2], k4.z, a2);
                     a3 = fmaf(st[ii + 3], k4.w, a3);
                 }
-                const float acc = rule ? 0.f : dr_group_sum((a0 + a1) + (a2 + a3), RS);
+                const float acc = (rule == 1 || rule == 2) ? 0.f : dr_group_sum((a0 + a1) + (a2 + a3), RS);
                 const float u = beta_s[tt] * (v_s[tt * VB + (live ? jl : 0)] - acc);
                 float o0 = 0.f, o1 = 0.f, o2 = 0.f, o3 = 0.f;
 #pragma unroll
@@ -586,7 +594,7 @@ static int delta_rule_launch(hipStream_t st, int DPT, dim3 grid, dim3 block, siz
 // qkv [T, 2 G D + H V] rows; b: rows whose first H columns are the heads' beta (before the sigmoid); ag [T, H D + H V];
 // S fp32 [slots, H, V, D] (column by column); o_raw fp32 [T, H V] scratch; out [T, H V]; max_q_len: the longest request's rows.
 // (ag: the decay's projection, H D columns of rows ld_ag apart; gate: the output gate's, H V columns of rows ld_gate
-// apart; rule 0: the delta rule, 1: the outer-product rule with decay exponent `rate`, for which b and A_log are null)
+// apart; rule 0: the delta rule, 3: with one decay per head (ag then has H columns), 1: the outer-product rule with decay exponent `rate`, for which b and A_log are null)
 static int delta_rule_run(const void* qkv, long long ld_qkv, const void* b, long long ld_b, const void* ag,
                           long long ld_ag, const void* gate, long long ld_gate, const float* A_log, const float* dt_bias,
                           const float* norm_w, float eps, float* S, const int* cu_q, const int* slot_ids, float* o_raw,
@@ -595,8 +603,8 @@ static int delta_rule_run(const void* qkv, long long ld_qkv, const void* b, long
     if (n_seqs <= 0 || T_tokens <= 0) return RA_OK;
     int RS, DPT, VB;
     if (!delta_rule_plan(D, V, &RS, &DPT, &VB) || H < 1 || G < 1 || H % G || n_seqs > 65535) return RA_ERR_ARG;
-    if (ld_qkv < (long long)2 * G * D + (long long)H * V || (rule == 0 && ld_b < H) ||
-        ld_ag < (rule == 2 ? (long long)H : (long long)H * D) || ld_gate < (long long)H * V)
+    if (ld_qkv < (long long)2 * G * D + (long long)H * V || ((rule == 0 || rule == 3) && ld_b < H) ||
+        ld_ag < (rule >= 2 ? (long long)H : (long long)H * D) || ld_gate < (long long)H * V)
         return RA_ERR_ARG;
     if (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16) return RA_ERR_ARG;
     int TC = delta_rule_chunk(DPT, RS, VB);
@@ -644,10 +652,10 @@ static int delta_rule_run(const void* qkv, long long ld_qkv, const void* b, long
     dim3 ogrid((unsigned)((n_rows + 3) / 4)), oblock(256);
     if (dtype == RA_DTYPE_F32)
         hipLaunchKernelGGL(delta_out_kernel<float>, ogrid, oblock, 0, st, o_raw, (const float*)gate, ld_gate, norm_w,
-                           eps, (float*)out, n_rows, H, V, rule);
+                           eps, (float*)out, n_rows, H, V, rule != 0);
     else
         hipLaunchKernelGGL(delta_out_kernel<bf16>, ogrid, oblock, 0, st, o_raw, (const bf16*)gate, ld_gate, norm_w,
-                           eps, (bf16*)out, n_rows, H, V, rule);
+                           eps, (bf16*)out, n_rows, H, V, rule != 0);
     return ra_launch_status();
 }
 
@@ -660,6 +668,18 @@ extern "C" int ra_delta_rule(const void* qkv, long long ld_qkv, const void* b, l
     const void* gate = (const char*)ag + (size_t)H * D * el;
     return delta_rule_run(qkv, ld_qkv, b, ld_b, ag, ld_ag, gate, ld_ag, A_log, dt_bias, norm_w, eps, S, cu_q, slot_ids,
                           o_raw, out, n_seqs, T_tokens, max_q_len, H, G, D, V, 0, 0.f, dtype, stream);
+}
+
+// The delta rule with one decay per head: a [T, H] the decay's projection before its bias, b [T, H] beta before the
+// sigmoid, gate [T, H V]; out = rmsnorm_V(o) norm_w silu(gate).
+extern "C" int ra_delta_rule_head(const void* qkv, long long ld_qkv, const void* b, long long ld_b, const void* a,
+                                  long long ld_a, const void* gate, long long ld_gate, const float* A_log,
+                                  const float* dt_bias, const float* norm_w, float eps, float* S, const int* cu_q,
+                                  const int* slot_ids, float* o_raw, void* out, int n_seqs, int T_tokens, int max_q_len,
+                                  int H, int G, int D, int V, int dtype, void* stream) {
+    if (A_log == nullptr || dt_bias == nullptr || norm_w == nullptr) return RA_ERR_ARG;
+    return delta_rule_run(qkv, ld_qkv, b, ld_b, a, ld_a, gate, ld_gate, A_log, dt_bias, norm_w, eps, S, cu_q, slot_ids,
+                          o_raw, out, n_seqs, T_tokens, max_q_len, H, G, D, V, 3, 0.f, dtype, stream);
 }
 
 // The outer-product rule: qkv rows [q: H D | k: H D | v: H V]; a [T, H D] the decay's logits before their bias;

@@ -6,7 +6,9 @@
 //                      x2 = h / sqrt(mean(h^2) + eps2) * w2. One workgroup per row, one pass over the row: its
 //                      elements stay in registers between the sum of squares and the two results.
 //   qkv_blend_prepare  one wave per (token, head) over the projection row [q heads | k heads | v heads], all heads
-//                      of D elements: a 32-bit bias per column is added; the first R elements of a q or k head turn by
+//                      of D elements (rows ld_qkv elements apart): a 32-bit bias per column is added (null: none); a
+//                      q or k head is divided by the root mean square of its first Dn elements and weighed (w_q, w_k
+//                      [D], null: no norm; elements from Dn on are zeros); the first R elements of a q or k head turn by
 //                      the token's position, element j with j + R/2; q goes to q_out [T, Hq, D], k to its row of the
 //                      key pool. v: mode 1 writes the first Dv elements of the biased v into `first` (32-bit,
 //                      [T, Hkv, Dv]: a head's true width, which layers of other row widths share) and v into the
@@ -168,7 +170,9 @@ extern "C" int ra_add_rmsnorm_pair(float* h, const void* a, const void* b, const
 
 // ------------------------------------------------------------------ q/k/v preparation with biases and blended values
 template <typename T>
-__global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, int Hq, int Hkv, int D, const float* __restrict__ bias,
+__global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, long long ld_qkv, int Hq, int Hkv, int D,
+                                         const float* __restrict__ bias, const float* __restrict__ w_q,
+                                         const float* __restrict__ w_k, int Dn, float eps,
                                          const int* __restrict__ positions, const float* __restrict__ cos_t,
                                          const float* __restrict__ sin_t, int R, T* __restrict__ q_out,
                                          T* __restrict__ k_pool, T* __restrict__ v_pool, const int* __restrict__ slots,
@@ -180,8 +184,9 @@ __global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, int Hq, int 
     const int heads = Hq + 2 * Hkv;
     const int t = (int)(row / heads);
     const int head = (int)(row % heads);
-    const T* src = qkv + row * D;
-    const float* b = bias + (size_t)head * D;
+    const T* src = qkv + (size_t)t * ld_qkv + (size_t)head * D;
+    const float* b = bias != nullptr ? bias + (size_t)head * D : nullptr;
+    auto value = [&](int c) { return b != nullptr ? to_f(src[c]) + b[c] : to_f(src[c]); };
     if (head >= Hq + Hkv) {
         // a value head: bias, the first layer's values out or blended in, the cache row
         const int kvh = head - Hq - Hkv;
@@ -192,7 +197,7 @@ __global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, int Hq, int 
             if (s >= 0 && s < pool_rows) dst = v_pool + ra_cache_offset(s, kvh, Hkv, P, D);
         }
         for (int c = lane; c < D; c += 64) {
-            float v = to_f(src[c]) + b[c];
+            float v = value(c);
             if (mode == 1 && c < Dv) fr[c] = v;
             else if (mode == 2) v = (1.0f - lambda) * v + (c < Dv ? lambda * fr[c] : 0.f);
             if (dst != nullptr) dst[c] = from_f<T>(v);
@@ -210,22 +215,32 @@ __global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, int Hq, int 
     }
     const int half = R >> 1;
     const int pos = positions[t];
+    const float* wn = head < Hq ? w_q : w_k;
+    float rstd = 1.f;
+    if (wn != nullptr) {
+        float ss = 0.f;
+        for (int c = lane; c < Dn; c += 64) ss = fmaf(value(c), value(c), ss);
+        rstd = 1.0f / sqrtf(wave_sum(ss) / (float)Dn + eps);
+    }
+    auto normed = [&](int c) { return wn != nullptr ? value(c) * rstd * wn[c] : value(c); };
     for (int j = lane; j < half; j += 64) {
-        const float x1 = to_f(src[j]) + b[j], x2 = to_f(src[j + half]) + b[j + half];
+        const float x1 = normed(j), x2 = normed(j + half);
         const float cs = cos_t[(size_t)pos * half + j], sn = sin_t[(size_t)pos * half + j];
         dst[j] = from_f<T>(x1 * cs - x2 * sn);
         dst[j + half] = from_f<T>(x2 * cs + x1 * sn);
     }
-    for (int c = R + lane; c < D; c += 64) dst[c] = from_f<T>(to_f(src[c]) + b[c]);
+    for (int c = R + lane; c < D; c += 64) dst[c] = from_f<T>(normed(c));
 }
 
-extern "C" int ra_qkv_blend_prepare(const void* qkv, int T_tokens, int Hq, int Hkv, int D, const float* bias,
+extern "C" int ra_qkv_blend_prepare(const void* qkv, long long ld_qkv, int T_tokens, int Hq, int Hkv, int D,
+                                    const float* bias, const float* w_q, const float* w_k, int Dn, float eps,
                                     const int* positions, const float* cos_t, const float* sin_t, int R, void* q_out,
                                     void* k_pool, void* v_pool, const int* slots, int P, long long pool_rows,
                                     float* first, int Dv, int mode, float lambda, int dtype, void* stream) {
     if (T_tokens <= 0) return RA_OK;
     if ((k_pool == nullptr) != (v_pool == nullptr) || (k_pool != nullptr && (P <= 0 || slots == nullptr))) return RA_ERR_ARG;
-    if (D < 1 || Hq < 1 || Hkv < 1 || R < 0 || R > D || (R & 1) || bias == nullptr || q_out == nullptr ||
+    if (D < 1 || Hq < 1 || Hkv < 1 || R < 0 || R > D || (R & 1) || q_out == nullptr ||
+        ld_qkv < (long long)(Hq + 2 * Hkv) * D || (w_q == nullptr) != (w_k == nullptr) || Dn < 1 || Dn > D ||
         (R > 0 && (cos_t == nullptr || sin_t == nullptr)) || mode < 0 || mode > 2 ||
         (mode != 0 && (first == nullptr || Dv < 1 || Dv > D)))
         return RA_ERR_ARG;
@@ -233,11 +248,11 @@ extern "C" int ra_qkv_blend_prepare(const void* qkv, int T_tokens, int Hq, int H
     dim3 block(256), grid((unsigned)((n_rows + 3) / 4));
     hipStream_t st = (hipStream_t)stream;
     if (dtype == RA_DTYPE_F32)
-        hipLaunchKernelGGL(qkv_blend_prepare_kernel<float>, grid, block, 0, st, (const float*)qkv, Hq, Hkv, D, bias,
+        hipLaunchKernelGGL(qkv_blend_prepare_kernel<float>, grid, block, 0, st, (const float*)qkv, ld_qkv, Hq, Hkv, D, bias, w_q, w_k, Dn, eps,
                            positions, cos_t, sin_t, R, (float*)q_out, (float*)k_pool, (float*)v_pool, slots, P, pool_rows,
                            first, Dv, mode, lambda, n_rows);
     else if (dtype == RA_DTYPE_BF16)
-        hipLaunchKernelGGL(qkv_blend_prepare_kernel<bf16>, grid, block, 0, st, (const bf16*)qkv, Hq, Hkv, D, bias,
+        hipLaunchKernelGGL(qkv_blend_prepare_kernel<bf16>, grid, block, 0, st, (const bf16*)qkv, ld_qkv, Hq, Hkv, D, bias, w_q, w_k, Dn, eps,
                            positions, cos_t, sin_t, R, (bf16*)q_out, (bf16*)k_pool, (bf16*)v_pool, slots, P, pool_rows,
                            first, Dv, mode, lambda, n_rows);
     else

@@ -63,9 +63,9 @@ def _declare(lib):
         "ra_attention_latent_plain_window": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, I, I, I, P],
         "ra_attention_latent_mfma_window_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P, I, P, I, P],
         "ra_add_rmsnorm_pair": [P, P, P, P, F, P, P, F, P, I, I, I, P],
-        "ra_qkv_blend_prepare": [P, I, I, I, I, P, P, P, P, I, P, P, P, P, I, L, P, I, I, F, I, P],
+        "ra_qkv_blend_prepare": [P, L, I, I, I, I, P, P, P, I, F, P, P, P, I, P, P, P, P, I, L, P, I, I, F, I, P],
         "ra_clamped_mul": [P, L, P, I, I, F, F, I, P],
-        "ra_causal_conv_bias": [P, L, P, P, P, P, P, P, L, I, I, I, I, I, I, P],
+        "ra_causal_conv_bias": [P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, P],
         "ra_scalar_rule": [P, L, P, L, P, L, P, P, P, P, I, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "ra_attention_latent_plain_fits": [I, I],
         "ra_attention_latent_mfma_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P, I, P, P],
@@ -106,20 +106,29 @@ def _declare(lib):
         "ra_gemm_sweep_fits": [I, I],
         "ra_gemm_sweep_workgroups": [I, I],
         "ra_gemm_sweep_norm_bf16": [P, P, P, I, I, I, I, I, I, P, I, I, F, P, P, P, P],
-        "ra_attention_plain": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, F, I, I, P],
+        "ra_attention_plain": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, F, I, I, P, F, L, P],
         "ra_causal_conv": [P, L, P, P, P, P, P, L, I, I, I, I, I, I, P],
         "ra_delta_rule": [P, L, P, L, P, L, P, P, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
+        "ra_delta_rule_head": [P, L, P, L, P, L, P, L, P, P, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
+        "ra_channel_recurrence": [P, P, P, P, P, L, P, P, P, P, P, F, P, L, I, I, I, I, I, I, I, P],
+        "ra_channel_recurrence_chunk": [I],
+        "ra_channel_recurrence_mfma": [I, I, I],
+        "ra_layer_norm_add": [P, P, P, F, P, I, I, I, P],
+        "ra_layer_norm_rows": [P, P, F, P, P, I, I, I, P],
+        "ra_stream_rows": [P, P, L, I, P],
+        "ra_softcap": [P, F, L, P],
         "ra_delta_rule_fits": [I, I],
         "ra_token_side": [P, P, P, P, L, I, P, P, P, F, I, I, I, I, P],
         "ra_relu_sq": [P, L, I, P],
         "ra_add_bias": [P, P, L, I, I, P],
         "ra_qk_prepare": [P, I, I, I, I, P, P, P, P, I, P, P, P, P, I, L, I, P],
         "ra_attention_decode_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, I, I, I, P],
-        "ra_attention_decode_extras_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, I, I, I, P, F, I, I, P],
+        "ra_attention_decode_extras_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, I, I, I, P, F, I, I, P, F, L, I,
+                                            P],
         "ra_attention_decode_fused_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, I, I, P, P, F, P, P, I, P],
         "ra_attention_decode_static_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, I, I, I, I, P],
         "ra_attention_decode_merge_waves": [I],
-        "ra_attention_prefill_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, F, I, I, P],
+        "ra_attention_prefill_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, F, I, I, P, F, L, I, P],
         "ra_attention_prefill_tile_rows": [I],
         "ra_sample": [P, I, I, P, P, P, P, P, P],
         "ra_sample_traced": [P, I, I, P, P, P, P, P, P, P],
@@ -598,22 +607,34 @@ class HipOps:
         return out
 
     def qkv_blend_prepare(self, qkv, n_q, n_kv, D, bias, positions, cos, sin, rotary_dim, q_out, k_pool, v_pool,
-                          slot_mapping, first=None, blend=None):
-        """q/k/v preparation of an attention with biases: rows of qkv are [n_q | n_kv | n_kv] heads of D; the fp32 bias
-        (one entry per column) is added, the first rotary_dim elements of every q and k head turn by the position
+                          slot_mapping, first=None, blend=None, w_q=None, w_k=None, norm_dim=None, eps=0.0):
+        """q/k/v preparation of an attention: rows of qkv (possibly a column slice of wider rows) are [n_q | n_kv | n_kv]
+        heads of D; the fp32 bias (one entry per column; None: none) is added, with w_q and w_k (fp32 [D]) every q and k
+        head is divided by the root mean square of its first norm_dim (None: all) elements and weighed (what a head has
+        beyond norm_dim must be zeros), the first rotary_dim elements of every q and k head turn by the position
         (element i with i + rotary_dim / 2), q goes to q_out [T, n_q, D], k and v to the pools' rows that slot_mapping
         names (pools None: nothing is written). first (fp32 [T, n_kv Dv], Dv <= D a head's true value width) with
         blend None: receives the first Dv elements of every head of the biased v; with blend lambda:
         v <- (1 - lambda) v + lambda first before it is stored."""
-        self._want(qkv, "qkv", dims=2)
+        ld_qkv = self._want_rows(qkv, "qkv")
         self._want(q_out, "q", qkv.dtype, 3)
         self._want(positions, "positions", torch.int32, 1)
-        self._want(bias, "bias", torch.float32, 1)
         T, R = qkv.shape[0], int(rotary_dim)
-        if qkv.shape[1] != (n_q + 2 * n_kv) * D or tuple(q_out.shape) != (T, n_q, D) or positions.shape[0] != T \
-                or bias.shape[0] != qkv.shape[1]:
-            raise KernelError(f"qkv_blend_prepare: qkv {tuple(qkv.shape)}, q {tuple(q_out.shape)}, bias {tuple(bias.shape)}, "
-                              f"{T} tokens")
+        if qkv.shape[1] != (n_q + 2 * n_kv) * D or tuple(q_out.shape) != (T, n_q, D) or positions.shape[0] != T:
+            raise KernelError(f"qkv_blend_prepare: qkv {tuple(qkv.shape)}, q {tuple(q_out.shape)}, {T} tokens")
+        if bias is not None:
+            self._want(bias, "bias", torch.float32, 1)
+            if bias.shape[0] != qkv.shape[1]:
+                raise KernelError(f"qkv_blend_prepare: bias {tuple(bias.shape)} for {qkv.shape[1]} columns")
+        if (w_q is None) != (w_k is None):
+            raise KernelError("qkv_blend_prepare: q and k norm weights come together")
+        norm_dim = D if norm_dim is None else int(norm_dim)
+        if not 1 <= norm_dim <= D:
+            raise KernelError(f"qkv_blend_prepare: norm over {norm_dim} elements of heads of {D}")
+        for w in (w_q, w_k) if w_q is not None else ():
+            self._want(w, "head norm weight", torch.float32, 1)
+            if w.shape[0] != D:
+                raise KernelError(f"qkv_blend_prepare: norm weight {tuple(w.shape)} for head size {D}")
         if R:
             self._want(cos, "cos table", torch.float32, 2)
             self._want(sin, "sin table", torch.float32, 2)
@@ -636,15 +657,17 @@ class HipOps:
             pool_rows = self._pool_rows(k_pool, v_pool, n_kv, D, qkv.dtype)
             P = k_pool.shape[2]
         self._check(self.lib.ra_qkv_blend_prepare(
-            _ptr(qkv), T, n_q, n_kv, D, _ptr(bias), _ptr(positions), _ptr(cos) if R else None, _ptr(sin) if R else None,
+            _ptr(qkv), ld_qkv, T, n_q, n_kv, D, _ptr(bias), _ptr(w_q), _ptr(w_k), norm_dim, float(eps), _ptr(positions),
+            _ptr(cos) if R else None, _ptr(sin) if R else None,
             R, _ptr(q_out), _ptr(k_pool), _ptr(v_pool), _ptr(slot_mapping) if k_pool is not None else None, P, pool_rows,
             _ptr(first), Dv, mode, float(blend or 0.0), _code(qkv.dtype), self._stream()), "qkv_blend_prepare")
 
-    def causal_conv(self, x, w, tail, step, out, add_input=False, silu=False, bias=None):
+    def causal_conv(self, x, w, tail, step, out, add_input=False, silu=False, bias=None, in_bias=None):
         """out = act(conv(x)) or act(x + conv(x)): a causal convolution over time on each channel, the last
         taps-1 inputs of every request kept in tail [slots, taps-1, C] between steps (rows by the step's
         slot_ids). x: [T, C], possibly a column slice of wider rows; w: fp32 [C, taps], last column the
-        current row's; out: [T, C] rows, not x."""
+        current row's; out: [T, C] rows, not x. bias (fp32 [C]): added to the filter's sum; in_bias (fp32 [C]): added to
+        every input first, rounded to x's type (the zeros before a request's start stay zeros)."""
         ld_x = self._want_rows(x, "conv input")
         ld_out = self._want_rows(out, "conv output", x.dtype)
         self._want(w, "conv weight", torch.float32, 2)
@@ -660,12 +683,14 @@ class HipOps:
             raise KernelError("causal_conv: a request's slot lies beyond the tail's rows")
         if out.data_ptr() == x.data_ptr():
             raise KernelError("causal_conv: the output must not be the input")
-        if bias is not None:
-            self._want(bias, "conv bias", torch.float32, 1)
-            if bias.shape[0] != C:
-                raise KernelError(f"causal_conv: bias {tuple(bias.shape)} for {C} channels")
+        if bias is not None or in_bias is not None:
+            for b in (bias, in_bias):
+                if b is not None:
+                    self._want(b, "conv bias", torch.float32, 1)
+                    if b.shape[0] != C:
+                        raise KernelError(f"causal_conv: bias {tuple(b.shape)} for {C} channels")
             self._check(self.lib.ra_causal_conv_bias(
-                _ptr(x), ld_x, _ptr(w), _ptr(bias), _ptr(tail), _ptr(step.cu_q), _ptr(step.slot_ids), _ptr(out), ld_out,
+                _ptr(x), ld_x, _ptr(in_bias), _ptr(w), _ptr(bias), _ptr(tail), _ptr(step.cu_q), _ptr(step.slot_ids), _ptr(out), ld_out,
                 step.n_seqs, step.max_q_len, C, taps, (1 if add_input else 0) | (2 if silu else 0), _code(x.dtype),
                 self._stream()), "causal_conv")
             return out
@@ -710,6 +735,124 @@ class HipOps:
             max(1, int(step.max_q_len)), H, G, D, V,
             _code(qkv.dtype), self._stream()), "delta_rule")
         return out
+
+    def delta_rule_head(self, qkv, beta, a, gate, a_log, dt_bias, norm_w, eps, state, step, out, H, G, D, V):
+        """The gated delta rule with one decay per head and token, g = exp(-exp(a_log) softplus(a + dt_bias)), and what
+        surrounds it in 32-bit (unit q and k, q times D^-1/2, sigmoid of beta); out = rmsnorm_V(o) * norm_w * silu(gate).
+        qkv: [T, 2 G D + H V] after the short convolution; beta, a: [T, H]; gate: [T, H V]; each may be a column slice of
+        wider rows. state: fp32 [slots, H, V, D] (S column by column), updated in place; out: [T, H V]."""
+        ld_qkv = self._want_rows(qkv, "delta-rule q/k/v")
+        ld_b = self._want_rows(beta, "delta-rule beta", qkv.dtype)
+        ld_a = self._want_rows(a, "delta-rule decay projection", qkv.dtype)
+        ld_g = self._want_rows(gate, "output gate", qkv.dtype)
+        self._want(out, "delta-rule output", qkv.dtype, 2)
+        self._want(state, "delta-rule state", torch.float32, 4)
+        T = qkv.shape[0]
+        for t, name, shape in ((a_log, "A_log", (H,)), (dt_bias, "dt_bias", (H,)), (norm_w, "norm weight", (V,))):
+            self._want(t, name, torch.float32)
+            if tuple(t.shape) != shape:
+                raise KernelError(f"delta_rule_head: {name} is {tuple(t.shape)}, wanted {shape}")
+        if qkv.shape[1] != 2 * G * D + H * V or tuple(out.shape) != (T, H * V) or tuple(beta.shape) != (T, H) \
+                or tuple(a.shape) != (T, H) or tuple(gate.shape) != (T, H * V) or T != step.n_tokens \
+                or tuple(state.shape[1:]) != (H, V, D) or H % G:
+            raise KernelError(f"delta_rule_head: qkv {tuple(qkv.shape)}, beta {tuple(beta.shape)}, a {tuple(a.shape)}, "
+                              f"gate {tuple(gate.shape)}, out {tuple(out.shape)}, state {tuple(state.shape)}, {H} heads over "
+                              f"{G} of {D} x {V}, step of {step.n_tokens}")
+        if max(step.slot_ids_host, default=0) >= state.shape[0]:
+            raise KernelError("delta_rule_head: a request's slot lies beyond the state's rows")
+        if not self.delta_rule_fits(D, V):
+            raise KernelError(f"delta_rule_head: heads of {D} x {V} are beyond the kernel")
+        o_raw = torch.empty(T, H * V, dtype=torch.float32, device=self.device)
+        self._check(self.lib.ra_delta_rule_head(
+            _ptr(qkv), ld_qkv, _ptr(beta), ld_b, _ptr(a), ld_a, _ptr(gate), ld_g, _ptr(a_log), _ptr(dt_bias), _ptr(norm_w),
+            float(eps), _ptr(state), _ptr(step.cu_q), _ptr(step.slot_ids), _ptr(o_raw), _ptr(out), step.n_seqs, T,
+            max(1, int(step.max_q_len)), H, G, D, V, _code(qkv.dtype), self._stream()), "delta_rule_head")
+        return out
+
+    def channel_recurrence(self, u, w_gates, gate_bias, rate, y, y_bias, state, step, out, out_scale=1.0):
+        """A gated linear recurrence per channel over the step's rows: r, i = sigmoid(W u + bias) with a matrix per block
+        of neighbouring channels, a = exp(rate r), S <- a S + sqrt(1 - a^2) i u, out = S gelu_tanh(y + y_bias) * out_scale,
+        all but u, y and out in 32-bit. u: [T, width] contiguous; w_gates: [blocks, 2, width / blocks, width / blocks]
+        (gate r first; rows are outputs); gate_bias: fp32 [2, width]; rate, y_bias: fp32 [width]; y: [T, width], possibly a
+        column slice; state: fp32 [slots, width], updated in place; out: [T, >= width] rows, possibly a column slice (the
+        columns beyond width become zeros)."""
+        self._want(u, "recurrence input", dims=2)
+        self._want(w_gates, "gate weights", u.dtype, 4)
+        ld_y = self._want_rows(y, "output branch", u.dtype)
+        ld_out = self._want_rows(out, "recurrence output", u.dtype)
+        self._want(state, "recurrence state", torch.float32, 2)
+        T, width = u.shape
+        blocks = w_gates.shape[0]
+        for t, name, shape in ((gate_bias, "gate bias", (2, width)), (rate, "rate", (width,)), (y_bias, "output bias", (width,))):
+            self._want(t, name, torch.float32)
+            if tuple(t.shape) != shape:
+                raise KernelError(f"channel_recurrence: {name} is {tuple(t.shape)}, wanted {shape}")
+        bw = width // blocks
+        if width % blocks or tuple(w_gates.shape) != (blocks, 2, bw, bw) or tuple(y.shape) != (T, width) \
+                or out.shape[0] != T or out.shape[1] < width or state.shape[1] != width or T != step.n_tokens:
+            raise KernelError(f"channel_recurrence: u {tuple(u.shape)}, gates {tuple(w_gates.shape)}, y {tuple(y.shape)}, "
+                              f"out {tuple(out.shape)}, state {tuple(state.shape)}, step of {step.n_tokens}")
+        if max(step.slot_ids_host, default=0) >= state.shape[0]:
+            raise KernelError("channel_recurrence: a request's slot lies beyond the state's rows")
+        longest = max(1, int(step.max_q_len))
+        # (decays and inputs of every row, and the summaries of the chunks of long requests)
+        floats = 2 * T * width
+        chunk = self.lib.ra_channel_recurrence_chunk(longest)
+        if longest > chunk:
+            floats += 2 * (T // chunk + step.n_seqs + 1) * width
+        scratch = torch.empty(floats, dtype=torch.float32, device=self.device)
+        self._check(self.lib.ra_channel_recurrence(
+            _ptr(u), _ptr(w_gates), _ptr(gate_bias), _ptr(rate), _ptr(y), ld_y, _ptr(y_bias), _ptr(state), _ptr(step.cu_q),
+            _ptr(step.slot_ids), _ptr(scratch), float(out_scale), _ptr(out), ld_out, out.shape[1], step.n_seqs, T, longest,
+            width, blocks, _code(u.dtype), self._stream()), "channel_recurrence")
+        return out
+
+    # ------------------------------------------------------------------ layer norm behind a sublayer
+    def layer_norm_add(self, h, y, weight, eps, out=None):
+        """h (fp32 [T, H]) += (y - mean) / sqrt(variance + eps) * weight, row by row, in 32-bit; out (None: not wanted)
+        receives the new rows of h in y's type."""
+        self._want(h, "residual stream", torch.float32, 2)
+        self._want(y, "sublayer output", dims=2)
+        self._want(weight, "norm weight", torch.float32, 1)
+        T, H = h.shape
+        if tuple(y.shape) != (T, H) or weight.shape[0] != H:
+            raise KernelError(f"layer_norm_add: h {tuple(h.shape)}, y {tuple(y.shape)}, weight {tuple(weight.shape)}")
+        if out is not None:
+            self._want(out, "stream rows", y.dtype, 2)
+            if tuple(out.shape) != (T, H):
+                raise KernelError(f"layer_norm_add: rows {tuple(out.shape)} for a stream {tuple(h.shape)}")
+        self._check(self.lib.ra_layer_norm_add(_ptr(h), _ptr(y), _ptr(weight), float(eps), _ptr(out), T, H, _code(y.dtype),
+                                               self._stream()), "layer_norm_add")
+
+    def layer_norm(self, h, weight, eps, out, rows=None):
+        """out[i] = (h[r] - mean) / sqrt(variance + eps) * weight with r = rows[i] (int32; None: r = i)."""
+        self._want(h, "residual stream", torch.float32, 2)
+        self._want(weight, "norm weight", torch.float32, 1)
+        self._want(out, "norm output", dims=2)
+        M = h.shape[0]
+        if rows is not None:
+            self._want(rows, "row list", torch.int32, 1)
+            M = rows.shape[0]
+        if weight.shape[0] != h.shape[1] or tuple(out.shape) != (M, h.shape[1]):
+            raise KernelError(f"layer_norm: h {tuple(h.shape)}, weight {tuple(weight.shape)}, out {tuple(out.shape)}")
+        self._check(self.lib.ra_layer_norm_rows(_ptr(h), _ptr(weight), float(eps), _ptr(out), _ptr(rows), M, h.shape[1],
+                                                _code(out.dtype), self._stream()), "layer_norm")
+
+    def stream_rows(self, h, out):
+        """out = the rows of h (fp32) in out's type."""
+        self._want(h, "residual stream", torch.float32, 2)
+        self._want(out, "stream rows", dims=2)
+        if out.shape != h.shape:
+            raise KernelError(f"stream_rows: h {tuple(h.shape)}, out {tuple(out.shape)}")
+        self._check(self.lib.ra_stream_rows(_ptr(h), _ptr(out), h.numel(), _code(out.dtype), self._stream()), "stream_rows")
+
+    def softcap(self, z, cap):
+        """z <- cap * tanh(z / cap) in place (fp32)."""
+        self._want(z, "logits", torch.float32)
+        if not float(cap) > 0:
+            raise KernelError(f"softcap: {cap} must be positive")
+        self._check(self.lib.ra_softcap(_ptr(z), float(cap), z.numel(), self._stream()), "softcap")
+        return z
 
     def outer_rule(self, qkv, a, gate, decay_bias, tau, norm_w, eps, state, step, out, H, D, V):
         """The gated outer-product memory of a linear attention over the step's rows: S <- diag(alpha) S + k v^T,
@@ -1252,13 +1395,19 @@ class HipOps:
         return None
 
     def attention(self, q, out, k_pool, v_pool, step, group, scale, window=0, head_scale=None, softcap=0.0,
-                  keep_first=0, sink=False):
+                  keep_first=0, sink=False, sink_logit=None, out_scale=1.0, fine_weights=False):
         """Attention of the step's queries over the paged cache. Optional: head_scale (fp32, one factor per query
         head on the scale), softcap c (score -> c tanh(score / c)), keep_first n (keys at positions below n
-        stay visible whatever the window), sink (one more key of score 0 without a value in the softmax)."""
+        stay visible whatever the window), sink (one more key of score 0 without a value in the softmax),
+        sink_logit (fp32, one per query head: that key's score, neither scaled nor capped), out_scale (a factor on the
+        result), fine_weights (bfloat16: the weights enter the product with the values with 16 bits of mantissa in
+        place of 8). out: [T, n_q, D], tokens possibly further apart than n_q D (columns of wider rows)."""
         self._want(q, "q", dims=3)
-        self._want(out, "attention output", q.dtype, 3)
         T, n_q, D = q.shape
+        if out.device != self.device or out.dtype != q.dtype or out.dim() != 3 or (D > 1 and out.stride(2) != 1) or \
+                (n_q > 1 and out.stride(1) != D) or (T > 1 and out.stride(0) < n_q * D):
+            raise KernelError(f"attention: output {tuple(out.shape)} with strides {out.stride()} of {out.dtype} on {out.device}")
+        ld_out = out.stride(0) if T > 1 else max(n_q * D, out.stride(0))
         g = step.groups[group]
         n_kv = k_pool.shape[1]
         self._pool_rows(k_pool, v_pool, n_kv, D, q.dtype)
@@ -1275,7 +1424,17 @@ class HipOps:
             self._want(head_scale, "head scale", torch.float32, 1)
             if head_scale.shape[0] != n_q:
                 raise KernelError(f"attention: head scale {tuple(head_scale.shape)} for {n_q} heads")
-        extras = head_scale is not None or softcap > 0.0 or keep_first > 0 or sink
+        out_scale = float(out_scale)
+        if sink_logit is not None:
+            self._want(sink_logit, "sink logits", torch.float32, 1)
+            if sink_logit.shape[0] != n_q:
+                raise KernelError(f"attention: sink logits {tuple(sink_logit.shape)} for {n_q} heads")
+            sink = True
+        fine_weights = bool(fine_weights)
+        if q.dtype == torch.bfloat16 and (ld_out % 4 or out.data_ptr() % 8):
+            raise KernelError(f"attention: output rows {ld_out} elements apart, or not aligned to four elements")
+        extras = head_scale is not None or softcap > 0.0 or keep_first > 0 or sink or out_scale != 1.0 or fine_weights \
+            or ld_out != n_q * D
         fast_decode = q.dtype == torch.bfloat16 and step.n_decode > 0 and D % 16 == 0 and D <= 256
         fast_prefill = q.dtype == torch.bfloat16 and bool(step.prefill_tiles) and D % 16 == 0 and D <= 256 and \
             (fast_decode or step.n_decode == 0)
@@ -1293,8 +1452,8 @@ class HipOps:
                 self._check(self.lib.ra_attention_decode_extras_bf16(
                     _ptr(q), _ptr(out), _ptr(part_acc), _ptr(part_ml), _ptr(k_pool), _ptr(v_pool), *tabs,
                     _ptr(step.decode_segs), nd, n_q, n_kv, D, P, float(scale), window, S, max_splits,
-                    1 if merge else 0, _ptr(head_scale), softcap, keep_first, 1 if sink else 0, self._stream()),
-                    "attention_decode_extras_bf16")
+                    1 if merge else 0, _ptr(head_scale), softcap, keep_first, 1 if sink else 0, _ptr(sink_logit), out_scale,
+                    ld_out, 1 if fine_weights else 0, self._stream()), "attention_decode_extras_bf16")
                 return
             self._check(self.lib.ra_attention_decode_bf16(
                 _ptr(q), _ptr(out), _ptr(part_acc), _ptr(part_ml), _ptr(k_pool), _ptr(v_pool), *tabs,
@@ -1319,13 +1478,14 @@ class HipOps:
             self._check(self.lib.ra_attention_prefill_bf16(
                 _ptr(q), _ptr(out), _ptr(k_pool), _ptr(v_pool), *tabs, _ptr(tiles), tiles.shape[0], rows,
                 split, n_q, n_kv, D, P, float(scale), window, _ptr(head_scale), softcap, keep_first,
-                1 if sink else 0, self._stream()), "attention_prefill_bf16")
+                1 if sink else 0, _ptr(sink_logit), out_scale, ld_out, 1 if fine_weights else 0, self._stream()),
+                "attention_prefill_bf16")
 
         def plain_part(toks, n_tok):
             self._check(self.lib.ra_attention_plain(
                 _ptr(q), _ptr(out), _ptr(k_pool), _ptr(v_pool), *tabs, _ptr(toks), step.n_seqs, n_tok,
                 n_q, n_kv, D, P, float(scale), window, _code(q.dtype), _ptr(head_scale), softcap, keep_first,
-                1 if sink else 0, self._stream()), "attention_plain")
+                1 if sink else 0, _ptr(sink_logit), out_scale, ld_out, self._stream()), "attention_plain")
 
         if fast_decode and fast_prefill and step.n_prefill_tokens > 0:
             # A step of prompt portions beside decoded tokens: the two kernels work on different rows of q and

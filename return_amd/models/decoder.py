@@ -12,7 +12,7 @@ import torch
 
 from ..parts.block import BLOCKS
 from ..parts.registry import part_class
-from ..parts.runtime import Normed, unscaled
+from ..parts.runtime import Normed, StreamRows, unscaled
 from ..parts.spec import ModelSpec
 
 
@@ -120,6 +120,8 @@ class Decoder:
             results[1].copy_(h)
             h = results[1]
         for i, call in enumerate(self.schedule):
+            if isinstance(pending, StreamRows) and (call.pass_input is not None or call.add_input or results is not None):
+                pending = None                            # the stream changes before the call: its rows as they were are of no use
             if call.pass_input is not None:
                 h, pending = self.pass_input.forward(h, pending, h_in, call.pass_input)
             if call.add_input:

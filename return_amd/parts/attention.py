@@ -170,21 +170,28 @@ register_part("mixer", "attention", PagedAttention)
 
 
 class BlendAttention:
-    """Grouped-query attention with biases on q, k and v, values of a width of their own, and values that may be
-    blended with those of an earlier layer.
+    """Grouped-query attention with values of a width of their own and, each by parameter, biases on q, k and v, norms
+    on queries and keys, values blended with those of an earlier layer, and a learned sink per head.
 
         q = W_q x + b_q (Hq heads of D),  k = W_k x + b_k (Hkv heads of D),  v = W_v x + b_v (Hkv heads of Dv)
         the first `rotary_dim` elements of every head of q and k turn by the position (the model's position part)
         v <- (1 - lambda) v + lambda v_first     in every layer that blends but the first such layer, whose v is
                                                  v_first for the same token; lambda is a stored number (role "blend")
         score = q . k * scale over the keys j with 0 <= i - j < window (None: every j <= i), softmax, W_o.
+    With bias False there are no biases. With qk_norm_eps every head of q and k is divided by its root mean square
+    (that eps inside the root) and weighed (roles q_norm, k_norm, [D] for all heads) before it turns. With sink the
+    softmax's denominator also holds exp(sink[h]) (role sink, [Hq]): a key that has no value and is not scaled. With
+    fine_weights the softmax's weights enter the product with the values with 16 bits of mantissa in bfloat16.
     The blended v is what the cache keeps. The biases are added, the rotation is done and the values are blended in
     32-bit by one kernel that also writes the cache rows. The cache rows of keys and values have one width, the
     larger of D and Dv (in bfloat16 a multiple of 16, so that the matrix-core kernels take it): the stacked weight
     of the first product and the output projection are filled up with zero rows and columns when the part is built,
     so a padded element is an exact zero everywhere and the attention kernels of the other designs serve unchanged.
+    The part can also be one side of a mixer of several (parts/side_by_side.py): with params inner it keeps no products
+    of its own; take_products() gives up the stacked first weight and the output projection, and run() does what lies
+    between the two, on a column slice of wider rows on either side.
     Parameters: hidden_size, num_heads, num_kv_heads, head_dim, value_dim (None: head_dim), scale (None: D^-1/2),
-    window, position, value_rows (name of the model's shared part through which the first blending layer hands its
+    bias (True unless given), qk_norm_eps, sink, fine_weights, inner, window, position, value_rows (name of the model's shared part through which the first blending layer hands its
     values on; None: this layer does not blend), first_of_blend (this layer is that first one).
     """
 
@@ -192,10 +199,15 @@ class BlendAttention:
     def tensor_shapes(params):
         H, Hq, Hkv, D = params["hidden_size"], params["num_heads"], params["num_kv_heads"], params["head_dim"]
         Dv = params.get("value_dim") or D
-        shapes = {"q_proj": (Hq * D, H), "q_bias": (Hq * D,), "k_proj": (Hkv * D, H), "k_bias": (Hkv * D,),
-                  "v_proj": (Hkv * Dv, H), "v_bias": (Hkv * Dv,), "o_proj": (H, Hq * Dv)}
+        shapes = {"q_proj": (Hq * D, H), "k_proj": (Hkv * D, H), "v_proj": (Hkv * Dv, H), "o_proj": (H, Hq * Dv)}
+        if params.get("bias", True):
+            shapes.update({"q_bias": (Hq * D,), "k_bias": (Hkv * D,), "v_bias": (Hkv * Dv,)})
         if params.get("value_rows"):
             shapes["blend"] = ()
+        if params.get("qk_norm_eps") is not None:
+            shapes.update({"q_norm": (D,), "k_norm": (D,)})
+        if params.get("sink"):
+            shapes["sink"] = (Hq,)
         return shapes
 
     @staticmethod
@@ -204,7 +216,9 @@ class BlendAttention:
             return lambda shape, gen: 0.2 + 0.6 * torch.rand(tuple(shape), generator=gen, dtype=torch.float32, device=gen.device)
         if role.endswith("_bias"):
             return lambda shape, gen: 0.1 * torch.randn(*shape, generator=gen, dtype=torch.float32, device=gen.device)
-        return "matrix"
+        if role == "sink":
+            return lambda shape, gen: torch.randn(*shape, generator=gen, dtype=torch.float32, device=gen.device)
+        return "norm" if role in ("q_norm", "k_norm") else "matrix"
 
     def __init__(self, params, tensors, rt, shared=None):
         self.rt = rt
@@ -226,7 +240,7 @@ class BlendAttention:
             raise KeyError(f"attention names position encoding {params['position']!r}, which the model lacks")
         if self.position is not None and (not hasattr(self.position, "tables") or
                                           getattr(self.position, "pairing", "half") != "half"):
-            raise ValueError("attention with biases rotates by tables, element i with i + rotary_dim / 2")
+            raise ValueError("attention with values of their own width rotates by tables, element i with i + rotary_dim / 2")
         self.value_rows = (shared or {}).get(params["value_rows"]) if params.get("value_rows") else None
         if params.get("value_rows") and self.value_rows is None:
             raise KeyError(f"attention names shared rows {params['value_rows']!r}, which the model lacks")
@@ -241,15 +255,35 @@ class BlendAttention:
             return out.reshape((heads * self.dp,) + tuple(t.shape[1:]))
 
         rows = [padded("q_proj", self.n_q, self.d), padded("k_proj", self.n_kv, self.d), padded("v_proj", self.n_kv, self.dv)]
-        self.w_qkv = rt.product(rt.matrix(torch.cat(rows, dim=0).contiguous()))
-        self.bias = rt.vector32(torch.cat([padded("q_bias", self.n_q, self.d), padded("k_bias", self.n_kv, self.d),
-                                           padded("v_bias", self.n_kv, self.dv)]))
+        self.inner = bool(params.get("inner"))
+        note = (lambda w, **kw: w) if self.inner else rt.product
+        self.w_qkv = note(rt.matrix(torch.cat(rows, dim=0).contiguous()))
+        self.bias = None
+        if params.get("bias", True):
+            self.bias = rt.vector32(torch.cat([padded("q_bias", self.n_q, self.d), padded("k_bias", self.n_kv, self.d),
+                                               padded("v_bias", self.n_kv, self.dv)]))
+        self.norms = {}
+        if params.get("qk_norm_eps") is not None:
+            self.norms = dict(w_q=rt.vector32(padded("q_norm", 1, self.d)), w_k=rt.vector32(padded("k_norm", 1, self.d)),
+                              norm_dim=self.d, eps=float(params["qk_norm_eps"]))
+        self.extras = {}
+        if params.get("sink"):
+            self.extras["sink_logit"] = rt.vector32(tensors["sink"])
+        if params.get("fine_weights"):
+            self.extras["fine_weights"] = True
         o = tensors["o_proj"].reshape(W, self.n_q, self.dv)
         o_pad = torch.zeros(W, self.n_q, self.dp, dtype=o.dtype, device=o.device)
         o_pad[:, :, :self.dv] = o
-        self.w_o = rt.product(rt.matrix(o_pad.reshape(W, self.n_q * self.dp).contiguous()), residual=True)
-        self.first_product = (self.w_qkv, False)          # (see PagedAttention)
-        self.last_product = self.w_o
+        self.w_o = note(rt.matrix(o_pad.reshape(W, self.n_q * self.dp).contiguous()), **({} if self.inner else {"residual": True}))
+        self.in_width, self.out_width = (self.n_q + 2 * self.n_kv) * self.dp, self.n_q * self.dp
+        if not self.inner:
+            self.first_product = (self.w_qkv, False)      # (see PagedAttention)
+            self.last_product = self.w_o
+
+    def take_products(self):
+        """(stacked first weight [in_width, W], output projection [W, out_width]), given up to the caller."""
+        products, self.w_qkv, self.w_o = (self.w_qkv, self.w_o), None, None
+        return products
 
     def cache_spec(self):
         return PagedKVSpec(self.n_kv, self.dp, self.window, 0)
@@ -260,11 +294,18 @@ class BlendAttention:
         return {"prefill_tile_rows": set(rows)} if rows else {}
 
     def forward(self, x, step, cache, write_cache=True, sink=None):
-        rt, ops = self.rt, self.rt.ops
+        ops = self.rt.ops
         project = sink.project if sink is not None else ops.linear
-        T, Hq, Hkv, D = x.shape[0], self.n_q, self.n_kv, self.dp
+        o = self.rt.empty(x.shape[0], self.out_width)
+        self.run(ops.linear(x, self.w_qkv), step, cache, write_cache, o)
+        return project(o, self.w_o)
+
+    def run(self, qkv, step, cache, write_cache, out, out_scale=1.0):
+        """From the first product's rows, [T, (Hq + 2 Hkv) * D] (columns of wider rows are fine), to the heads' results
+        side by side times out_scale in out, [T, Hq * D] (columns of wider rows too)."""
+        rt, ops = self.rt, self.rt.ops
+        T, Hq, Hkv, D = qkv.shape[0], self.n_q, self.n_kv, self.dp
         tables = step.groups[cache.group]
-        qkv = ops.linear(x, self.w_qkv)                              # [T, (Hq + 2 Hkv) * D]
         cos, sin, rot = self.position.tables() if self.position is not None else (None, None, 0)
         first = None
         if self.value_rows is not None:
@@ -276,11 +317,10 @@ class BlendAttention:
         q = rt.empty(T, Hq, D)
         ops.qkv_blend_prepare(qkv, Hq, Hkv, D, self.bias, step.positions, cos, sin, rot, q,
                               cache.k_pool if write_cache else None, cache.v_pool if write_cache else None,
-                              tables.slot_mapping, first, self.blend)
-        o = rt.empty(T, Hq, D)
-        ops.attention(q, o, cache.k_pool, cache.v_pool, step, cache.group, self.scale,
-                      int(self.window) if self.window else 0)
-        return project(o.view(T, Hq * D), self.w_o)
+                              tables.slot_mapping, first, self.blend, **self.norms)
+        extras = self.extras if out_scale == 1.0 else dict(self.extras, out_scale=float(out_scale))
+        ops.attention(q, out.view(T, Hq, D), cache.k_pool, cache.v_pool, step, cache.group, self.scale,
+                      int(self.window) if self.window else 0, **extras)
 
 
 register_part("mixer", "blend_attention", BlendAttention)

@@ -20,7 +20,7 @@ from __future__ import annotations
 
 import inspect
 
-from .runtime import Normed, NormSink, Pair, ResidualSink, Scaled
+from .runtime import Normed, NormSink, Pair, ResidualSink, Scaled, StreamRows, unscaled
 
 
 _TAKES_SINK = {}
@@ -288,7 +288,61 @@ class ParallelPreNormBlock:
         return h, Pair(y, f)
 
 
-BLOCKS = {"parallel_pre_norm": ParallelPreNormBlock, "pre_post_norm": PrePostNormBlock, "pre_norm": PreNormBlock, "pre_norm_conv_side": ConvSideBlock, "pre_norm_scaled": ScaledPreNormBlock}
+class PostNormBlock:
+    """A layer whose sublayers read the stream as it is and enter it through a layer norm of their output, the
+    feed-forward optional:
+
+        h += mixer_post_norm(mixer(h));  h += feed_forward_post_norm(feed_forward(h))
+
+    Parts by name: mixer, mixer_post_norm and, both or neither, feed_forward + feed_forward_post_norm (layer norms). One
+    kernel norms a sublayer's output, adds it into the 32-bit stream and leaves the stream's rows in the compute dtype
+    for the next sublayer's first product: between sublayers (and layers of this kind) nothing is pending and those rows
+    are handed on as StreamRows. In 32-bit the stream itself is what the sublayers read."""
+
+    def __init__(self, spec, build):
+        self.mixer, self.mixer_post_norm = build("mixer"), build("mixer_post_norm")
+        self.feed_forward = build("feed_forward") if "feed_forward" in spec.parts else None
+        self.feed_forward_post_norm = build("feed_forward_post_norm") if self.feed_forward is not None else None
+        for norm in (self.mixer_post_norm, self.feed_forward_post_norm):
+            if norm is not None and not getattr(norm, "centered", False):
+                raise ValueError("a layer with norms behind its sublayers only takes layer norms")
+
+    def cache_spec(self):
+        return self.mixer.cache_spec()
+
+    def step_needs(self):
+        return self.mixer.step_needs() if hasattr(self.mixer, "step_needs") else {}
+
+    @staticmethod
+    def _enter(h, y, norm):
+        """h += norm(y); returns the stream's rows for the next sublayer."""
+        rt = norm.rt
+        x = h if rt.dtype == h.dtype else rt.empty(h.shape[0], h.shape[1])
+        rt.ops.layer_norm_add(h, y, norm.weight, norm.eps, None if x is h else x)
+        return x
+
+    def forward(self, h, pending, step, cache, write_cache=True):
+        rt = self.mixer_post_norm.rt
+        if isinstance(pending, StreamRows):
+            x = pending.tensor
+        else:
+            if isinstance(pending, Pair):
+                rt.ops.residual_add(h, pending.first)
+                pending = pending.second
+            delta, factor = unscaled(pending)
+            if delta is not None:
+                rt.ops.residual_add(h, delta, scale=factor)
+            x = h
+            if rt.dtype != h.dtype:
+                x = rt.empty(h.shape[0], h.shape[1])
+                rt.ops.stream_rows(h, x)
+        x = self._enter(h, self.mixer.forward(x, step, cache, write_cache), self.mixer_post_norm)
+        if self.feed_forward is not None:
+            x = self._enter(h, self.feed_forward.forward(x, step), self.feed_forward_post_norm)
+        return h, StreamRows(x)
+
+
+BLOCKS = {"post_norm": PostNormBlock, "parallel_pre_norm": ParallelPreNormBlock, "pre_post_norm": PrePostNormBlock, "pre_norm": PreNormBlock, "pre_norm_conv_side": ConvSideBlock, "pre_norm_scaled": ScaledPreNormBlock}
 
 
 def register_arrangement(name, cls):

@@ -192,3 +192,76 @@ class GatedLinearAttention:
 
 
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+
+
+class HeadDeltaMixer:
+    """The gated delta rule with one decay per head and token.
+
+        q, k, v    = silu(short causal filter(W x))    (a filter per channel, no bias; q, k: kv_heads of D, v: heads of V)
+        q, k       <- unit vectors per head, x / sqrt(sum x^2 + 1e-6); q also times D^-1/2
+        beta       = sigmoid(W_b x),  g = exp(-exp(A_log[h]) * softplus(W_a x + dt_bias[h]))        one each per head
+        S          <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+        y          = W_o (o / rms(o) * w_norm * silu(W_g x))        rms over the head's V, w_norm [V]
+    Head h reads q/k head h // (heads / kv_heads). It is ChannelDeltaMixer's recurrence with a decay that is the same for
+    every row of S and another output gate, on the same kernels (rule "head"), with the same state layout. x goes into one
+    product, [W_q; W_k; W_v | W_b | W_a | W_g], each piece filled up with zero rows to a multiple of 16; the filter and the
+    recurrence read their columns in place. Kept between steps per request: the filters' last taps - 1 inputs and S.
+    Parameters: hidden_size, num_heads, num_kv_heads, head_dim (D), value_dim (V), conv_taps, eps.
+    """
+
+    @staticmethod
+    def tensor_shapes(params):
+        W, H, G, D, V = (params["hidden_size"], params["num_heads"], params["num_kv_heads"], params["head_dim"],
+                         params["value_dim"])
+        taps = params["conv_taps"]
+        return {"q_proj": (G * D, W), "k_proj": (G * D, W), "v_proj": (H * V, W), "q_conv": (G * D, taps),
+                "k_conv": (G * D, taps), "v_conv": (H * V, taps), "b_proj": (H, W), "a_proj": (H, W), "A_log": (H,),
+                "dt_bias": (H,), "o_norm": (V,), "g_proj": (H * V, W), "o_proj": (W, H * V)}
+
+    @staticmethod
+    def random_init(params, role):
+        return ChannelDeltaMixer.random_init(params, role)
+
+    def __init__(self, params, tensors, rt, shared=None):
+        self.rt = rt
+        W = int(params["hidden_size"])
+        self.H, self.G = int(params["num_heads"]), int(params["num_kv_heads"])
+        self.D, self.V = int(params["head_dim"]), int(params["value_dim"])
+        self.taps, self.eps = int(params["conv_taps"]), float(params["eps"])
+        if self.H % self.G:
+            raise ValueError(f"{self.H} heads are not a multiple of {self.G} q/k heads")
+        if hasattr(rt.ops, "delta_rule_fits") and not rt.ops.delta_rule_fits(self.D, self.V):
+            raise ValueError(f"heads of {self.D} x {self.V} are beyond the delta-rule kernel")
+        self.c_conv = 2 * self.G * self.D + self.H * self.V
+
+        def padded(names):
+            m = torch.cat([rt.matrix(tensors[n]) for n in names], dim=0)
+            pad = -m.shape[0] % 16
+            return m if not pad else torch.cat([m, torch.zeros(pad, W, dtype=rt.dtype, device=rt.device)], dim=0)
+        pieces = [padded(names) for names in (("q_proj", "k_proj", "v_proj"), ("b_proj",), ("a_proj",), ("g_proj",))]
+        self.at_b, self.at_a, self.at_g = (sum(m.shape[0] for m in pieces[:i]) for i in (1, 2, 3))
+        self.w_in = rt.product(torch.cat(pieces, dim=0).contiguous())
+        self.w_conv = torch.cat([rt.vector32(tensors[n]) for n in ("q_conv", "k_conv", "v_conv")], dim=0).contiguous()
+        self.a_log, self.dt_bias, self.w_norm = (rt.vector32(tensors[n]) for n in ("A_log", "dt_bias", "o_norm"))
+        self.w_o = rt.product(rt.matrix(tensors["o_proj"]))
+
+    def cache_spec(self):
+        return StateSpec((("conv", (self.taps - 1, self.c_conv), self.rt.dtype_name),
+                          ("S", (self.H, self.V, self.D), "float32")))      # S column by column
+
+    def forward(self, x, step, cache, write_cache=True):
+        rt, ops = self.rt, self.rt.ops
+        if not write_cache:
+            raise ValueError("a delta-rule mixer advances its state with every call; it cannot only read it")
+        T, H = x.shape[0], self.H
+        z = ops.linear(x, self.w_in)                                           # [T, q | k | v | b | a | gate]
+        qkv = rt.empty(T, self.c_conv)
+        ops.causal_conv(z[:, :self.c_conv], self.w_conv, cache.tensors["conv"], step, qkv, silu=True)
+        o = rt.empty(T, H * self.V)
+        ops.delta_rule_head(qkv, z[:, self.at_b:self.at_b + H], z[:, self.at_a:self.at_a + H],
+                            z[:, self.at_g:self.at_g + H * self.V], self.a_log, self.dt_bias, self.w_norm, self.eps,
+                            cache.tensors["S"], step, o, H, self.G, self.D, self.V)
+        return ops.linear(o, self.w_o)
+
+
+register_part("mixer", "head_delta", HeadDeltaMixer)

@@ -37,7 +37,8 @@ class TokenEmbedding:
 
 
 class LinearHead:
-    """logits = x @ W^T in fp32. When tied, ``weight`` names the embedding table."""
+    """logits = x @ W^T in fp32. When tied, ``weight`` names the embedding table. With params softcap c the logits
+    leave as c tanh(logits / c)."""
 
     @staticmethod
     def tensor_shapes(params):
@@ -50,9 +51,11 @@ class LinearHead:
     def __init__(self, params, tensors, rt, shared=None):
         self.rt = rt
         self.weight = rt.product(rt.matrix(tensors["weight"]), out_dtype=torch.float32)
+        self.softcap = float(params.get("softcap") or 0.0)
 
     def forward(self, x):
-        return self.rt.ops.linear(x, self.weight, out_dtype=torch.float32)
+        logits = self.rt.ops.linear(x, self.weight, out_dtype=torch.float32)
+        return self.rt.ops.softcap(logits, self.softcap) if self.softcap else logits
 
 
 register_part("embedding", "token_embedding", TokenEmbedding)

@@ -9,7 +9,7 @@ is multiplied into the 32-bit weight when the part is built).
 from __future__ import annotations
 
 from .registry import register_part
-from .runtime import Pair, ScaledRows, unscaled
+from .runtime import Pair, ScaledRows, StreamRows, unscaled
 
 
 class RMSNorm:
@@ -50,6 +50,8 @@ class RMSNorm:
             if delta.norm is not self or out_rows is not None:
                 raise ValueError("rows prepared for another norm, or for all rows where some are wanted")
             return delta
+        if isinstance(delta, StreamRows):                   # (nothing is left to add)
+            delta = None
         if isinstance(delta, Pair):
             # two outputs that both enter the stream: the first is added by a kernel of its own
             self.rt.ops.residual_add(h, delta.first)
@@ -61,6 +63,42 @@ class RMSNorm:
             self.rt.ops.add_rmsnorm(h, delta, self.weight, self.eps, out, out_rows, delta_scale=factor)
         else:
             self.rt.ops.add_rmsnorm(h, delta, self.weight, self.eps, out, out_rows)
+        return out
+
+
+class LayerNorm:
+    """y = (x - mean) / sqrt(variance + eps) * w over the last axis, the variance the mean of the squared deviations; a
+    weight and no bias, all in 32-bit, rounded to the compute dtype at the end."""
+
+    centered = True             # (an arrangement that puts a norm behind a sublayer asks which kind it has)
+
+    @staticmethod
+    def tensor_shapes(params):
+        return {"weight": (params["size"],)}
+
+    @staticmethod
+    def random_init(params, role):
+        return "norm"
+
+    def __init__(self, params, tensors, rt, shared=None):
+        self.size = int(params["size"])
+        self.eps = float(params["eps"])
+        self.rt = rt
+        self.weight = rt.vector32(tensors["weight"])
+
+    def forward(self, h, delta=None, out_rows=None):
+        """h (fp32 [T, size]) += delta in place; returns norm(h) (only rows out_rows, if given)."""
+        ops = self.rt.ops
+        if isinstance(delta, StreamRows):                   # (nothing is left to add)
+            delta = None
+        if isinstance(delta, Pair):
+            ops.residual_add(h, delta.first)
+            delta = delta.second
+        delta, factor = unscaled(delta)
+        if delta is not None:
+            ops.residual_add(h, delta, scale=factor)
+        out = self.rt.empty(h.shape[0] if out_rows is None else out_rows.shape[0], self.size)
+        ops.layer_norm(h, self.weight, self.eps, out, out_rows)
         return out
 
 
@@ -77,4 +115,5 @@ class Factor:
 
 
 register_part("norm", "rms_norm", RMSNorm)
+register_part("norm", "layer_norm", LayerNorm)
 register_part("norm", "factor", Factor)

@@ -72,6 +72,19 @@ class Normed:
         return self.tensor.shape
 
 
+class StreamRows:
+    """Nothing is pending, and ``tensor`` [T, H] holds the residual stream's rows in the compute dtype, formed by the
+    kernel that formed the stream: what a sublayer that reads the stream as it is (no norm in front) begins with."""
+    __slots__ = ("tensor",)
+
+    def __init__(self, tensor):
+        self.tensor = tensor
+
+    @property
+    def shape(self):
+        return self.tensor.shape
+
+
 class Pair:
     """Two outputs of one layer that both enter the residual stream (sublayers that ran side by side on the same
     stream): h += first + second. Whatever adds the pending output into the stream takes both."""

@@ -156,7 +156,7 @@ class TorchOps:
     # rollout/attention.py:126-139 over the tables of rollout/cache.py:282-328,
     # gathered as opd/test_parallel.py:14-42 does
     def attention(self, q, out, k_pool, v_pool, step, group, scale, window=0, head_scale=None, softcap=0.0,
-                  keep_first=0, sink=False):
+                  keep_first=0, sink=False, sink_logit=None, out_scale=1.0, fine_weights=False):
         g = step.groups[group]
         n_q, n_kv = q.shape[1], k_pool.shape[1]
         cu_q, cu_p = step.cu_q.tolist(), g.cu_pages.tolist()
@@ -184,12 +184,14 @@ class TorchOps:
                     far = far & (k_pos[None, :] >= keep_first)
                 hide = hide | far
             score = score.masked_fill(hide[None], float("-inf"))
-            if sink:                                        # one more key of score 0 that has no value
-                zero = torch.zeros_like(score[..., :1])
-                prob = torch.cat([score, zero], dim=-1).softmax(-1)[..., :-1]
+            if sink or sink_logit is not None:              # one more key (of score 0, or a learned score) that has no value
+                extra = torch.zeros_like(score[..., :1])
+                if sink_logit is not None:
+                    extra = extra + sink_logit.float()[:, None, None]
+                prob = torch.cat([score, extra], dim=-1).softmax(-1)[..., :-1]
             else:
                 prob = score.softmax(-1)
-            out[a:b] = torch.einsum("hqk,khd->qhd", prob, vv).to(out.dtype)
+            out[a:b] = (out_scale * torch.einsum("hqk,khd->qhd", prob, vv)).to(out.dtype)
 
     # ---- attention with two score maps per head over the same values
     def maps_qkv_prepare(self, qkv, n_q, n_kv, maps, D, Dv, positions, cos, sin, rotary_dim, interleaved, q_out,
@@ -314,11 +316,17 @@ class TorchOps:
 
     # ---- attention with biases, one row width for q, k and v, values blended with an earlier layer's
     def qkv_blend_prepare(self, qkv, n_q, n_kv, D, bias, positions, cos, sin, rotary_dim, q_out, k_pool, v_pool,
-                          slot_mapping, first=None, blend=None):
+                          slot_mapping, first=None, blend=None, w_q=None, w_k=None, norm_dim=None, eps=0.0):
         T = qkv.shape[0]
-        x = qkv.float() + bias
-        q = self._turn(x[:, :n_q * D].reshape(T, n_q, D), positions, cos, sin, rotary_dim)
-        k = self._turn(x[:, n_q * D:(n_q + n_kv) * D].reshape(T, n_kv, D), positions, cos, sin, rotary_dim)
+        x = qkv.float() + (bias if bias is not None else 0.0)
+
+        def normed(v, w):
+            if w is None:
+                return v
+            n = D if norm_dim is None else norm_dim
+            return v / torch.sqrt((v[..., :n] ** 2).sum(-1, keepdim=True) / n + eps) * w
+        q = self._turn(normed(x[:, :n_q * D].reshape(T, n_q, D), w_q), positions, cos, sin, rotary_dim)
+        k = self._turn(normed(x[:, n_q * D:(n_q + n_kv) * D].reshape(T, n_kv, D), w_k), positions, cos, sin, rotary_dim)
         v = x[:, (n_q + n_kv) * D:]
         if first is not None:                               # [T, n_kv Dv]: the heads' true width, Dv <= D
             Dv = first.shape[1] // n_kv
@@ -368,8 +376,10 @@ class TorchOps:
         x.copy_((x.float() + bias).to(x.dtype))
         return x
 
-    def causal_conv(self, x, w, tail, step, out, add_input=False, silu=False, bias=None):
+    def causal_conv(self, x, w, tail, step, out, add_input=False, silu=False, bias=None, in_bias=None):
         taps = w.shape[1]
+        if in_bias is not None:
+            x = (x.float() + in_bias).to(x.dtype)
         cu, slots = step.cu_q_host, step.slot_ids_host
         for s in range(step.n_seqs):
             a, b = cu[s], cu[s + 1]
@@ -415,6 +425,70 @@ class TorchOps:
                 o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * norm_w * gate[t]
                 out[t] = o.reshape(-1).to(out.dtype)
         return out
+
+    def delta_rule_head(self, qkv, beta, a, gate, a_log, dt_bias, norm_w, eps, state, step, out, H, G, D, V):
+        """The delta rule with one decay per head, g = exp(-exp(a_log) softplus(a + dt_bias)), and the gate silu."""
+        cu, slots = step.cu_q_host, step.slot_ids_host
+        T, rep = qkv.shape[0], H // G
+        q = qkv[:, :G * D].float().view(T, G, D)
+        k = qkv[:, G * D:2 * G * D].float().view(T, G, D)
+        v = qkv[:, 2 * G * D:].float().view(T, H, V)
+        q = (q / torch.sqrt((q * q).sum(-1, keepdim=True) + 1e-6) * D ** -0.5).repeat_interleave(rep, dim=1)
+        k = (k / torch.sqrt((k * k).sum(-1, keepdim=True) + 1e-6)).repeat_interleave(rep, dim=1)
+        b = torch.sigmoid(beta.float())
+        g = torch.exp(-torch.exp(a_log) * torch.nn.functional.softplus(a.float() + dt_bias, threshold=30.0))
+        c = gate.float().view(T, H, V)
+        c = c * torch.sigmoid(c)
+        for s in range(step.n_seqs):
+            S = state[slots[s]].transpose(1, 2)               # kept [H, V, D]; a view [H, D, V], updated in place
+            for t in range(cu[s], cu[s + 1]):
+                S *= g[t][:, None, None]
+                u = b[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+                S += k[t][:, :, None] * u[:, None, :]
+                o = torch.einsum("hdv,hd->hv", S, q[t])
+                o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * norm_w * c[t]
+                out[t] = o.reshape(-1).to(out.dtype)
+        return out
+
+    def channel_recurrence(self, u, w_gates, gate_bias, rate, y, y_bias, state, step, out, out_scale=1.0):
+        """r, i = sigmoid(block matrices u + bias); a = exp(rate r); S <- a S + sqrt(1 - a^2) i u;
+        out = S gelu_tanh(y + y_bias) out_scale, zeros in the columns beyond the recurrence's."""
+        cu, slots = step.cu_q_host, step.slot_ids_host
+        T, C = u.shape
+        B = w_gates.shape[0]
+        uf = u.float()
+        gate = lambda j: torch.sigmoid(torch.einsum("tbc,bdc->tbd", uf.view(T, B, C // B), w_gates[:, j].float()).reshape(T, C)
+                                       + gate_bias[j])
+        log_a = rate * gate(0)
+        a, x = torch.exp(log_a), torch.sqrt(-torch.expm1(2.0 * log_a)) * gate(1) * uf
+        z = y.float() + y_bias
+        z = 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3))) * out_scale
+        out[:, C:] = 0
+        for s in range(step.n_seqs):
+            S = state[slots[s]]
+            for t in range(cu[s], cu[s + 1]):
+                S.mul_(a[t]).add_(x[t])
+                out[t, :C] = (S * z[t]).to(out.dtype)
+        return out
+
+    # ---- a layer norm behind a sublayer
+    def layer_norm_add(self, h, y, weight, eps, out=None):
+        c = y.float() - y.float().mean(-1, keepdim=True)
+        h += c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight
+        if out is not None:
+            out.copy_(h.to(out.dtype))
+
+    def layer_norm(self, h, weight, eps, out, rows=None):
+        v = h if rows is None else h[rows.long()]
+        c = v - v.mean(-1, keepdim=True)
+        out.copy_((c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight).to(out.dtype))
+
+    def stream_rows(self, h, out):
+        out.copy_(h.to(out.dtype))
+
+    def softcap(self, z, cap):
+        z.copy_(cap * torch.tanh(z / cap))
+        return z
 
     def outer_rule(self, qkv, a, gate, decay_bias, tau, norm_w, eps, state, step, out, H, D, V):
         """S <- diag(alpha) S + k v^T, o = S^T q with alpha = sigmoid(a + bias)^(1/tau); the read-out normed over the
