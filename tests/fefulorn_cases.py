@@ -230,18 +230,20 @@ def run_in_pieces(parts, xs, pieces, P=16, pages=(2, 0, 3, 1), slot=1):
     i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)
     T = xs[0].shape[0]
     caches, tile_rows = [], set()
-    for part in parts:
-        spec = part.cache_spec()
+
+    def view(spec):
         if isinstance(spec, PagedKVSpec):
             if len(pages) * P < T:
                 raise ValueError("too few pages for these rows")
-            caches.append(types.SimpleNamespace(
+            width = spec.head_dim if spec.value_dim is None else spec.value_dim
+            return types.SimpleNamespace(
                 group=0, k_pool=torch.zeros(max(pages) + 2, spec.num_kv_heads, P, spec.head_dim, dtype=dt, device=dev),
-                v_pool=torch.zeros(max(pages) + 2, spec.num_kv_heads, P,
-                                   spec.head_dim if spec.value_dim is None else spec.value_dim, dtype=dt, device=dev)))
-        else:
-            caches.append(types.SimpleNamespace(tensors={
-                name: torch.zeros(slot + 2, *shape, dtype=getattr(torch, kind), device=dev) for name, shape, kind in spec.tensors}))
+                v_pool=torch.zeros(max(pages) + 2, spec.num_kv_heads, P, width, dtype=dt, device=dev))
+        return types.SimpleNamespace(tensors={
+            name: torch.zeros(slot + 2, *shape, dtype=getattr(torch, kind), device=dev) for name, shape, kind in spec.tensors})
+    for part in parts:
+        spec = part.cache_spec()
+        caches.append(tuple(view(s) for s in spec) if isinstance(spec, (tuple, list)) else view(spec))
         tile_rows |= set((part.step_needs() if hasattr(part, "step_needs") else {}).get("prefill_tile_rows", ()))
     outs, at = [[] for _ in parts], 0
     for n in pieces:

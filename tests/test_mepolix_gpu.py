@@ -1,0 +1,501 @@
+"""Mepolix on the GPU: every new kernel alone against its torch stand-in; the attention with inputs made so that one far
+key or the sink decides (a page's first and last row, the first places, far back; as a prompt's portion and decoded), on
+the plain and the matrix-core kernels; each mixer of the package in pieces against the plain function; the engine against
+the plain model whole, with a decoded tail, in portions down to two tokens and in mixed batches with pages and slots used
+again, in both precisions and on configurations drawn from seeds; long decoding; greedy generation through
+Engine.generate with and without graphs; the command line; the trace program."""
+import os
+
+import pytest
+import torch
+
+from tests import trace_tools as tt
+from tests.mepolix_cases import (CASES, attention_tensors, build_attention, build_delta, build_parallel, build_recurrence,
+                                 deciding_rows, delta_tensors, make_folder, recurrence_tensors, run_in_pieces, runtime)
+from tests.plain import mepolix_plain as plain
+from tests.test_fefulorn_gpu import i32, paged_step, rnd, row_error, state_step, tol
+from tests.torch_ops import TorchOps
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+DTYPES = [torch.float32, torch.bfloat16]
+RANDOM_SEEDS = [501, 502, 503, 504, 505, 506, 507, 508, 509, 510]
+
+
+@pytest.fixture(scope="module")
+def ops():
+    from return_amd.kernels.hip_ops import HipOps
+    return HipOps(DEV)
+
+
+@pytest.fixture(scope="module")
+def ref():
+    return TorchOps(DEV)
+
+
+def d64(w):
+    return {k: v.double() for k, v in w.items()}
+
+
+# ------------------------------------------------------------------ kernels alone
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,H", [(1, 64), (7, 76), (33, 210), (300, 4096), (2, 5000), (5, 9)])
+def test_layer_norm_kernels(ops, ref, dtype, T, H):
+    w = 1 + rnd(H, seed=4, scale=0.2)
+    for want_rows in (True, False):
+        ha = rnd(T, H, seed=1, scale=2.0)
+        hb, y = ha.clone(), (rnd(T, H, seed=2) + 5.0).to(dtype)            # (a mean far from zero)
+        xa, xb = (torch.zeros(T, H, dtype=dtype, device=DEV) for _ in range(2))
+        ops.layer_norm_add(ha, y, w, 1e-5, xa if want_rows else None)
+        ref.layer_norm_add(hb, y, w, 1e-5, xb)
+        torch.testing.assert_close(ha, hb, atol=2e-5, rtol=2e-5)
+        if want_rows:
+            torch.testing.assert_close(xa.float(), xb.float(), **tol(dtype))
+    rows = i32([T - 1, 0, T // 2])
+    a, b = (torch.zeros(3, H, dtype=dtype, device=DEV) for _ in range(2))
+    ops.layer_norm(ha, w, 1e-6, a, rows)
+    ref.layer_norm(ha, w, 1e-6, b, rows)
+    torch.testing.assert_close(a.float(), b.float(), **tol(dtype))
+    ops.stream_rows(ha, xa)
+    assert torch.equal(xa, ha.to(dtype))
+
+
+def test_soft_cap(ops):
+    z = rnd(5, 331, seed=1, scale=30.0)
+    want = 12.0 * torch.tanh(z.double() / 12.0)
+    ops.softcap(z, 12.0)
+    torch.testing.assert_close(z.double(), want, atol=1e-5, rtol=1e-6)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("Hq,Hkv,D,Dn,R,P,T", [(4, 2, 16, 12, 8, 16, 37), (3, 3, 10, 10, 10, 4, 5), (8, 1, 64, 32, 32, 16, 70),
+                                               (2, 2, 12, 5, 0, 8, 1), (5, 5, 128, 128, 64, 16, 19), (6, 2, 80, 66, 2, 32, 33)])
+def test_preparation_with_head_norms_and_no_biases(ops, ref, dtype, Hq, Hkv, D, Dn, R, P, T):
+    """Rows are columns of wider rows; what a head has beyond its true width is zero."""
+    n = (Hq + 2 * Hkv) * D
+    wide = rnd(T, n + 40, dtype=dtype, seed=1)
+    heads = wide[:, 8:8 + n].view(T, Hq + 2 * Hkv, D)
+    heads[:, :Hq + Hkv, Dn:] = 0
+    w = torch.zeros(2, D, device=DEV)
+    w[:, :Dn] = 1 + rnd(2, Dn, seed=2, scale=0.3)
+    positions = i32([(7 * t) % 90 for t in range(T)])
+    R = min(R, Dn // 2 * 2)
+    cos, sin = rnd(90, max(R // 2, 1), seed=3), rnd(90, max(R // 2, 1), seed=4)
+    pages = -(-T // P) + 2
+    slots = i32(torch.randperm(pages * P, generator=torch.Generator().manual_seed(6))[:T].tolist())
+    outs = []
+    for k in (ops, ref):
+        q = torch.zeros(T, Hq, D, dtype=dtype, device=DEV)
+        kp, vp = (torch.zeros(pages, Hkv, P, D, dtype=dtype, device=DEV) for _ in range(2))
+        k.qkv_blend_prepare(wide[:, 8:8 + n], Hq, Hkv, D, None, positions, cos if R else None, sin if R else None, R, q, kp, vp,
+                            slots, w_q=w[0], w_k=w[1], norm_dim=Dn, eps=1e-5)
+        outs.append((q, kp, vp))
+    for a, b in zip(*outs):
+        torch.testing.assert_close(a.float(), b.float(), **tol(dtype))
+
+
+ATTENTION = [
+    # heads, kv heads, D, P, [(q_len, q_start)]
+    (4, 2, 64, 16, [(5, 0), (17, 30), (33, 100)]),
+    (6, 3, 128, 16, [(1, 99), (24, 8), (1, 0), (2, 262), (1, 400)]),
+    (5, 5, 24, 4, [(40, 3), (1, 200)]),
+    (16, 1, 32, 64, [(1, 700), (1, 64), (1, 1), (1, 3000)]),
+    (34, 2, 16, 16, [(1, 150), (200, 120), (1, 8)]),
+    (2, 1, 80, 16, [(2, 0), (2, 14), (2, 15), (2, 16), (40, 16)]),
+    (4, 4, 192, 16, [(64, 0), (130, 64), (1, 500)]),
+    (8, 8, 64, 16, [(1, 4000)] * 32),
+    (4, 2, 272, 16, [(9, 60), (1, 100)]),
+]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("Hq,Hkv,D,P,segs", ATTENTION)
+def test_attention_kernels_with_learned_sinks(ops, ref, dtype, Hq, Hkv, D, P, segs):
+    """A sink per head (from far below the scores to far above), the result times a factor into columns of wider rows."""
+    q_lens, q_starts = [s[0] for s in segs], [s[1] for s in segs]
+    need = [-(-(a + b) // P) for a, b in segs]
+    perm = torch.randperm(sum(need) + 3, generator=torch.Generator().manual_seed(5)).tolist()
+    pages_of = [[perm.pop() for _ in range(k)] for k in need]
+    step = paged_step(q_lens, q_starts, P, pages_of)
+    kp, vp = (rnd(sum(need) + 3, Hkv, P, D, dtype=dtype, seed=s) for s in (51, 52))
+    T = sum(q_lens)
+    q = rnd(T, Hq, D, dtype=dtype, seed=53, scale=2.0)
+    sink = torch.linspace(-20.0, 12.0, Hq, device=DEV)
+    for fine in (False, True):
+        wide = [torch.full((T, Hq * D + 48), 7.0, dtype=dtype, device=DEV) for _ in range(2)]
+        for k, o in zip((ops, ref), wide):
+            k.attention(q, o[:, 16:16 + Hq * D].view(T, Hq, D), kp, vp, step, 0, D ** -0.5, sink_logit=sink, out_scale=-0.75,
+                        fine_weights=fine)
+        torch.testing.assert_close(wide[0].float(), wide[1].float(), **tol(dtype))
+        assert bool((wide[0][:, :16] == 7.0).all()) and bool((wide[0][:, 16 + Hq * D:] == 7.0).all())
+    plain_out, no_sink = torch.empty_like(q), torch.empty_like(q)
+    ops.attention(q, plain_out, kp, vp, step, 0, D ** -0.5, sink_logit=sink)
+    ops.attention(q, no_sink, kp, vp, step, 0, D ** -0.5)
+    assert (plain_out.float() - no_sink.float())[:, -1].abs().max() > 0.05
+
+
+@pytest.mark.parametrize("q_len,q_start", [(1, 900), (64, 836), (2, 898)])
+def test_fine_weights_are_finer(ops, q_len, q_start):
+    """One value far out under a weight near one, its opposites under small weights: the rounding of the weights to 8
+    bits of mantissa shows beside the rest, and is gone with 16."""
+    H, D, P = 4, 64, 16
+    n = q_len + q_start
+    pages = [list(range(-(-n // P)))]
+    step = paged_step([q_len], [q_start], P, pages)
+    kp, vp = rnd(len(pages[0]), H, P, D, dtype=torch.bfloat16, seed=1), rnd(len(pages[0]), H, P, D, dtype=torch.bfloat16, seed=2, scale=64.0)
+    q = rnd(q_len, H, D, dtype=torch.bfloat16, seed=3)
+    errs = []
+    k, v = (x.double().transpose(1, 2).reshape(-1, H, D)[:n] for x in (kp, vp))
+    s = torch.einsum("qhd,khd->hqk", q.double(), k) * 0.05
+    i, j = torch.arange(q_start, n, device=DEV)[:, None], torch.arange(n, device=DEV)[None, :]
+    want = torch.einsum("hqk,khd->qhd", s.masked_fill(j > i, float("-inf")).softmax(-1), v)
+    for fine in (False, True):
+        o = torch.empty_like(q)
+        ops.attention(q, o, kp, vp, step, 0, 0.05, sink_logit=torch.full((H,), -60.0, device=DEV), fine_weights=fine)
+        errs.append((o.double() - want).pow(2).mean().sqrt())
+    rounding = (want.to(torch.bfloat16).double() - want).pow(2).mean().sqrt()
+    assert errs[1] < 1.15 * rounding and errs[1] < errs[0]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("C,taps,q_lens", [(40, 4, [5, 1, 33]), (300, 2, [1, 1]), (16, 8, [70]), (513, 3, [2, 17, 1]), (24, 1, [3, 20])])
+def test_convolution_with_biased_inputs(ops, ref, dtype, C, taps, q_lens):
+    """From a tail of zeros (a request's start: zeros, not biased inputs) and on; the tail holds the biased inputs."""
+    n, T = len(q_lens), sum(q_lens)
+    slots = torch.randperm(n + 1, generator=torch.Generator().manual_seed(n)).tolist()[:n]
+    x = rnd(T, C + 24, dtype=dtype, seed=1)[:, 8:8 + C]
+    w, bias, in_bias = rnd(C, taps, seed=2, scale=0.5), rnd(C, seed=3, scale=0.3), rnd(C, seed=4)
+    tail_a = torch.zeros(n + 1, taps - 1, C, dtype=dtype, device=DEV)
+    tail_b = tail_a.clone()
+    for _ in range(2):
+        step = state_step(q_lens, slots)
+        a, b = torch.zeros(T, C, dtype=dtype, device=DEV), torch.zeros(T, C, dtype=dtype, device=DEV)
+        ops.causal_conv(x, w, tail_a, step, a, bias=bias, in_bias=in_bias)
+        ref.causal_conv(x, w, tail_b, step, b, bias=bias, in_bias=in_bias)
+        torch.testing.assert_close(a.float(), b.float(), **tol(dtype))
+        torch.testing.assert_close(tail_a.float(), tail_b.float(), atol=0, rtol=0)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("C,blocks,q_lens", [
+    (64, 4, [1, 1, 1]), (72, 3, [5, 1, 33]), (80, 1, [40]), (27, 3, [2, 17]), (320, 2, [1, 32, 1, 31]), (300, 5, [1] * 40),
+    (48, 6, [65, 2]), (2560, 16, [300]), (16, 2, [2500, 1]), (600, 1, [9, 100]), (128, 2, [33, 32, 64, 1])])
+def test_channel_recurrence(ops, ref, dtype, C, blocks, q_lens):
+    """Two steps in a row over slots that hold something; chunks of every kind (single rows, one chunk, a chunk's edge,
+    several, longer chunks for a long request), blocks that the matrix cores take and blocks that they do not, columns of
+    wider rows on both sides."""
+    n, T, bw = len(q_lens), sum(q_lens), C // blocks
+    slots = torch.randperm(n + 1, generator=torch.Generator().manual_seed(n)).tolist()[:n]
+    y = rnd(T, C + 24, dtype=dtype, seed=1)[:, 16:16 + C]
+    u = rnd(T, C, dtype=dtype, seed=2)
+    w = rnd(blocks, 2, bw, bw, dtype=dtype, seed=3, scale=bw ** -0.5)
+    gate_bias, y_bias = rnd(2, C, seed=4), rnd(C, seed=5, scale=0.3)
+    rate = -8.0 * torch.nn.functional.softplus(rnd(C, seed=6, scale=2.0) - 4.0)
+    state_a = rnd(n + 1, C, seed=7)
+    state_b = state_a.clone()
+    extra = -C % 16 + 16
+    for _ in range(2):
+        step = state_step(q_lens, slots)
+        outs = []
+        for k, state in ((ops, state_a), (ref, state_b)):
+            wide = torch.full((T, C + extra + 32), 3.0, dtype=dtype, device=DEV)
+            k.channel_recurrence(u, w, gate_bias, rate, y, y_bias, state, step, wide[:, 16:16 + C + extra], 1.5)
+            outs.append(wide)
+        torch.testing.assert_close(outs[0].float(), outs[1].float(), **tol(dtype))
+        torch.testing.assert_close(state_a, state_b, atol=2e-5, rtol=2e-5)
+        assert bool((outs[0][:, :16] == 3.0).all()) and bool((outs[0][:, 16 + C + extra:] == 3.0).all())
+        assert bool((outs[0][:, 16 + C:16 + C + extra] == 0.0).all())
+
+
+def test_channel_recurrence_decays_near_one(ops, ref):
+    """log a of 1e-7 and of -40: the input's factor keeps its digits, the state of 3,000 rows is the plain one."""
+    C, T = 16, 3000
+    u, w = rnd(T, C, seed=1), torch.zeros(2, 2, 8, 8, device=DEV)
+    gate_bias = torch.zeros(2, C, device=DEV)
+    rate = torch.cat([torch.full((8,), -2e-7), torch.full((8,), -80.0)]).to(DEV)
+    y, y_bias = torch.ones(T, C, device=DEV), torch.zeros(C, device=DEV)
+    sa = torch.zeros(2, C, device=DEV)
+    out = torch.empty(T, C, device=DEV)
+    step = state_step([T], [1])
+    ops.channel_recurrence(u, w, gate_bias, rate, y, y_bias, sa, step, out)
+    log_a = rate.double() * 0.5
+    S = torch.zeros(C, dtype=torch.float64, device=DEV)
+    for t in range(T):
+        S = torch.exp(log_a) * S + torch.sqrt(-torch.expm1(2 * log_a)) * 0.5 * u[t].double()
+    torch.testing.assert_close(sa[1].double(), S, atol=1e-7, rtol=1e-4)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,D,V,q_lens", [
+    (2, 1, 32, 48, [1, 1, 1]), (3, 3, 8, 12, [5, 1, 33]), (4, 2, 64, 64, [40]), (2, 2, 16, 8, [2, 17]), (4, 1, 16, 32, [1, 19]),
+    (2, 1, 128, 128, [1, 70]), (6, 3, 40, 32, [9, 300]), (3, 1, 7, 10, [37, 2]), (3, 3, 40, 33, [3, 64, 1]), (1, 1, 4, 64, [130]),
+    (8, 8, 128, 64, [1] * 6), (2, 1, 256, 130, [12, 1])])
+def test_delta_rule_with_one_decay_per_head(ops, ref, dtype, H, G, D, V, q_lens):
+    n, T = len(q_lens), sum(q_lens)
+    slots = torch.randperm(n + 1, generator=torch.Generator().manual_seed(n)).tolist()[:n]
+    c = 2 * G * D + H * V
+    wide = rnd(T, c + H * V + 48, dtype=dtype, seed=1)
+    qkv, gate = wide[:, :c], wide[:, c:c + H * V]
+    beta, a = wide[:, c + H * V + 8:c + H * V + 8 + H], wide[:, c + H * V + 24:c + H * V + 24 + H]
+    a_log, dt_bias, norm_w = rnd(H, seed=2, scale=0.5) - 0.5, rnd(H, seed=3) - 1.0, 1 + rnd(V, seed=4, scale=0.1)
+    state_a = rnd(n + 1, H, V, D, seed=5, scale=0.3)
+    state_b = state_a.clone()
+    for _ in range(2):
+        step = state_step(q_lens, slots)
+        o, p = torch.empty(T, H * V, dtype=dtype, device=DEV), torch.empty(T, H * V, dtype=dtype, device=DEV)
+        ops.delta_rule_head(qkv, beta, a, gate, a_log, dt_bias, norm_w, 1e-5, state_a, step, o, H, G, D, V)
+        ref.delta_rule_head(qkv, beta, a, gate, a_log, dt_bias, norm_w, 1e-5, state_b, step, p, H, G, D, V)
+        torch.testing.assert_close(o.float(), p.float(), **tol(dtype))
+        torch.testing.assert_close(state_a, state_b, atol=1e-4, rtol=1e-4)
+
+
+# ------------------------------------------------------------------ one far key decides
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("sizes", [dict(heads=3, kv_heads=1, dim=10, vdim=6), dict(heads=4, kv_heads=2, dim=64, vdim=48),
+                                   dict(heads=2, kv_heads=2, dim=32, vdim=80)], ids=["plain_kernel", "matrix_cores", "wide_values"])
+@pytest.mark.parametrize("key_at", [0, 3, 15, 16, 333])
+def test_a_far_key_decides(ops, dtype, sizes, key_at):
+    W, query_at, eps = 32, 610, 1e-5
+    T = query_at + 3
+    m = dict(sizes, scale=1.0)
+    w = attention_tensors(torch.Generator().manual_seed(9), W, m, torch.bfloat16 if dtype == "bfloat16" else torch.float32)
+    x, m["scale"] = deciding_rows(T, W, query_at, key_at, w, m, seed=4)
+    if dtype == "bfloat16":
+        x = x.bfloat16().float()
+    for sink, stays in ((-40.0, True), (60.0, False)):
+        w["sink"] = torch.full((m["heads"],), sink)
+        want = plain.sink_attention(x.double(), d64(w), m, eps)
+        alone = (x[key_at].double() @ d64(w)["v"].T).view(m["kv_heads"], -1).repeat_interleave(m["heads"] // m["kv_heads"], 0).reshape(-1) \
+            @ d64(w)["o"].T
+        assert ((want[query_at] - alone).abs().max() < 1e-3) == stays
+        for pieces in ([T], [query_at] + [1] * 3, [key_at + 1, T - key_at - 1]):
+            rt = runtime(ops, dtype, DEV, positions=1024)
+            got, = run_in_pieces([build_attention(rt, W, m, w, eps)], [x], pieces, pages=tuple(reversed(range(-(-T // 16)))))
+            err = (got.double() - want)[query_at].abs().max() / alone.abs().max()
+            assert err < (1e-4 if dtype == "float32" else 5e-2), f"{pieces}: {err}"
+
+
+# ------------------------------------------------------------------ the mixers of the package in pieces
+PIECES = ([150], [100] + [1] * 50, [5, 2, 1, 17, 64, 61])
+
+
+@pytest.mark.parametrize("m", [
+    {"left": dict(heads=4, kv_heads=2, dim=8, vdim=12, scale=0.7, rot={"base": 500.0, "dims": 6, "scaling": {"factor": 4.0, "original": 16, "fast": 4.0, "slow": 0.5}}),
+     "right": dict(width=27, blocks=3, conv=3), "left_scale": 0.4, "right_scale": -1.5},
+    {"left": dict(heads=4, kv_heads=1, dim=64, vdim=48, scale=0.2, rot={"base": 5000.0, "dims": 16}),
+     "right": dict(width=96, blocks=2, conv=4), "left_scale": 1.0, "right_scale": 1.0}], ids=["odd_sizes", "matrix_cores"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_mixers_side_by_side_in_pieces(ops, dtype, m):
+    g = torch.Generator().manual_seed(3)
+    W, eps = 40, 1e-5
+    store = torch.bfloat16 if dtype == "bfloat16" else torch.float32
+    wl, wr = attention_tensors(g, W, m["left"], store), recurrence_tensors(g, W, m["right"], store)
+    x = torch.randn(150, W, generator=g).to(store).float()
+    want = plain.parallel(x.double(), {**{"left." + k: v for k, v in wl.items()}, **{"right." + k: v for k, v in wr.items()}}, m, eps)
+    for pieces in PIECES:
+        got, = run_in_pieces([build_parallel(runtime(ops, dtype, DEV), W, m, wl, wr, eps)], [x], pieces, pages=tuple(reversed(range(10))))
+        if dtype == "float32":
+            torch.testing.assert_close(got.double(), want, atol=1e-4, rtol=1e-4)
+        else:
+            assert (got.double() - want).pow(2).mean().sqrt() < 0.02 * want.pow(2).mean().sqrt()
+
+
+@pytest.mark.parametrize("m", [dict(heads=4, kv_heads=2, dim=6, vdim=10, conv=3), dict(heads=3, kv_heads=1, dim=12, vdim=5, conv=1),
+                               dict(heads=4, kv_heads=2, dim=64, vdim=128, conv=4)], ids=["grouped", "one_tap", "full_size"])
+def test_delta_mixer_in_pieces(ops, m):
+    g = torch.Generator().manual_seed(m["heads"])
+    W, eps = 40, 1e-5
+    w = delta_tensors(g, W, m)
+    x = torch.randn(150, W, generator=g)
+    want, _, _ = plain.delta(x.double(), d64(w), m, eps)
+    for pieces in PIECES:
+        got, = run_in_pieces([build_delta(runtime(ops, "float32", DEV), W, m, w, eps)], [x], pieces, pages=tuple(range(10)))
+        torch.testing.assert_close(got.double(), want, atol=1e-4, rtol=1e-4)
+
+
+@pytest.mark.parametrize("m", [dict(width=24, blocks=3, conv=4), dict(width=35, blocks=5, conv=1), dict(width=256, blocks=4, conv=8)],
+                         ids=["blocks", "one_tap", "long_filter"])
+def test_channel_recurrence_part_in_pieces(ops, m):
+    g = torch.Generator().manual_seed(m["conv"])
+    W = 40
+    w = recurrence_tensors(g, W, m)
+    x = torch.randn(150, W, generator=g)
+    want, _, _ = plain.gated_recurrence(x.double(), d64(w), m)
+    for pieces in PIECES:
+        got, = run_in_pieces([build_recurrence(runtime(ops, "float32", DEV), W, m, w)], [x], pieces, pages=tuple(range(10)))
+        torch.testing.assert_close(got.double(), want, atol=1e-4, rtol=1e-4)
+
+
+# ------------------------------------------------------------------ the engine against the plain model
+LENGTHS = {"a": 5, "b": 17, "c": 33, "d": 100, "e": 64, "f": 150, "g": 1, "h": 47}
+# A row's error: the root mean square over the vocabulary of the difference of the logits, its mean taken off, over
+# the root mean square of the plain logits.
+ROW_ERROR = {"float32": 5e-5, "bfloat16": 0.12}
+ROW_ERROR_16_MEAN = 0.03
+
+
+def make_runner(folder, dtype, max_tokens, page=16, **kw):
+    from return_amd.config import EngineConfig
+    from return_amd.engine import ModelRunner
+    ec = EngineConfig(dtype=dtype, page_size=page, max_token=max_tokens, max_reside=4, max_step_tokens=max(max_tokens, 4),
+                      prefill_chunk=max_tokens, tune_products=False, check_invariants=True, **kw)
+    return ModelRunner(folder, engine_config=ec)
+
+
+@pytest.fixture(scope="module", params=sorted(CASES))
+def model(request, tmp_path_factory):
+    folder = make_folder(tmp_path_factory, request.param)
+    cfg, w = plain.read_folder(folder)
+    reqs = {rid: tt.random_tokens(cfg["vocab"], n, seed=ord(rid)) for rid, n in LENGTHS.items()}
+    want = {rid: plain.logits(cfg, w, toks) for rid, toks in reqs.items()}
+    return folder, cfg, reqs, want
+
+
+def compare(got, want, reqs, dtype):
+    errs = []
+    for rid, toks in reqs.items():
+        for p in range(len(toks)):
+            e = row_error(got[(rid, p)], want[rid][p])
+            errs.append(e)
+            assert e <= ROW_ERROR[dtype], f"request {rid} position {p} (first wrong place): row error {e:.3e}"
+    if dtype == "bfloat16":
+        assert sum(errs) / len(errs) <= ROW_ERROR_16_MEAN, f"mean row error {sum(errs) / len(errs):.3e}"
+    return max(errs)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("cut", ["whole", "tail_decoded", "portions", "mixed"])
+def test_engine_matches_plain(model, dtype, cut):
+    folder, cfg, reqs, want = model
+    steps = {"whole": tt.whole, "tail_decoded": tt.tail_decoded, "portions": tt.portions, "mixed": tt.mixed}[cut](reqs)
+    runner = make_runner(folder, dtype, tt.peak_tokens(steps))
+    got = tt.run_in_process(runner, steps)
+    print(f"mepolix {dtype} {cut}: largest row error {compare(got, want, reqs, dtype):.2e}")
+    assert not runner.cache.live and all(g.pages.in_use() == 0 for g in runner.cache.groups)
+
+
+@pytest.mark.parametrize("seed", RANDOM_SEEDS)
+def test_configurations_drawn_at_random(tmp_path_factory, seed):
+    folder = make_folder(tmp_path_factory, seed)
+    cfg, w = plain.read_folder(folder)
+    lens = {"a": 1 + seed % 3, "b": 20 + seed % 50, "c": 100 + 7 * (seed % 30), "d": 2 + seed % 60}
+    reqs = {rid: tt.random_tokens(cfg["vocab"], n, seed=seed + ord(rid)) for rid, n in lens.items()}
+    want = {rid: plain.logits(cfg, w, toks) for rid, toks in reqs.items()}
+    steps = tt.mixed(reqs, seed=seed)
+    got = tt.run_in_process(make_runner(folder, "float32", tt.peak_tokens(steps), page=(4, 16, 64)[seed % 3]), steps)
+    compare(got, want, reqs, "float32")
+    got = tt.run_in_process(make_runner(folder, "bfloat16", tt.peak_tokens(steps)), steps)
+    rows = [row_error(got[(rid, p)], want[rid][p]) for rid, toks in reqs.items() for p in range(len(toks))]
+    assert sum(rows) / len(rows) < 0.05, f"mean row error {sum(rows) / len(rows):.3e}"
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["a", "c"])
+def test_long_decoding(tmp_path_factory, dtype, name):
+    """A short prompt and 380 tokens one by one: states and filter tails are carried through every step."""
+    folder = make_folder(tmp_path_factory, name)
+    cfg, w = plain.read_folder(folder)
+    toks = tt.random_tokens(cfg["vocab"], 400, seed=4)
+    got = tt.run_in_process(make_runner(folder, dtype, 448), tt.tail_decoded({"r": toks}, tail=380))
+    print(f"mepolix {name} {dtype} long decoding: largest row error "
+          f"{compare(got, {'r': plain.logits(cfg, w, toks)}, {'r': toks}, dtype):.2e}")
+
+
+def test_batches_of_unequal_requests_equal_each_alone(tmp_path_factory):
+    folder = make_folder(tmp_path_factory, "b")
+    cfg, _ = plain.read_folder(folder)
+    reqs = {rid: tt.random_tokens(cfg["vocab"], n, seed=ord(rid)) for rid, n in (("a", 70), ("b", 3), ("c", 41), ("d", 1))}
+    sizes = {"a": [30, 1, 1, 38], "b": [1, 2], "c": [2, 39], "d": [1]}
+    alone = {}
+    for rid, toks in reqs.items():
+        r = make_runner(folder, "float32", 256)
+        alone.update(tt.run_in_process(r, tt.portions({rid: toks}, sizes=tuple(sizes[rid]))))
+    steps, at = [], {rid: 0 for rid in reqs}
+    for k in range(4):
+        entries, end = [], []
+        for rid, toks in reqs.items():
+            if k < len(sizes[rid]):
+                n = sizes[rid][k]
+                entries.append({"id": rid, "tokens": toks[at[rid]:at[rid] + n], "want": list(range(n))})
+                at[rid] += n
+                if at[rid] == len(toks):
+                    end.append(rid)
+        steps.append({"step": k, "entries": entries, "end": end})
+    together = tt.run_in_process(make_runner(folder, "float32", 256), steps)
+    for key, row in alone.items():
+        assert row_error(together[key], row) < 2e-5
+
+
+# ------------------------------------------------------------------ generation and the programs
+def test_greedy_generation_through_the_engine(tmp_path_factory):
+    from return_amd import SamplingParams
+    from return_amd.engine import Engine
+    for name in ("a", "c"):
+        folder = make_folder(tmp_path_factory, name)
+        cfg, w = plain.read_folder(folder)
+        prompts = [tt.random_tokens(cfg["vocab"], n, seed=n) for n in (1, 8, 31, 64, 90)]
+        want = [plain.greedy(cfg, w, p, 10) for p in prompts]
+        for graphs in (False, True):
+            eng = Engine(folder, dtype="float32", page_size=16, max_token=1024, max_reside=4, max_step_tokens=64,
+                         prefill_chunk=24, use_graphs=graphs, check_invariants=True)
+            got = eng.generate(prompts, SamplingParams(temperature=0.0, max_new_tokens=10))
+            assert [r.output_ids for r in got] == want, f"model {name}, graphs {graphs}"
+            assert not eng.runner.cache.live
+
+
+def test_bf16_generation_from_graphs_equals_eager(tmp_path_factory):
+    from return_amd import SamplingParams
+    from return_amd.engine import Engine
+    folder = make_folder(tmp_path_factory, "c")
+    cfg, _ = plain.read_folder(folder)
+    prompts = [tt.random_tokens(cfg["vocab"], n, seed=n) for n in (3, 40, 77)]
+    outs = []
+    for graphs in (False, True):
+        eng = Engine(folder, dtype="bfloat16", page_size=16, max_token=1024, max_reside=4, use_graphs=graphs)
+        outs.append([r.output_ids for r in eng.generate(prompts, SamplingParams(temperature=0.0, max_new_tokens=24))])
+    assert outs[0] == outs[1]
+
+
+def test_command_line_makes_a_model_and_generates(tmp_path):
+    """random-model writes a folder from a config.json alone; generate answers greedy requests as the plain model would
+    and a sampled one with a token among the plain model's first five."""
+    import json
+    import subprocess
+    import sys
+    from tests.mepolix_cases import MEPO_B
+    cfg_path = tmp_path / "config.json"
+    cfg_path.write_text(json.dumps(MEPO_B))
+    folder = str(tmp_path / "model")
+    made = subprocess.run([sys.executable, "-m", "return_amd.cli", "random-model", "--config", str(cfg_path), "--out", folder,
+                           "--seed", "5", "--std", "0.2", "--embedding-std", "0.5"], cwd=tt.ROOT, capture_output=True, text=True,
+                          timeout=300)
+    assert made.returncode == 0, made.stderr
+    cfg, w = plain.read_folder(folder)
+    reqs = [{"session_id": "s0", "prompt_ids": tt.random_tokens(cfg["vocab"], 9, seed=1), "max_new_tokens": 5, "temperature": 0.0},
+            {"session_id": "s1", "prompt_ids": tt.random_tokens(cfg["vocab"], 40, seed=2), "max_new_tokens": 4, "temperature": 0.0},
+            {"session_id": "s2", "prompt_ids": tt.random_tokens(cfg["vocab"], 3, seed=3), "max_new_tokens": 6, "temperature": 0.8,
+             "top_k": 5, "top_p": 0.9}]
+    f = tmp_path / "reqs.jsonl"
+    f.write_text("\n".join(json.dumps(r) for r in reqs))
+    out = subprocess.run([sys.executable, "-m", "return_amd.cli", "generate", "--model", folder, "--dtype", "float32",
+                          "--max-reside", "4", "--max-token", "1024", "--requests", str(f)],
+                         cwd=tt.ROOT, capture_output=True, text=True, timeout=300)
+    assert out.returncode == 0, out.stderr
+    lines = [json.loads(l) for l in out.stdout.strip().splitlines()]
+    assert [l["session_id"] for l in lines] == ["s0", "s1", "s2"]
+    for l, r in zip(lines[:2], reqs[:2]):
+        assert l["output_ids"] == plain.greedy(cfg, w, r["prompt_ids"], r["max_new_tokens"])
+    toks = reqs[2]["prompt_ids"] + lines[2]["output_ids"]
+    lg = plain.logits(cfg, w, toks)
+    for i, tok in enumerate(lines[2]["output_ids"]):
+        assert tok in lg[len(reqs[2]["prompt_ids"]) - 1 + i].topk(5).indices.tolist()
+
+
+def test_trace_program_on_a_model_folder(tmp_path_factory, tmp_path):
+    folder = make_folder(tmp_path_factory, "b")
+    cfg, w = plain.read_folder(folder)
+    reqs = {rid: tt.random_tokens(cfg["vocab"], n, seed=ord(rid)) for rid, n in (("a", 40), ("b", 7), ("c", 90))}
+    steps = tt.mixed(reqs, seed=3, max_live=3)
+    got = tt.run_program(folder, "float32", steps, str(tmp_path), tt.peak_tokens(steps), cfg["vocab"],
+                         env=dict(os.environ))
+    compare(got, {rid: plain.logits(cfg, w, t) for rid, t in reqs.items()}, reqs, "float32")
