@@ -1109,11 +1109,138 @@ def fefulorn(args):
             "measured": peaks, "designs": out}
 
 
+# The Mepolix design beside the Kofipel design at equal sizes: --workload mepolix
+def mepolix_shape(width, heads, kv_heads, head_dim, ff, layers, vocab, block=128):
+    """config.json of a Mepolix model of `layers` layers, three delta-rule layers to one with an attention and a channel
+    recurrence (as wide as the stream, blocks of `block` channels) side by side, a dense feed-forward in every layer."""
+    mlp = {"kind": "dense", "ff": ff}
+    delta = {"type": "delta", "mlp": mlp,
+             "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "conv": 4}}
+    both = {"type": "parallel", "mlp": mlp,
+            "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+                               "rot": {"base": 1e6, "dims": head_dim,
+                                       "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}},
+                      "right": {"width": width, "blocks": width // block, "conv": 4}, "left_scale": 0.8, "right_scale": 1.2}}
+    return {"architecture": "Mepolix", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+            "layers": [both if i % 4 == 3 else delta for i in range(layers)]}
+
+
+def _mepolix_mixer_weights(layer, W):
+    """Elements of a mixer's matrices."""
+    m = layer["mixer"]
+    if layer["type"] == "delta":
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        return (2 * G * D + 2 * H * V + 2 * H) * W + W * H * V
+    a, r = m["left"], m["right"]
+    H, G, D, V = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+    return ((H + G) * D + G * V) * W + W * H * V + 3 * W * r["width"] + 2 * r["width"] * (r["width"] // r["blocks"])
+
+
+def mepolix_bytes(raw, elt, batch, ctx):
+    """Bytes one decode step has to move: every matrix once, the keys and values, every state read and written, the head."""
+    W = raw["width"]
+    total = raw["vocab"] * W * elt
+    for layer in raw["layers"]:
+        m = layer["mixer"]
+        total += _mepolix_mixer_weights(layer, W) * elt
+        if layer["type"] == "delta":
+            total += batch * 2 * m["heads"] * m["dim"] * m["vdim"] * 4
+        else:
+            total += batch * (ctx * m["left"]["kv_heads"] * (m["left"]["dim"] + m["left"]["vdim"]) * elt + 2 * m["right"]["width"] * 4)
+        total += 3 * W * layer["mlp"]["ff"] * elt
+    return total
+
+
+def mepolix_flops(raw, T):
+    """Operations of a prompt of T tokens: the products and the attention, and the recurrences (the delta rule per token
+    and head 6 D V, on the vector units in 32-bit)."""
+    W = raw["width"]
+    lin = raw["vocab"] * W / T
+    attn = rec = 0.0
+    for layer in raw["layers"]:
+        m = layer["mixer"]
+        lin += _mepolix_mixer_weights(layer, W) + 3 * W * layer["mlp"]["ff"]
+        if layer["type"] == "delta":
+            rec += 6.0 * T * m["heads"] * m["dim"] * m["vdim"]
+        else:
+            attn += T * (T + 1) / 2 * m["left"]["heads"] * 2.0 * (m["left"]["dim"] + m["left"]["vdim"])
+            rec += 2.0 * T * m["right"]["width"]
+    return 2.0 * T * lin + attn, rec
+
+
+def mepolix(args):
+    """Prefill of 2,048 tokens and decode at batch 1, 8 and 64 over 2,048-token prefixes of the Mepolix design at two
+    sizes that resemble a model's layers (eight layers, random weights), each beside the Kofipel design (the closest one
+    here: three delta-rule layers to one attention layer) with the same width, heads, feed-forward width and layer
+    count and every key in its window, through the same engine; the step's time by kernel for both. value: Mepolix decode
+    tok/s at batch 8 on the larger size."""
+    import torch
+    from return_amd.engine.runner import StepEntry
+    elt = 2 if args.dtype == "bfloat16" else 4
+    layers, vocab = 8, 32000
+    sizes = {"w2048": dict(width=2048, heads=16, kv_heads=4, head_dim=128, ff=8192),
+             "w4096": dict(width=4096, heads=32, kv_heads=8, head_dim=128, ff=12288)}
+    k, w = max(8, min(args.steps, 32)), min(args.warmup, 4)
+    out, peaks = {}, None
+    for tag, sz in sizes.items():
+        raws = {"mepolix": (mepolix_shape(layers=layers, vocab=vocab, **sz), mepolix_flops, mepolix_bytes),
+                "kofipel": (kofipel_shape(layers=layers, vocab=vocab, window=8192, keep_first=0, **sz), kofipel_flops, kofipel_bytes)}
+        for design, (raw, flops_of, bytes_of) in raws.items():
+            cfg, runner = build_runner(0, args.dtype, 64, raw=raw, std=0.02, use_graphs=not args.no_graphs,
+                                       tune_products=not args.no_tune, defer_norms=not args.no_defer_norms)
+            if peaks is None:
+                peaks = measured_peaks(runner, args.dtype)
+            rec = {}
+            toks = [(7 * i + 3) % vocab for i in range(PREFILL_TOKENS)]
+
+            def prompt():
+                runner.add_request("p")
+                runner.step([StepEntry("p", toks, [PREFILL_TOKENS - 1])])
+                runner.free_request("p")
+            prompt()
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            for _ in range(3):
+                prompt()
+            torch.cuda.synchronize()
+            secs = (time.perf_counter() - t0) / 3
+            mfma, vector = flops_of(raw, PREFILL_TOKENS)
+            rec["prefill_2048"] = prefill_record(cfg, args.dtype, PREFILL_TOKENS, secs, peaks=peaks, flops=mfma)
+            rec["prefill_2048"]["recurrence_GFLOP_fp32"] = round(vector / 1e9, 1)
+            rec["prefill_2048"]["kernels"] = kernel_split(prompt, 2)
+            for b in (1, 8, 64):
+                ids = seat_requests(runner, b, CONTEXT)
+                secs = decode_steps(runner, ids, k, w, vocab)
+                ms = secs / k * 1e3
+                point = {"tok_s": round(b * k / secs, 1), "ms_per_step": round(ms, 4)}
+                got = bytes_of(raw, elt, b, CONTEXT + w + (k + 1) // 2) / (ms * 1e-3) / 1e9
+                point.update({"bound": "hbm", "achieved": round(got, 1), "frac": round(got / PEAK_HBM_GBS, 4),
+                              "frac_of_measured": round(got / peaks["read_GBs"], 4)})
+
+                def one_step():
+                    t = runner.decode_launch(ids, None, [0.0] * b, [0] * b, [1.0] * b, [0.0] * b, feed_rows=list(range(b)))
+                    runner.decode_collect(t)
+                point["kernels"] = kernel_split(one_step, 4)
+                release(runner, ids)
+                rec[f"decode_b{b}"] = point
+            out[f"{design}_{tag}"] = rec
+            del runner
+            torch.cuda.empty_cache()
+    head = out["mepolix_w4096"]["decode_b8"]
+    return {"metric": "decode tok/s (Mepolix design, width 4096, 8 layers, random weights)", "value": head["tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": k, "warmup": w, "ms_per_step": head["ms_per_step"],
+            "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic",
+            "config": {"model": "Mepolix and Kofipel designs at equal sizes", "layers": layers, "vocab": vocab,
+                       "sizes": sizes, "global_batch": 8, "seq_len": CONTEXT, "parallelism": "single GPU"},
+            "measured": peaks, "designs": out}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--workload", default="decode_8b",
                     choices=["decode_8b", "continuous_4b", "long_32b", "contexts_8b", "products_8b", "decode_4b",
-                             "decode_32b", "kofipel", "rupezen", "safilorn", "fefulorn"],
+                             "decode_32b", "kofipel", "rupezen", "safilorn", "fefulorn", "mepolix"],
                     help="decode_8b: the headline run; the others: the 4B and 32B shapes with their own "
                          "workloads (one JSON line each, other fields)")
     ap.add_argument("--gpus", type=int, default=1)
@@ -1147,7 +1274,7 @@ def main():
         return 1
     if args.workload != "decode_8b":
         print(json.dumps({"continuous_4b": continuous_4b, "long_32b": long_32b,
-                          "contexts_8b": contexts_8b, "products_8b": products_8b, "kofipel": kofipel, "rupezen": rupezen, "safilorn": safilorn, "fefulorn": fefulorn,
+                          "contexts_8b": contexts_8b, "products_8b": products_8b, "kofipel": kofipel, "rupezen": rupezen, "safilorn": safilorn, "fefulorn": fefulorn, "mepolix": mepolix,
                           "decode_4b": lambda a: decode_shape(a, QWEN3_4B, "Qwen3-4B", 0.02),
                           "decode_32b": lambda a: decode_shape(a, QWEN3_32B, "Qwen3-32B", 0.01)}[args.workload](args)))
         return 0
