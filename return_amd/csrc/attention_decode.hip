@@ -92,8 +92,10 @@ struct DecodeExtras {
 // are multiplied by after the sink has entered (their scale, the result's factor and 1 / denominator).
 __device__ __forceinline__ float decode_finish(float mx, float l, const DecodeExtras& ex, int head) {
     float rescale = 1.f;
-    if (ex.sink) {
-        const float sl = ex.sink_logit != nullptr ? ex.sink_logit[head] * 1.44269504088896340736f : 0.f;
+    if (ex.sink && ex.sink_logit == nullptr) {
+        l += __builtin_amdgcn_exp2f(-mx);                // the key of score 0 without a value
+    } else if (ex.sink) {                                // one with a score of its own, which may be far above the others
+        const float sl = ex.sink_logit[head] * 1.44269504088896340736f;
         const float top = fmaxf(mx, sl);
         rescale = __builtin_amdgcn_exp2f(mx - top);
         l = fmaf(l, rescale, __builtin_amdgcn_exp2f(sl - top));

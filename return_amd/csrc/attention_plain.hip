@@ -258,8 +258,10 @@ __global__ __launch_bounds__(WAVES * 64) void attn_plain_kernel(
                 num = fmaf(acc_s[(w * QR + r) * D + e], ew, num);
                 den = fmaf(ml_s[(w * QR + r) * 2 + 1], ew, den);
             }
-            if (sink) {                                  // one more key that has no value
-                const float sl = sink_logit != nullptr ? sink_logit[head] : 0.f;
+            if (sink && sink_logit == nullptr) {
+                den += expf(-mm);                        // one more key of score 0 that has no value
+            } else if (sink) {                           // one with a score of its own, which may be far above the others
+                const float sl = sink_logit[head];
                 const float top = fmaxf(mm, sl), ew = (mm == -INFINITY) ? 0.f : expf(mm - top);
                 num *= ew;
                 den = fmaf(den, ew, expf(sl - top));

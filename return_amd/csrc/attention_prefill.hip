@@ -439,8 +439,10 @@ __global__ __launch_bounds__(256 * KSPLIT) __attribute__((amdgpu_waves_per_eu(2)
         float inv;
         if constexpr (XT != 0) {
             float rescale = 1.f;
-            if (sink) {                                  // the key without a value
-                const float sl = sink_logit != nullptr ? sink_logit[head] : 0.f;
+            if (sink && sink_logit == nullptr) {
+                l_run[qg] += __builtin_amdgcn_exp2f(-m_run[qg] * scale2);            // the key of score 0 without a value
+            } else if (sink) {                           // one with a score of its own, which may be far above the others
+                const float sl = sink_logit[head];
                 const float top = fmaxf(m_run[qg], sl);
                 rescale = __builtin_amdgcn_exp2f((m_run[qg] - top) * scale2);
                 l_run[qg] = fmaf(l_run[qg], rescale, __builtin_amdgcn_exp2f((sl - top) * scale2));

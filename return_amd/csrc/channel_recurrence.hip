@@ -48,12 +48,12 @@ struct LruStep {                 // what a step of single tokens needs beyond th
     int width_out;
 };
 
-#define LRU_WAVES 4
+// (one wave a workgroup while the waves are few, four otherwise)
 template <int RT, bool STEP>
-__global__ __launch_bounds__(64 * LRU_WAVES) void lru_gates_mfma_kernel(
+__global__ __launch_bounds__(256) void lru_gates_mfma_kernel(
     const bf16* __restrict__ u, const bf16* __restrict__ w, const float* __restrict__ bias, const float* __restrict__ rate,
     float* __restrict__ a_out, float* __restrict__ x_out, int T_tokens, int width, int bw, int n_tiles, LruStep sx) {
-    const int tile = blockIdx.x * LRU_WAVES + (threadIdx.x >> 6);
+    const int tile = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
     if (tile >= n_tiles) return;                         // (no barrier in this kernel)
     const int lane = threadIdx.x & 63, n = lane & 15, g = lane >> 4;
     const int per_block = (bw + 15) / 16;
@@ -66,6 +66,28 @@ __global__ __launch_bounds__(64 * LRU_WAVES) void lru_gates_mfma_kernel(
     const bf16* ur[RT];
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) ur[rt] = u + (size_t)min(t0 + rt * 16 + n, T_tokens - 1) * width + (size_t)b * bw;
+    // lane (n, g) of the results: row n of each group of 16, channels 4g .. 4g + 3 of the tile. What the epilogue reads
+    // is asked for here, so that it arrives with the operands.
+    const bool ch_ok = c0 + 4 * g < bw;
+    const int ch = b * bw + (ch_ok ? c0 + 4 * g : 0);
+    const float4_t rb = *reinterpret_cast<const float4_t*>(bias + ch);
+    const float4_t ib = *reinterpret_cast<const float4_t*>(bias + width + ch);
+    const float4_t ra = *reinterpret_cast<const float4_t*>(rate + ch);
+    [[maybe_unused]] float4_t yb, st[RT];
+    [[maybe_unused]] uint2 yw[RT];
+    [[maybe_unused]] float* Sp[RT];
+    uint2 uw[RT];
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        const int t = min(t0 + rt * 16 + n, T_tokens - 1);
+        uw[rt] = *reinterpret_cast<const uint2*>(u + (size_t)t * width + ch);
+        if constexpr (STEP) {
+            yw[rt] = *reinterpret_cast<const uint2*>(sx.y + (size_t)t * sx.ld_y + ch);
+            Sp[rt] = sx.S + (size_t)sx.slot_ids[t] * width + ch;
+            st[rt] = *reinterpret_cast<const float4_t*>(Sp[rt]);
+        }
+    }
+    if constexpr (STEP) yb = *reinterpret_cast<const float4_t*>(sx.y_bias + ch);
     float4_t accr[RT], acci[RT];
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) accr[rt] = acci[rt] = float4_t{0.f, 0.f, 0.f, 0.f};
@@ -98,19 +120,13 @@ __global__ __launch_bounds__(64 * LRU_WAVES) void lru_gates_mfma_kernel(
             }
         }
     }
-    if (c0 + 4 * g >= bw) return;
-    // lane (n, g): row n of each group of 16, channels 4g .. 4g + 3 of the tile
-    const int ch = b * bw + c0 + 4 * g;
-    const float4_t rb = *reinterpret_cast<const float4_t*>(bias + ch);
-    const float4_t ib = *reinterpret_cast<const float4_t*>(bias + width + ch);
-    const float4_t ra = *reinterpret_cast<const float4_t*>(rate + ch);
+    if (!ch_ok) return;
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
         const int t = t0 + rt * 16 + n;
         if (t >= T_tokens) continue;
-        const uint2 uw = *reinterpret_cast<const uint2*>(u + (size_t)t * width + ch);
-        const float uf[4] = {__uint_as_float(uw.x << 16), __uint_as_float(uw.x & 0xffff0000u), __uint_as_float(uw.y << 16),
-                             __uint_as_float(uw.y & 0xffff0000u)};
+        const float uf[4] = {__uint_as_float(uw[rt].x << 16), __uint_as_float(uw[rt].x & 0xffff0000u),
+                             __uint_as_float(uw[rt].y << 16), __uint_as_float(uw[rt].y & 0xffff0000u)};
         float4_t a4, x4;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
@@ -120,19 +136,16 @@ __global__ __launch_bounds__(64 * LRU_WAVES) void lru_gates_mfma_kernel(
             x4[e] = x;
         }
         if constexpr (STEP) {
-            float* Sp = sx.S + (size_t)sx.slot_ids[t] * width + ch;
-            const uint2 yw = *reinterpret_cast<const uint2*>(sx.y + (size_t)t * sx.ld_y + ch);
-            const float yf[4] = {__uint_as_float(yw.x << 16), __uint_as_float(yw.x & 0xffff0000u),
-                                 __uint_as_float(yw.y << 16), __uint_as_float(yw.y & 0xffff0000u)};
-            const float4_t yb = *reinterpret_cast<const float4_t*>(sx.y_bias + ch);
-            float4_t s4 = *reinterpret_cast<const float4_t*>(Sp);
+            const float yf[4] = {__uint_as_float(yw[rt].x << 16), __uint_as_float(yw[rt].x & 0xffff0000u),
+                                 __uint_as_float(yw[rt].y << 16), __uint_as_float(yw[rt].y & 0xffff0000u)};
+            float4_t s4 = st[rt];
             float o[4];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 s4[e] = fmaf(a4[e], s4[e], x4[e]);
                 o[e] = s4[e] * lru_gelu(yf[e] + yb[e]) * sx.out_scale;
             }
-            *reinterpret_cast<float4_t*>(Sp) = s4;
+            *reinterpret_cast<float4_t*>(Sp[rt]) = s4;
             uint2 ow;
             ow.x = (uint32_t)f2bf_bits(o[0]) | ((uint32_t)f2bf_bits(o[1]) << 16);
             ow.y = (uint32_t)f2bf_bits(o[2]) | ((uint32_t)f2bf_bits(o[3]) << 16);
@@ -323,10 +336,13 @@ extern "C" int ra_channel_recurrence(const void* u, const void* w, const float* 
     if (!step && scratch == nullptr) return RA_ERR_ARG;
     if (mfma) {
         const int n_tiles = blocks * ((bw + 15) / 16);
-        const int rt = T_tokens <= 16 ? 1 : T_tokens <= 32 ? 2 : 4;
+        // as many rows a wave as still leave enough waves for the chip
+        int rt = 1;
+        while (rt < 4 && (long long)n_tiles * ((T_tokens + 32 * rt - 1) / (32 * rt)) >= 2048 && T_tokens > 16 * rt) rt *= 2;
         const int row_tiles = (T_tokens + 16 * rt - 1) / (16 * rt);
         if (row_tiles > 65535) return RA_ERR_ARG;
-        dim3 grid((n_tiles + LRU_WAVES - 1) / LRU_WAVES, row_tiles), block(64 * LRU_WAVES);
+        const int waves = (long long)n_tiles * row_tiles <= 1024 ? 1 : 4;
+        dim3 grid((n_tiles + waves - 1) / waves, row_tiles), block(64 * waves);
 #define LRU_GO(RT_, STEP_)                                                                                            \
     hipLaunchKernelGGL((lru_gates_mfma_kernel<RT_, STEP_>), grid, block, 0, st, (const bf16*)u, (const bf16*)w, bias, rate, \
                        a, x, T_tokens, width, bw, n_tiles, sx)

@@ -333,6 +333,11 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
         constexpr int ROWS = DR_BATCH / EPL;                // rows a wave asks for at once
         for (int t0 = fw; t0 < nt; t0 += (DR_FEEDERS / 64) * ROWS) {
             float fq[ROWS][EPL], fk[ROWS][EPL], fa[ROWS][EPL];
+            // (rules 2 and 3: lane m asks for the step of the batch's row m and forms that row's decay)
+            float step_m = 0.f;
+            const int t_m = t0 + lane * (DR_FEEDERS / 64);
+            const bool has_m = rule >= 2 && lane < ROWS && t_m < nt;
+            if (has_m) step_m = to_f(ag[(size_t)(base + c0 + t_m) * ld_ag + h]) + dt_bias[h];
 #pragma unroll
             for (int m = 0; m < ROWS; ++m) {
                 const int tt = t0 + m * (DR_FEEDERS / 64);
@@ -344,8 +349,8 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                         const T* row = qkv + (size_t)(base + c0 + tt) * ld_qkv;
                         fq[m][e] = to_f(row[kvh * D + i]);
                         fk[m][e] = to_f(row[G * D + kvh * D + i]);
-                        fa[m][e] = rule >= 2 ? to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h]) + dt_bias[h]
-                                   : a_sign * (to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h * D + i]) + dt_bias[h * D + i]);
+                        if (rule < 2)
+                            fa[m][e] = a_sign * (to_f(ag[(size_t)(base + c0 + tt) * ld_ag + h * D + i]) + dt_bias[h * D + i]);
                     }
                 }
             }
@@ -353,6 +358,7 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                 feed_values();                               // behind the first batch's loads: all on their way together
                 values_done = true;
             }
+            const float decay_m = has_m ? expf(neg_a * dr_softplus_exact(step_m)) : 1.f;
 #pragma unroll
             for (int m = 0; m < ROWS; ++m) {
                 const int tt = t0 + m * (DR_FEEDERS / 64);
@@ -365,8 +371,8 @@ __global__ __launch_bounds__(DR_WALKERS + DR_FEEDERS) __attribute__((amdgpu_wave
                 }
                 sk = (rule == 1 || rule == 2) ? 1.f : 1.0f / sqrtf(dr_wave_sum(sk) + 1e-6f);
                 sq = (rule == 1 || rule == 2) ? q_scale : q_scale / sqrtf(dr_wave_sum(sq) + 1e-6f);
-                // (rules 2 and 3: one decay for the whole row; lanes with an element of the row hold its step in fa[m][0])
-                const float row_decay = (rule >= 2 && lane < D) ? expf(neg_a * dr_softplus_exact(fa[m][0])) : 1.f;
+                // (rules 2 and 3: one decay for the whole row)
+                const float row_decay = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(decay_m), m));
 #pragma unroll
                 for (int e = 0; e < EPL; ++e) {
                     const int i = lane + 64 * e;

@@ -232,6 +232,68 @@ __global__ void qkv_blend_prepare_kernel(const T* __restrict__ qkv, long long ld
     for (int c = R + lane; c < D; c += 64) dst[c] = from_f<T>(normed(c));
 }
 
+// The same without biases and blending, for heads of D = 64, 128, 256 or 512 elements that turn wholly or not at all:
+// D / 8 neighbouring lanes share a head, each with four neighbours of its first half and the four they turn with, so a
+// wave takes 512 / D heads of a token, reads and writes 8 or 16 bytes a lane, and sums the squares by lane moves.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void qkv_heads_prepare_kernel(const T* __restrict__ qkv, long long ld_qkv, int Hq, int Hkv,
+                                                                const float* __restrict__ w_q, const float* __restrict__ w_k,
+                                                                int Dn, float eps, const int* __restrict__ positions,
+                                                                const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+                                                                T* __restrict__ q_out, T* __restrict__ k_pool,
+                                                                T* __restrict__ v_pool, const int* __restrict__ slots, int P,
+                                                                long long pool_rows, long long n_rows) {
+    constexpr int D = 8 * LPH, HALF = 4 * LPH;
+    const long long row = ((long long)blockIdx.x * 256 + threadIdx.x) / LPH;
+    const int l = threadIdx.x % LPH;
+    const int heads = Hq + 2 * Hkv;
+    const bool live = row < n_rows;                          // (every lane stays for the sums)
+    const int t = live ? (int)(row / heads) : 0, head = live ? (int)(row % heads) : 0;
+    const T* src = qkv + (size_t)t * ld_qkv + (size_t)head * D;
+    float4 a = pr_load4(src + 4 * l), b = pr_load4(src + HALF + 4 * l);
+    const bool value = head >= Hq + Hkv;
+    T* dst = nullptr;
+    if (live) {
+        if (head < Hq) {
+            dst = q_out + ((size_t)t * Hq + head) * D;
+        } else if (k_pool != nullptr) {
+            const long long s = slots[t];
+            if (s >= 0 && s < pool_rows)
+                dst = (value ? v_pool : k_pool) + ra_cache_offset(s, value ? head - Hq - Hkv : head - Hq, Hkv, P, D);
+        }
+    }
+    const float* wn = head < Hq ? w_q : w_k;
+    const bool turn = cos_t != nullptr;
+    const float4 one = make_float4(1.f, 1.f, 1.f, 1.f), zero = make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 wa = one, wb = one, cs = one, sn = zero;
+    if (wn != nullptr) {
+        wa = pr_load4(wn + 4 * l);
+        wb = pr_load4(wn + HALF + 4 * l);
+    }
+    if (turn) {
+        const size_t at = (size_t)positions[t] * HALF + 4 * l;
+        cs = pr_load4(cos_t + at);
+        sn = pr_load4(sin_t + at);
+    }
+    float ss = fmaf(a.x, a.x, fmaf(a.y, a.y, fmaf(a.z, a.z, a.w * a.w)));
+    ss += fmaf(b.x, b.x, fmaf(b.y, b.y, fmaf(b.z, b.z, b.w * b.w)));
+#pragma unroll
+    for (int o = 1; o < LPH; o <<= 1) ss += __shfl_xor(ss, o, 64);
+    if (dst == nullptr) return;
+    if (!value) {
+        const float rstd = wn != nullptr ? 1.0f / sqrtf(ss / (float)Dn + eps) : 1.f;
+        a = make_float4(a.x * rstd * wa.x, a.y * rstd * wa.y, a.z * rstd * wa.z, a.w * rstd * wa.w);
+        b = make_float4(b.x * rstd * wb.x, b.y * rstd * wb.y, b.z * rstd * wb.z, b.w * rstd * wb.w);
+        if (turn) {
+            const float4 u = a, v = b;
+            a = make_float4(u.x * cs.x - v.x * sn.x, u.y * cs.y - v.y * sn.y, u.z * cs.z - v.z * sn.z, u.w * cs.w - v.w * sn.w);
+            b = make_float4(v.x * cs.x + u.x * sn.x, v.y * cs.y + u.y * sn.y, v.z * cs.z + u.z * sn.z, v.w * cs.w + u.w * sn.w);
+        }
+    }
+    pr_store4(dst + 4 * l, a);
+    pr_store4(dst + HALF + 4 * l, b);
+}
+
 extern "C" int ra_qkv_blend_prepare(const void* qkv, long long ld_qkv, int T_tokens, int Hq, int Hkv, int D,
                                     const float* bias, const float* w_q, const float* w_k, int Dn, float eps,
                                     const int* positions, const float* cos_t, const float* sin_t, int R, void* q_out,
@@ -247,6 +309,25 @@ extern "C" int ra_qkv_blend_prepare(const void* qkv, long long ld_qkv, int T_tok
     const long long n_rows = (long long)T_tokens * (Hq + 2 * Hkv);
     dim3 block(256), grid((unsigned)((n_rows + 3) / 4));
     hipStream_t st = (hipStream_t)stream;
+    const auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    if (bias == nullptr && mode == 0 && (R == 0 || R == D) && (D == 64 || D == 128 || D == 256 || D == 512) && ld_qkv % 4 == 0 &&
+        aligned(qkv) && aligned(q_out) && aligned(k_pool) && aligned(v_pool) && aligned(w_q) && aligned(w_k) &&
+        aligned(cos_t) && aligned(sin_t) && (dtype == RA_DTYPE_F32 || dtype == RA_DTYPE_BF16)) {
+        dim3 hgrid((unsigned)((n_rows * (D / 8) + 255) / 256));
+#define QKV_HEADS(T_, LPH_)                                                                                            \
+    hipLaunchKernelGGL((qkv_heads_prepare_kernel<T_, LPH_>), hgrid, block, 0, st, (const T_*)qkv, ld_qkv, Hq, Hkv, w_q, w_k, \
+                       Dn, eps, positions, R ? cos_t : nullptr, R ? sin_t : nullptr, (T_*)q_out, (T_*)k_pool,         \
+                       (T_*)v_pool, slots, P, pool_rows, n_rows)
+#define QKV_HEADS_D(T_)                                                                                                \
+    do {                                                                                                               \
+        if (D == 64) QKV_HEADS(T_, 8); else if (D == 128) QKV_HEADS(T_, 16);                                           \
+        else if (D == 256) QKV_HEADS(T_, 32); else QKV_HEADS(T_, 64);                                                  \
+    } while (0)
+        if (dtype == RA_DTYPE_F32) QKV_HEADS_D(float); else QKV_HEADS_D(bf16);
+#undef QKV_HEADS_D
+#undef QKV_HEADS
+        return ra_launch_status();
+    }
     if (dtype == RA_DTYPE_F32)
         hipLaunchKernelGGL(qkv_blend_prepare_kernel<float>, grid, block, 0, st, (const float*)qkv, ld_qkv, Hq, Hkv, D, bias, w_q, w_k, Dn, eps,
                            positions, cos_t, sin_t, R, (float*)q_out, (float*)k_pool, (float*)v_pool, slots, P, pool_rows,

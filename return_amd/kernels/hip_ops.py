@@ -1431,7 +1431,7 @@ class HipOps:
                 raise KernelError(f"attention: sink logits {tuple(sink_logit.shape)} for {n_q} heads")
             sink = True
         fine_weights = bool(fine_weights)
-        if q.dtype == torch.bfloat16 and (ld_out % 4 or out.data_ptr() % 8):
+        if q.dtype == torch.bfloat16 and D % 16 == 0 and D <= 256 and (ld_out % 4 or out.data_ptr() % 8):
             raise KernelError(f"attention: output rows {ld_out} elements apart, or not aligned to four elements")
         extras = head_scale is not None or softcap > 0.0 or keep_first > 0 or sink or out_scale != 1.0 or fine_weights \
             or ld_out != n_q * D

@@ -69,7 +69,9 @@ def test_soft_cap(ops):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("Hq,Hkv,D,Dn,R,P,T", [(4, 2, 16, 12, 8, 16, 37), (3, 3, 10, 10, 10, 4, 5), (8, 1, 64, 32, 32, 16, 70),
-                                               (2, 2, 12, 5, 0, 8, 1), (5, 5, 128, 128, 64, 16, 19), (6, 2, 80, 66, 2, 32, 33)])
+                                               (2, 2, 12, 5, 0, 8, 1), (5, 5, 128, 128, 64, 16, 19), (6, 2, 80, 66, 2, 32, 33),
+                                               (4, 2, 64, 64, 64, 16, 37), (3, 1, 128, 100, 0, 8, 21), (5, 1, 128, 128, 128, 16, 1),
+                                               (6, 2, 256, 256, 256, 4, 9), (2, 1, 512, 512, 0, 16, 5)])
 def test_preparation_with_head_norms_and_no_biases(ops, ref, dtype, Hq, Hkv, D, Dn, R, P, T):
     """Rows are columns of wider rows; what a head has beyond its true width is zero."""
     n = (Hq + 2 * Hkv) * D
