@@ -25,6 +25,10 @@ Interfaces (``rt`` is the return_amd.parts.runtime.Runtime of the engine):
                 forward(x, step, cache) -> y      x, y: [T, H] compute dtype
                     step: return_amd.engine.batch.StepBatch; cache: the view the cache
                     manager gives for this call's cache layer (None without cache_spec)
+                optional, for a mixer that can be one side of several on the same input (mixer "side_by_side"):
+                with params inner = True it notes no products of its own; take_products() -> (first weight,
+                output projection), in_width / out_width their outer sizes; run(z, step, cache, write_cache, out,
+                out_scale) does what lies between them, z and out being columns of wider rows
   feed_forward  forward(x, step) -> y
 
   Optional, for a mixer or feed-forward whose input goes into ONE product and whose output comes out
