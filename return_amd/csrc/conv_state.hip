@@ -20,9 +20,10 @@
 #include "common.h"
 
 #define CONV_SEG 16
-#define CONV_MAX_TAPS 8
+#define CONV_MAX_TAPS 17       // taps - 1 inputs must fit one segment
 
-template <typename T>
+// MT: the most taps of this instantiation (4, 8 or CONV_MAX_TAPS)
+template <typename T, int MT>
 __global__ __launch_bounds__(256) void causal_conv_kernel(
     const T* __restrict__ x, long long ld_x, const float* __restrict__ w, T* __restrict__ tail,
     const int* __restrict__ cu_q, const int* __restrict__ slot_ids, T* __restrict__ out, long long ld_out,
@@ -44,9 +45,9 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
         const float v = to_f(x[(size_t)(base + li) * ld_x + c]);
         return in_bias != nullptr ? round_to<T>(v + bi) : v;
     };
-    float wt[CONV_MAX_TAPS], win[CONV_MAX_TAPS], old[CONV_MAX_TAPS];
+    float wt[MT], win[MT], old[MT];
 #pragma unroll
-    for (int j = 0; j < CONV_MAX_TAPS; ++j) {
+    for (int j = 0; j < MT; ++j) {
         wt[j] = j < taps ? w[(size_t)c * taps + j] : 0.f;
         win[j] = old[j] = 0.f;
         if (j < back) {
@@ -59,32 +60,32 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
         const float cur = input(li);
         float y = b0;
 #pragma unroll
-        for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+        for (int j = 0; j < MT - 1; ++j)
             if (j < back) y = fmaf(wt[j], win[j], y);
 #pragma unroll
-        for (int j = 0; j < CONV_MAX_TAPS; ++j)
+        for (int j = 0; j < MT; ++j)
             if (j == back) y = fmaf(wt[j], cur, y);
         if (flags & 1) y += cur;
         if (flags & 2) y = y / (1.f + expf(-y));
         out[(size_t)(base + li) * ld_out + c] = from_f<T>(y);
 #pragma unroll
-        for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+        for (int j = 0; j < MT - 1; ++j)
             if (j + 1 < back) win[j] = win[j + 1];
 #pragma unroll
-        for (int j = 0; j < CONV_MAX_TAPS; ++j)
+        for (int j = 0; j < MT; ++j)
             if (j == back - 1) win[j] = cur;
     }
     if (first == 0) {
         // the new tail: the last taps-1 inputs of (old tail, this step's rows)
 #pragma unroll
-        for (int j = 0; j < CONV_MAX_TAPS - 1; ++j) {
+        for (int j = 0; j < MT - 1; ++j) {
             if (j < back) {
                 const int li = q_len - back + j;
                 float v = 0.f;
                 if (li >= 0) v = input(li);
                 else {
 #pragma unroll
-                    for (int k = 0; k < CONV_MAX_TAPS - 1; ++k)
+                    for (int k = 0; k < MT - 1; ++k)
                         if (k == back + li) v = old[k];
                 }
                 my_tail[(size_t)j * C] = from_f<T>(v);
@@ -102,12 +103,16 @@ static int causal_conv_run(const void* x, long long ld_x, const float* in_bias, 
     if (n_seqs > 65535 || (C + 255) / 256 > 65535) return RA_ERR_ARG;
     if (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16) return RA_ERR_ARG;
     dim3 grid((max_q_len + CONV_SEG - 1) / CONV_SEG, n_seqs, (C + 255) / 256), block(256);
-    if (dtype == RA_DTYPE_F32)
-        hipLaunchKernelGGL(causal_conv_kernel<float>, grid, block, 0, (hipStream_t)stream, (const float*)x, ld_x, w,
-                           (float*)tail, cu_q, slot_ids, (float*)out, ld_out, C, taps, flags, bias, in_bias);
-    else
-        hipLaunchKernelGGL(causal_conv_kernel<bf16>, grid, block, 0, (hipStream_t)stream, (const bf16*)x, ld_x, w,
-                           (bf16*)tail, cu_q, slot_ids, (bf16*)out, ld_out, C, taps, flags, bias, in_bias);
+#define CONV_GO(T_, MT_)                                                                                                 \
+    hipLaunchKernelGGL((causal_conv_kernel<T_, MT_>), grid, block, 0, (hipStream_t)stream, (const T_*)x, ld_x, w, (T_*)tail, \
+                       cu_q, slot_ids, (T_*)out, ld_out, C, taps, flags, bias, in_bias)
+#define CONV_TAPS(T_)                                                                                                    \
+    do {                                                                                                                 \
+        if (taps <= 4) CONV_GO(T_, 4); else if (taps <= 8) CONV_GO(T_, 8); else CONV_GO(T_, CONV_MAX_TAPS);              \
+    } while (0)
+    if (dtype == RA_DTYPE_F32) CONV_TAPS(float); else CONV_TAPS(bf16);
+#undef CONV_TAPS
+#undef CONV_GO
     return ra_launch_status();
 }
 

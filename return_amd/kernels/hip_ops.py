@@ -677,8 +677,8 @@ class HipOps:
         if tuple(out.shape) != (T, C) or w.shape[0] != C or tuple(tail.shape[1:]) != (taps - 1, C) or T != step.n_tokens:
             raise KernelError(f"causal_conv: x {tuple(x.shape)}, w {tuple(w.shape)}, tail {tuple(tail.shape)}, "
                               f"out {tuple(out.shape)}, step of {step.n_tokens}")
-        if not 1 <= taps <= 8:
-            raise KernelError(f"causal_conv: {taps} taps, the kernel takes 1 to 8")
+        if not 1 <= taps <= 17:
+            raise KernelError(f"causal_conv: {taps} taps, the kernel takes 1 to 17")
         if max(step.slot_ids_host, default=0) >= tail.shape[0]:
             raise KernelError("causal_conv: a request's slot lies beyond the tail's rows")
         if out.data_ptr() == x.data_ptr():

@@ -160,7 +160,8 @@ def test_fine_weights_are_finer(ops, q_len, q_start):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("C,taps,q_lens", [(40, 4, [5, 1, 33]), (300, 2, [1, 1]), (16, 8, [70]), (513, 3, [2, 17, 1]), (24, 1, [3, 20])])
+@pytest.mark.parametrize("C,taps,q_lens", [(40, 4, [5, 1, 33]), (300, 2, [1, 1]), (16, 8, [70]), (513, 3, [2, 17, 1]), (24, 1, [3, 20]),
+                                           (70, 11, [4, 40, 1]), (33, 17, [16, 17, 50])])
 def test_convolution_with_biased_inputs(ops, ref, dtype, C, taps, q_lens):
     """From a tail of zeros (a request's start: zeros, not biased inputs) and on; the tail holds the biased inputs."""
     n, T = len(q_lens), sum(q_lens)
