@@ -21,7 +21,7 @@ import sys
 
 import numpy as np
 
-MAX_LIVE = 8            # default of --max-live: traces keep up to four requests live, with room to spare
+MAX_LIVE = 4            # default of --max-live: traces keep at most four requests live, whose slots are used again
 PAGE_SIZE = 16          # default of --page-size
 ROUND_TO = 64           # a request's token count is rounded up to this for --max-tokens (or to a larger page)
 

@@ -3,7 +3,7 @@
 Sources are return_amd/csrc/*.hip. The library is kept in-tree (return_amd/_lib/); if that
 folder cannot be written, in a per-user folder under the temporary directory. A stored
 hash of sources and flags decides whether what is there is still current, so a fresh
-checkout compiles at its first call and prints a line now and then while it does.
+checkout compiles at its first call and prints a line for every unit it has compiled.
 """
 from __future__ import annotations
 
@@ -14,7 +14,6 @@ import shutil
 import subprocess
 import sys
 import tempfile
-import threading
 import time
 
 ARCH = "gfx950"
@@ -130,13 +129,6 @@ def build(force: bool = True) -> str:
     units = compile_units()
     t0 = time.time()
     _say(f"compiling {len(units)} HIP units for {ARCH} into {out_dir}")
-    done = threading.Event()
-
-    def heartbeat():
-        while not done.wait(15.0):
-            _say(f"still compiling ({time.time() - t0:.0f} s)")
-
-    threading.Thread(target=heartbeat, daemon=True).start()
     try:
         def one(unit):
             src, defines, name = unit
@@ -155,7 +147,6 @@ def build(force: bool = True) -> str:
             f.write(source_hash())
         os.replace(tmp + ".hash", lib + ".hash")
     finally:
-        done.set()
         shutil.rmtree(obj_dir, ignore_errors=True)
     _say(f"built {lib} in {time.time() - t0:.0f} s")
     return lib
