@@ -11,11 +11,13 @@
 // and nothing of it is read or written.
 //
 //   latent_kv_prepare   per token, from the rows z = [a: Q | b: C | r: R | ...] of the first product:
-//                       cq = a / sqrt(mean(a^2) + eps) * wq  (the query's latent, to cq_out),
+//                       cq = a / sqrt(mean(a^2) + eps) * wq  (the query's latent, to cq_out; Q may be 0: no such part),
 //                       c = b / sqrt(mean(b^2) + eps) * wc   (to the value pool's row of the token's slot),
 //                       kr = r with its first `rot` elements turned by the token's position, element i with
-//                       i + rot/2 (to the key pool's row).
-//   latent_q_prepare    qq[t][h] = [q_lat[h][t] | turned q[t][h][D:]]  (q rows are heads of [D | R]).
+//                       i + rot/2 (to the key pool's row). With q (rows of heads of [D | R], ld_q apart) also what
+//                       latent_q_prepare does to the rotated part of every head, in the same pass over the token.
+//   latent_q_prepare    qq[t][h] = [q_lat[h][t] | turned q[t][h][D:]]  (q rows are heads of [D | R]; q_lat null: the
+//                       first C elements are left as they are, a product writes them there itself).
 //   attention_latent_plain   a workgroup per (token, QR heads): the heads of a token read the same rows, so a
 //                       row that is loaded serves QR scores. The waves take the blocks of 64 keys in turn (block b,
 //                       counted from position 0, is wave b % WAVES's), so a row's sums are formed in an order that
@@ -32,17 +34,37 @@ __global__ __launch_bounds__(256) void latent_kv_prepare_kernel(
     const T* __restrict__ z, long long ld_z, int Q, int C, int R, const float* __restrict__ wq,
     const float* __restrict__ wc, float eps, const int* __restrict__ positions, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, int rot, T* __restrict__ cq_out, T* __restrict__ k_pool, T* __restrict__ v_pool,
-    const int* __restrict__ slot_mapping, int P) {
+    const int* __restrict__ slot_mapping, int P, const T* __restrict__ q, long long ld_q, int Hn, int D,
+    T* __restrict__ qq) {
     __shared__ float scratch[16];
     const int t = blockIdx.x, tid = threadIdx.x;
     const T* zr = z + (size_t)t * ld_z;
     float ss = 0.f;
-    for (int i = tid; i < Q; i += 256) {
-        const float a = to_f(zr[i]);
-        ss = fmaf(a, a, ss);
+    if (Q > 0) {
+        for (int i = tid; i < Q; i += 256) {
+            const float a = to_f(zr[i]);
+            ss = fmaf(a, a, ss);
+        }
+        const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)Q + eps);
+        for (int i = tid; i < Q; i += 256) cq_out[(size_t)t * Q + i] = from_f<T>(to_f(zr[i]) * rq * wq[i]);
     }
-    const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)Q + eps);
-    for (int i = tid; i < Q; i += 256) cq_out[(size_t)t * Q + i] = from_f<T>(to_f(zr[i]) * rq * wq[i]);
+    if (q != nullptr) {
+        const int half = rot >> 1, pos = positions[t];
+        const T* qr = q + (size_t)t * ld_q + D;
+        T* dst = qq + (size_t)t * Hn * (C + R) + C;
+        for (int j = tid; j < Hn * R; j += 256) {
+            const int h = j / R, i = j - h * R;
+            const T* src = qr + (size_t)h * (D + R);
+            float v = to_f(src[i]);
+            if (i < rot) {
+                const int f = i < half ? i : i - half;
+                const float cs = cos_t[(size_t)pos * half + f], sn = sin_t[(size_t)pos * half + f];
+                const float other = to_f(src[i < half ? i + half : i - half]);
+                v = i < half ? v * cs - other * sn : v * cs + other * sn;
+            }
+            dst[(size_t)h * (C + R) + i] = from_f<T>(v);
+        }
+    }
     if (v_pool == nullptr) return;
     ss = 0.f;
     for (int i = tid; i < C; i += 256) {
@@ -71,21 +93,23 @@ __global__ __launch_bounds__(256) void latent_kv_prepare_kernel(
 extern "C" int ra_latent_kv_prepare(const void* z, long long ld_z, int T_tokens, int Q, int C, int R, const float* wq,
                                     const float* wc, float eps, const int* positions, const float* cos_t,
                                     const float* sin_t, int rot, void* cq_out, void* k_pool, void* v_pool,
-                                    const int* slot_mapping, int P, int dtype, void* stream) {
+                                    const int* slot_mapping, int P, const void* q, long long ld_q, int Hn, int D, void* qq,
+                                    int dtype, void* stream) {
     if (T_tokens <= 0) return RA_OK;
-    if (Q < 1 || C < 1 || R < 0 || rot < 0 || rot > R || (rot & 1) || ld_z < (long long)Q + C + R || P < 1 ||
+    if (Q < 0 || C < 1 || R < 0 || rot < 0 || rot > R || (rot & 1) || ld_z < (long long)Q + C + R || P < 1 ||
         (rot > 0 && (cos_t == nullptr || sin_t == nullptr)) || (v_pool != nullptr && slot_mapping == nullptr) ||
-        (v_pool != nullptr && R > 0 && k_pool == nullptr))
+        (v_pool != nullptr && R > 0 && k_pool == nullptr) || (Q > 0 && (wq == nullptr || cq_out == nullptr)) ||
+        (q != nullptr && (Hn < 1 || D < 0 || ld_q < (long long)Hn * (D + R) || qq == nullptr || (long long)Hn * R > 0x7fffffffLL)))
         return RA_ERR_ARG;
     hipStream_t st = (hipStream_t)stream;
     if (dtype == RA_DTYPE_F32)
         hipLaunchKernelGGL(latent_kv_prepare_kernel<float>, dim3(T_tokens), dim3(256), 0, st, (const float*)z, ld_z, Q, C, R,
                            wq, wc, eps, positions, cos_t, sin_t, rot, (float*)cq_out, (float*)k_pool, (float*)v_pool,
-                           slot_mapping, P);
+                           slot_mapping, P, (const float*)q, ld_q, Hn, D, (float*)qq);
     else if (dtype == RA_DTYPE_BF16)
         hipLaunchKernelGGL(latent_kv_prepare_kernel<bf16>, dim3(T_tokens), dim3(256), 0, st, (const bf16*)z, ld_z, Q, C, R,
                            wq, wc, eps, positions, cos_t, sin_t, rot, (bf16*)cq_out, (bf16*)k_pool, (bf16*)v_pool,
-                           slot_mapping, P);
+                           slot_mapping, P, (const bf16*)q, ld_q, Hn, D, (bf16*)qq);
     else
         return RA_ERR_ARG;
     return ra_launch_status();
@@ -98,8 +122,10 @@ __global__ __launch_bounds__(256) void latent_q_prepare_kernel(
     T* __restrict__ qq) {
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
     T* dst = qq + ((size_t)t * Hn + h) * (C + R);
-    const T* lat = q_lat + ((size_t)h * T_tokens + t) * C;
-    for (int i = tid; i < C; i += 256) dst[i] = lat[i];
+    if (q_lat != nullptr) {
+        const T* lat = q_lat + ((size_t)h * T_tokens + t) * C;
+        for (int i = tid; i < C; i += 256) dst[i] = lat[i];
+    }
     const T* qr = q + ((size_t)t * Hn + h) * (D + R) + D;
     const int half = rot >> 1, pos = positions[t];
     for (int i = tid; i < R; i += 256) {

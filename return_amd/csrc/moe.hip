@@ -1,18 +1,20 @@
 // Routed feed-forward (mixture of experts): the router's choice, the grouping of (token, choice) pairs by
 // expert, the experts' products over those groups, and the weighted sum.
 //
-//   route     z [T][E] 32-bit router logits -> ids [T][top], weights [T][top]
+//   route     z [T][E] 32-bit router logits (rows ld_z apart) -> ids [T][top], weights [T][top]
 //             s = sigmoid(z) (or softmax-free: only sigmoid is built); choice score c = s + bias (bias may be
 //             null). Experts form n_groups equal groups of neighbours; a group's score is the sum of its two
 //             largest choice scores (its largest, for groups of one); only the keep best groups stay eligible.
 //             The top eligible experts by choice score are taken, largest first (ties: the lower number); the
 //             weights are their s, divided by their sum + norm_eps. Law 2: s = softmax(z) over all experts, the
-//             choice is made on s, a group's score is its largest s, the weights are the chosen s as they are.
+//             choice is made on s, a group's score is its largest s, the weights are the chosen s as they are. Law 3:
+//             as law 0, the weights are the chosen s as they are.
 //   plan      pairs p = t * top + k grouped by expert: order[] lists the pairs expert by expert, and tiles[]
 //             lists (expert, first place in order[], places) for runs of at most `rows` places of one expert.
 //             One workgroup (a counting sort). A pair's result does not depend on its place in a tile.
 //   product   for every tile: y[p] = W_e x[row(p)] with row(p) = p / top (the token's row) or p itself;
-//             gated: W_e = [gate rows; up rows], y = silu(gate) * up. An FMA form for every size and both
+//             gated: W_e = [gate rows; up rows], y = silu(gate) * up; with in_scale [n_pairs] the pair's row of x is
+//             taken times in_scale[p] (the two sums are, which is the same). An FMA form for every size and both
 //             storage types, and two matrix-core forms for bfloat16 with K % 8 == 0: operands straight from
 //             memory for tiles of 16 or 64 rows (few rows an expert: the weights are read once, the time is
 //             the reading), tiles of 128 rows staged in LDS where an expert has many rows.
@@ -27,8 +29,13 @@
 struct MoeAct {
     int kind;
     float limit, slope;
+    const float* in_scale;      // a factor on a pair's input row (null: none)
 };
-__device__ __forceinline__ float moe_gate(float g, float u, const MoeAct act) {
+// both halves of pair p from their 32-bit sums: scaled, rounded to what a product kernel would have stored, activated
+template <typename T>
+__device__ __forceinline__ float moe_gate(float g, float u, const MoeAct act, float in_scale) {
+    g = round_to<T>(g * in_scale);
+    u = round_to<T>(u * in_scale);
     if (act.kind == 1) {
         g = fminf(g, act.limit);
         u = fminf(fmaxf(u, -act.limit), act.limit);
@@ -38,7 +45,7 @@ __device__ __forceinline__ float moe_gate(float g, float u, const MoeAct act) {
 }
 
 // ------------------------------------------------------------------ route: one wave per token
-__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ bias,
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ z, long long ld_z, const float* __restrict__ bias,
                                                         int T, int E, int top, int n_groups, int keep, float norm_eps,
                                                         int* __restrict__ ids, float* __restrict__ weights, int law) {
     extern __shared__ float sm[];                          // per wave: s[E], c[E], group score [n_groups]
@@ -53,20 +60,20 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     // are the chosen s as they are
     float z_top = -INFINITY, z_den = 1.f;
     if (law == 2) {
-        for (int e = lane; e < E; e += 64) z_top = fmaxf(z_top, z[(size_t)t * E + e]);
+        for (int e = lane; e < E; e += 64) z_top = fmaxf(z_top, z[(size_t)t * ld_z + e]);
         z_top = wave_max(z_top);
         float part = 0.f;
-        for (int e = lane; e < E; e += 64) part += expf(z[(size_t)t * E + e] - z_top);
+        for (int e = lane; e < E; e += 64) part += expf(z[(size_t)t * ld_z + e] - z_top);
         z_den = wave_sum(part);
     }
     for (int e = lane; e < E; e += 64) {
         // law 1: the choice is made on the logits plus their bias, and the weights are the softmax over the chosen
         // ones alone (s holds the logit, turned into exp(logit - largest) as it is taken)
-        const float zv = z[(size_t)t * E + e];
+        const float zv = z[(size_t)t * ld_z + e];
         const float v = law == 2 ? expf(zv - z_top) / z_den
                                  : law == 1 ? zv + (bias ? bias[e] : 0.f) : 1.0f / (1.0f + expf(-zv));
         s[e] = v;
-        c[e] = law != 0 ? v : v + (bias ? bias[e] : 0.f);
+        c[e] = law == 1 || law == 2 ? v : v + (bias ? bias[e] : 0.f);
     }
     __builtin_amdgcn_wave_barrier();
     if (n_groups > 1 && keep < n_groups) {
@@ -114,26 +121,26 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     }
     if (lane < top) {
         ids[(size_t)t * top + lane] = my_id;
-        weights[(size_t)t * top + lane] = law == 2 ? my_w : my_w / (sum + norm_eps);
+        weights[(size_t)t * top + lane] = law >= 2 ? my_w : my_w / (sum + norm_eps);
     }
 }
 
-extern "C" int ra_moe_route_law(const float* z, const float* bias, int T, int E, int top, int n_groups, int keep,
+extern "C" int ra_moe_route_law(const float* z, long long ld_z, const float* bias, int T, int E, int top, int n_groups, int keep,
                                 float norm_eps, int* ids, float* weights, int law, void* stream) {
     if (T <= 0) return RA_OK;
-    if (law < 0 || law > 2 || (law == 1 && n_groups != 1)) return RA_ERR_ARG;
+    if (law < 0 || law > 3 || ld_z < E || (law == 1 && n_groups != 1)) return RA_ERR_ARG;
     if (E < 1 || E > MOE_MAX_EXPERTS || top < 1 || top > E || top > 64 || n_groups < 1 || E % n_groups || keep < 1 ||
         keep > n_groups || (long long)keep * (E / n_groups) < top)
         return RA_ERR_ARG;
     const size_t lds = (size_t)4 * (2 * E + n_groups) * sizeof(float);
-    hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), lds, (hipStream_t)stream, z, bias, T, E, top,
+    hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), lds, (hipStream_t)stream, z, ld_z, bias, T, E, top,
                        n_groups, keep, norm_eps, ids, weights, law);
     return ra_launch_status();
 }
 
 extern "C" int ra_moe_route(const float* z, const float* bias, int T, int E, int top, int n_groups, int keep,
                             float norm_eps, int* ids, float* weights, void* stream) {
-    return ra_moe_route_law(z, bias, T, E, top, n_groups, keep, norm_eps, ids, weights, 0, stream);
+    return ra_moe_route_law(z, E, bias, T, E, top, n_groups, keep, norm_eps, ids, weights, 0, stream);
 }
 
 // ------------------------------------------------------------------ plan: one workgroup
@@ -237,10 +244,7 @@ __global__ __launch_bounds__(256) void moe_product_fma_kernel(
         if (p < 0) continue;
         float v = ag[i];
         if (GATED) {
-            // the two products are stored values of type T before the activation, as a product kernel and an
-            // activation kernel apart would have them
-            const float g = round_to<T>(ag[i]), u = round_to<T>(au[i]);
-            v = moe_gate(g, u, act);
+            v = moe_gate<T>(ag[i], au[i], act, act.in_scale != nullptr ? act.in_scale[p] : 1.0f);
         }
         y[(size_t)p * N + col] = from_f<T>(v);
     }
@@ -319,6 +323,7 @@ __global__ __launch_bounds__(256) void moe_product_mfma_kernel(
     for (int r = 0; r < RT; ++r) {
         if (pair[r] < 0) continue;
         bf16* yr = y + (size_t)pair[r] * N;
+        const float scale = GATED && act.in_scale != nullptr ? act.in_scale[pair[r]] : 1.0f;
 #pragma unroll
         for (int c = 0; c < CT; ++c) {
             const int col = col0 + 16 * c + 4 * g;
@@ -326,10 +331,7 @@ __global__ __launch_bounds__(256) void moe_product_mfma_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 v[i] = ag[r][c][i];
-                if (GATED) {
-                    const float gg = round_to<bf16>(ag[r][c][i]), uu = round_to<bf16>(au[r][c][i]);
-                    v[i] = moe_gate(gg, uu, act);
-                }
+                if (GATED) v[i] = moe_gate<bf16>(ag[r][c][i], au[r][c][i], act, scale);
             }
             if (col + 3 < N && (N & 3) == 0) {
                 uint2 pk;
@@ -442,7 +444,9 @@ __global__ __launch_bounds__(256) void moe_product_tile_kernel(
     for (int j = 0; j < 4; ++j) {
         const int m = wm * 64 + j * 16 + n;
         if (m >= n_rows) continue;
-        bf16* yr = y + (size_t)order[at + m] * N;
+        const int p = order[at + m];
+        bf16* yr = y + (size_t)p * N;
+        const float scale = GATED && act.in_scale != nullptr ? act.in_scale[p] : 1.0f;
 #pragma unroll
         for (int i = 0; i < (GATED ? 2 : 4); ++i) {
             const int col = GATED ? n0 + wn * 32 + i * 16 + 4 * g : n0 + wn * 64 + i * 16 + 4 * g;
@@ -450,10 +454,7 @@ __global__ __launch_bounds__(256) void moe_product_tile_kernel(
 #pragma unroll
             for (int c = 0; c < 4; ++c) {
                 v[c] = acc[i][j][c];
-                if (GATED) {
-                    const float gg = round_to<bf16>(acc[i][j][c]), uu = round_to<bf16>(acc[i + 2][j][c]);
-                    v[c] = moe_gate(gg, uu, act);
-                }
+                if (GATED) v[c] = moe_gate<bf16>(acc[i][j][c], acc[i + 2][j][c], act, scale);
             }
             if (col + 3 < N && (N & 3) == 0) {
                 uint2 pk;
@@ -478,13 +479,14 @@ extern "C" int ra_moe_tile_rows(int n_pairs, int E, int K, int dtype) {
 // x [rows][K]; w [E][N or 2N][K]; y [n_pairs][N]; the row of pair p in x is p / top_div (top_div = top: the
 // token's row; 1: the pair's own row). max_tiles: the grid's first dimension, at least the number of tiles
 // the plan can have (n_pairs / rows + E); workgroups beyond meta[0] leave at once.
-// (act_kind, limit, slope: what a gated product makes of its halves, see MoeAct)
+// (act_kind, limit, slope, in_scale: what a gated product makes of its halves, see MoeAct)
 extern "C" int ra_moe_product_act(const void* x, const void* w, void* y, const int* order, const int* tiles,
                                   const int* meta, int max_tiles, int tile_rows, int N, int K, int top_div, int gated,
-                                  int act_kind, float limit, float slope, int dtype, void* stream) {
+                                  int act_kind, float limit, float slope, const float* in_scale, int dtype,
+                                  void* stream) {
     if (max_tiles <= 0) return RA_OK;
-    if (N < 1 || K < 1 || top_div < 1 || act_kind < 0 || act_kind > 1) return RA_ERR_ARG;
-    const MoeAct act = {act_kind, limit, slope};
+    if (N < 1 || K < 1 || top_div < 1 || act_kind < 0 || act_kind > 1 || (in_scale != nullptr && !gated)) return RA_ERR_ARG;
+    const MoeAct act = {act_kind, limit, slope, in_scale};
     hipStream_t st = (hipStream_t)stream;
     if (dtype == RA_DTYPE_BF16 && K % 8 == 0 && tile_rows == MT_BM) {
         const int cn = gated ? 64 : 128;
@@ -524,45 +526,50 @@ extern "C" int ra_moe_product_act(const void* x, const void* w, void* y, const i
 extern "C" int ra_moe_product(const void* x, const void* w, void* y, const int* order, const int* tiles,
                               const int* meta, int max_tiles, int tile_rows, int N, int K, int top_div, int gated,
                               int dtype, void* stream) {
-    return ra_moe_product_act(x, w, y, order, tiles, meta, max_tiles, tile_rows, N, K, top_div, gated, 0, 0.f, 0.f, dtype,
+    return ra_moe_product_act(x, w, y, order, tiles, meta, max_tiles, tile_rows, N, K, top_div, gated, 0, 0.f, 0.f, nullptr, dtype,
                               stream);
 }
 
 // ------------------------------------------------------------------ combine
-template <typename T>
+template <typename T, typename L>
 __global__ void moe_combine_kernel(const T* __restrict__ y, const float* __restrict__ weights, T* __restrict__ out,
                                    int top, int N, long long total, const T* __restrict__ extra,
-                                   const T* __restrict__ logit, long long ld_logit) {
+                                   const L* __restrict__ logit, long long ld_logit) {
     const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= total) return;
     const long long t = i / N;
     const int c = (int)(i - t * N);
     float acc = 0.f;
-    for (int k = 0; k < top; ++k) acc = fmaf(weights[t * top + k], to_f(y[((size_t)t * top + k) * N + c]), acc);
+    for (int k = 0; k < top; ++k)
+        acc = fmaf(weights != nullptr ? weights[t * top + k] : 1.0f, to_f(y[((size_t)t * top + k) * N + c]), acc);
     // one more term that every token has: extra[t] times sigmoid(logit[t]), added last
     if (extra != nullptr) acc = fmaf(to_f(extra[i]), 1.0f / (1.0f + expf(-to_f(logit[t * ld_logit]))), acc);
     out[i] = from_f<T>(acc);
 }
 
-// extra [T, N] and logit (one number a token, rows ld_logit elements apart) may be null: no further term
+// weights null: factors of one. extra [T, N] and logit (one number a token, rows ld_logit elements apart, of type
+// logit_dtype: the rows' own or 32-bit) may be null: no further term
 extern "C" int ra_moe_combine_extra(const void* y, const float* weights, void* out, int T, int top, int N,
-                                    const void* extra, const void* logit, long long ld_logit, int dtype, void* stream) {
+                                    const void* extra, const void* logit, int logit_dtype, long long ld_logit, int dtype,
+                                    void* stream) {
     const long long total = (long long)T * N;
     if (total <= 0) return RA_OK;
-    if ((extra == nullptr) != (logit == nullptr) || (extra != nullptr && ld_logit < 1)) return RA_ERR_ARG;
-    dim3 block(256), grid((unsigned)((total + 255) / 256));
-    if (dtype == RA_DTYPE_F32)
-        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, block, 0, (hipStream_t)stream, (const float*)y, weights,
-                           (float*)out, top, N, total, (const float*)extra, (const float*)logit, ld_logit);
-    else if (dtype == RA_DTYPE_BF16)
-        hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, block, 0, (hipStream_t)stream, (const bf16*)y, weights,
-                           (bf16*)out, top, N, total, (const bf16*)extra, (const bf16*)logit, ld_logit);
-    else
+    if ((extra == nullptr) != (logit == nullptr) || (extra != nullptr && ld_logit < 1) ||
+        (logit_dtype != dtype && logit_dtype != RA_DTYPE_F32))
         return RA_ERR_ARG;
+    dim3 block(256), grid((unsigned)((total + 255) / 256));
+#define MOE_COMBINE(T_, L_)                                                                                              \
+    hipLaunchKernelGGL((moe_combine_kernel<T_, L_>), grid, block, 0, (hipStream_t)stream, (const T_*)y, weights, (T_*)out, \
+                       top, N, total, (const T_*)extra, (const L_*)logit, ld_logit)
+    if (dtype == RA_DTYPE_F32) MOE_COMBINE(float, float);
+    else if (dtype == RA_DTYPE_BF16 && logit_dtype == RA_DTYPE_BF16) MOE_COMBINE(bf16, bf16);
+    else if (dtype == RA_DTYPE_BF16) MOE_COMBINE(bf16, float);
+    else return RA_ERR_ARG;
+#undef MOE_COMBINE
     return ra_launch_status();
 }
 
 extern "C" int ra_moe_combine(const void* y, const float* weights, void* out, int T, int top, int N, int dtype,
                               void* stream) {
-    return ra_moe_combine_extra(y, weights, out, T, top, N, nullptr, nullptr, 0, dtype, stream);
+    return ra_moe_combine_extra(y, weights, out, T, top, N, nullptr, nullptr, dtype, 0, dtype, stream);
 }

@@ -1,5 +1,5 @@
-// Row kernels of a layer whose sublayers run side by side, of an attention with biases and blended values, and of
-// an expert that every token uses.
+// Row kernels of a layer whose sublayers run side by side, of attentions with biases, blended values, norms over whole
+// projections and gates on their output, and of feed-forwards whose halves meet in a kernel of their own.
 //
 //   add_rmsnorm_pair   h += a + b (the 32-bit stream; a and b, in the storage type, may each be null), then two RMS
 //                      norms of the same row with weights of their own: x1 = h / sqrt(mean(h^2) + eps1) * w1,
@@ -13,8 +13,14 @@
 //                      key pool. v: mode 1 writes the first Dv elements of the biased v into `first` (32-bit,
 //                      [T, Hkv, Dv]: a head's true width, which layers of other row widths share) and v into the
 //                      value pool; mode 2 stores (1 - lambda) v + lambda first[t]; mode 0 stores v.
-//   clamped_mul        out[t][i] = g sigmoid(slope g) (u + 1) with g = min(gu[t][i], limit),
-//                      u = clamp(gu[t][I + i], -limit, limit); gu rows are ld_gu elements apart.
+//   qkv_rows_prepare   one workgroup per token over the same row [q heads | k heads | v heads]: the whole query part is
+//                      divided by the root mean square of its nq elements and weighed (w_q [Hq D]), the whole key part
+//                      by that of its nk elements (w_k [Hkv D]; elements beyond a head's true width are zeros and do
+//                      not count), the first R elements of every q and k head turn as above, q goes to q_out, k and v
+//                      to their cache rows.
+//   gate_rows          o[t][i] *= sigmoid(g[t][i]); both rows apart by their own distances
+//   gated_rows         out[t][i] from gu[t][i] and gu[t][I + i] (32-bit or storage type, rows ld_gu elements apart): kind 0
+//                      silu(g) u; kind 1 g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit).
 #include "common.h"
 #include <algorithm>
 
@@ -341,33 +347,200 @@ extern "C" int ra_qkv_blend_prepare(const void* qkv, long long ld_qkv, int T_tok
     return ra_launch_status();
 }
 
-// ------------------------------------------------------------------ the shared expert's activation
-template <typename T>
-__global__ void clamped_mul_kernel(const T* __restrict__ gu, long long ld_gu, T* __restrict__ out, int I, float limit,
-                                   float slope, size_t total) {
-    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
-        const size_t t = i / I;
-        const int c = (int)(i - t * I);
-        const float g = fminf(to_f(gu[t * ld_gu + c]), limit);
-        const float u = fminf(fmaxf(to_f(gu[t * ld_gu + I + c]), -limit), limit);
-        out[i] = from_f<T>(g / (1.0f + expf(-slope * g)) * (u + 1.0f));
+// ------------------------------------------------------------------ q/k/v preparation with norms over whole projections
+// V elements at a time: of a q or k head R/2/V units of (V, and the V they turn with) and (D - R)/V units that pass, of a
+// v head D/V units. 0 <= unit < total of all heads; the row is read twice (the second time from the caches).
+template <typename T, int V> struct PrVec;
+template <typename T> struct PrVec<T, 1> {
+    static __device__ __forceinline__ void load(const T* p, float (&v)[1]) { v[0] = to_f(*p); }
+    static __device__ __forceinline__ void store(T* p, const float (&v)[1]) { *p = from_f<T>(v[0]); }
+};
+template <typename T> struct PrVec<T, 4> {
+    static __device__ __forceinline__ void load(const T* p, float (&v)[4]) {
+        const float4 t = pr_load4(p);
+        v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
+    }
+    static __device__ __forceinline__ void store(T* p, const float (&v)[4]) { pr_store4(p, make_float4(v[0], v[1], v[2], v[3])); }
+};
+
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void qkv_rows_prepare_kernel(const T* __restrict__ qkv, long long ld_qkv, int Hq, int Hkv,
+                                                               int D, const float* __restrict__ w_q,
+                                                               const float* __restrict__ w_k, int nq, int nk, float eps,
+                                                               const int* __restrict__ positions,
+                                                               const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+                                                               int R, T* __restrict__ q_out, T* __restrict__ k_pool,
+                                                               T* __restrict__ v_pool, const int* __restrict__ slots, int P,
+                                                               long long pool_rows) {
+    __shared__ float scratch[16];
+    const int t = blockIdx.x, tid = threadIdx.x, nt = blockDim.x;
+    const T* src = qkv + (size_t)t * ld_qkv;
+    const int wq = Hq * D, wk = Hkv * D;
+    float sq = 0.f, sk = 0.f;
+    for (int c = tid * V; c < wq + wk; c += nt * V) {
+        float v[V], s = 0.f;
+        PrVec<T, V>::load(src + c, v);
+#pragma unroll
+        for (int e = 0; e < V; ++e) s = fmaf(v[e], v[e], s);
+        if (c < wq) sq += s; else sk += s;                   // (V divides D, so a group lies in one part)
+    }
+    const float rq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
+    const float rk = 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);
+    long long slot = -1;
+    if (k_pool != nullptr) {
+        slot = slots[t];
+        if (slot >= pool_rows) slot = -1;
+    }
+    const int half = R >> 1, pairs = half / V, passing = (D - R) / V, per = pairs + passing, per_v = D / V;
+    const int n_qk = (slot >= 0 ? Hq + Hkv : Hq) * per, n_all = n_qk + (slot >= 0 ? Hkv * per_v : 0);
+    const int pos = positions[t];
+    for (int unit = tid; unit < n_all; unit += nt) {
+        if (unit >= n_qk) {
+            const int kvh = (unit - n_qk) / per_v, c = (unit - n_qk - kvh * per_v) * V;
+            float v[V];
+            PrVec<T, V>::load(src + wq + wk + (size_t)kvh * D + c, v);
+            PrVec<T, V>::store(v_pool + ra_cache_offset(slot, kvh, Hkv, P, D) + c, v);
+            continue;
+        }
+        const int head = unit / per, u = unit - head * per;
+        const bool is_q = head < Hq;
+        const float rstd = is_q ? rq : rk;
+        const float* wn = is_q ? w_q + (size_t)head * D : w_k + (size_t)(head - Hq) * D;
+        const T* hs = src + (size_t)head * D;
+        T* dst = is_q ? q_out + ((size_t)t * Hq + head) * D : k_pool + ra_cache_offset(slot, head - Hq, Hkv, P, D);
+        float a[V], wa[V];
+        if (u < pairs) {
+            const int j = u * V;
+            float b[V], wb[V], cs[V], sn[V], oa[V], ob[V];
+            PrVec<T, V>::load(hs + j, a);
+            PrVec<T, V>::load(hs + half + j, b);
+            PrVec<float, V>::load(wn + j, wa);
+            PrVec<float, V>::load(wn + half + j, wb);
+            PrVec<float, V>::load(cos_t + (size_t)pos * half + j, cs);
+            PrVec<float, V>::load(sin_t + (size_t)pos * half + j, sn);
+#pragma unroll
+            for (int e = 0; e < V; ++e) {
+                const float x1 = a[e] * rstd * wa[e], x2 = b[e] * rstd * wb[e];
+                oa[e] = x1 * cs[e] - x2 * sn[e];
+                ob[e] = x2 * cs[e] + x1 * sn[e];
+            }
+            PrVec<T, V>::store(dst + j, oa);
+            PrVec<T, V>::store(dst + half + j, ob);
+        } else {
+            const int c = R + (u - pairs) * V;
+            PrVec<T, V>::load(hs + c, a);
+            PrVec<float, V>::load(wn + c, wa);
+#pragma unroll
+            for (int e = 0; e < V; ++e) a[e] = a[e] * rstd * wa[e];
+            PrVec<T, V>::store(dst + c, a);
+        }
     }
 }
 
-extern "C" int ra_clamped_mul(const void* gu, long long ld_gu, void* out, int T_tokens, int I, float limit, float slope,
-                              int dtype, void* stream) {
+extern "C" int ra_qkv_rows_prepare(const void* qkv, long long ld_qkv, int T_tokens, int Hq, int Hkv, int D, const float* w_q,
+                                   const float* w_k, int nq, int nk, float eps, const int* positions, const float* cos_t,
+                                   const float* sin_t, int R, void* q_out, void* k_pool, void* v_pool, const int* slots,
+                                   int P, long long pool_rows, int dtype, void* stream) {
     if (T_tokens <= 0) return RA_OK;
-    if (I < 1 || ld_gu < 2LL * I || !(limit > 0.f)) return RA_ERR_ARG;
-    const size_t total = (size_t)T_tokens * I;
-    const unsigned blocks = (unsigned)std::min<size_t>((total + 255) / 256, 65535u * 16u);
-    hipStream_t st = (hipStream_t)stream;
-    if (dtype == RA_DTYPE_F32)
-        hipLaunchKernelGGL(clamped_mul_kernel<float>, dim3(blocks), dim3(256), 0, st, (const float*)gu, ld_gu, (float*)out,
-                           I, limit, slope, total);
-    else if (dtype == RA_DTYPE_BF16)
-        hipLaunchKernelGGL(clamped_mul_kernel<bf16>, dim3(blocks), dim3(256), 0, st, (const bf16*)gu, ld_gu, (bf16*)out, I,
-                           limit, slope, total);
-    else
+    if ((k_pool == nullptr) != (v_pool == nullptr) || (k_pool != nullptr && (P <= 0 || slots == nullptr))) return RA_ERR_ARG;
+    if (D < 1 || Hq < 1 || Hkv < 1 || R < 0 || R > D || (R & 1) || q_out == nullptr || w_q == nullptr || w_k == nullptr ||
+        positions == nullptr || ld_qkv < (long long)(Hq + 2 * Hkv) * D || nq < 1 || nq > Hq * D || nk < 1 || nk > Hkv * D ||
+        (R > 0 && (cos_t == nullptr || sin_t == nullptr)) || (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16))
         return RA_ERR_ARG;
+    hipStream_t st = (hipStream_t)stream;
+    const auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    const bool vec = D % 4 == 0 && R % 8 == 0 && ld_qkv % 4 == 0 && aligned(qkv) && aligned(q_out) && aligned(k_pool) &&
+                     aligned(v_pool) && aligned(w_q) && aligned(w_k) && aligned(cos_t) && aligned(sin_t);
+    const int threads = T_tokens <= 256 ? 1024 : 256;        // few tokens: one round of reads a thread
+#define QKV_ROWS(T_, V_)                                                                                                 \
+    hipLaunchKernelGGL((qkv_rows_prepare_kernel<T_, V_>), dim3(T_tokens), dim3(threads), 0, st, (const T_*)qkv, ld_qkv, Hq, \
+                       Hkv, D, w_q, w_k, nq, nk, eps, positions, cos_t, sin_t, R, (T_*)q_out, (T_*)k_pool, (T_*)v_pool, \
+                       slots, P, pool_rows)
+    if (dtype == RA_DTYPE_F32) { if (vec) QKV_ROWS(float, 4); else QKV_ROWS(float, 1); }
+    else { if (vec) QKV_ROWS(bf16, 4); else QKV_ROWS(bf16, 1); }
+#undef QKV_ROWS
+    return ra_launch_status();
+}
+
+// ------------------------------------------------------------------ a gate on every element of a row
+template <typename T, int V>
+__global__ void gate_rows_kernel(T* __restrict__ o, long long ld_o, const T* __restrict__ g, long long ld_g, int N,
+                                 long long total) {
+    const int per = N / V;
+    for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (long long)gridDim.x * blockDim.x) {
+        const long long t = i / per;
+        const int c = (int)(i - t * per) * V;
+        float a[V], b[V];
+        PrVec<T, V>::load(o + t * ld_o + c, a);
+        PrVec<T, V>::load(g + t * ld_g + c, b);
+#pragma unroll
+        for (int e = 0; e < V; ++e) a[e] = a[e] / (1.0f + expf(-b[e]));
+        PrVec<T, V>::store(o + t * ld_o + c, a);
+    }
+}
+
+extern "C" int ra_gate_rows(void* o, long long ld_o, const void* g, long long ld_g, int T_tokens, int N, int dtype,
+                            void* stream) {
+    if (T_tokens <= 0) return RA_OK;
+    if (N < 1 || ld_o < N || ld_g < N || o == nullptr || g == nullptr || (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16))
+        return RA_ERR_ARG;
+    hipStream_t st = (hipStream_t)stream;
+    const bool vec = N % 4 == 0 && ld_o % 4 == 0 && ld_g % 4 == 0 && ((uintptr_t)o & 15) == 0 && ((uintptr_t)g & 15) == 0;
+    const long long total = (long long)T_tokens * (N / (vec ? 4 : 1));
+    const unsigned blocks = (unsigned)std::min<long long>((total + 255) / 256, 65535LL * 16);
+#define GATE_ROWS(T_, V_)                                                                                       \
+    hipLaunchKernelGGL((gate_rows_kernel<T_, V_>), dim3(blocks), dim3(256), 0, st, (T_*)o, ld_o, (const T_*)g, ld_g, N, total)
+    if (dtype == RA_DTYPE_F32) { if (vec) GATE_ROWS(float, 4); else GATE_ROWS(float, 1); }
+    else { if (vec) GATE_ROWS(bf16, 4); else GATE_ROWS(bf16, 1); }
+#undef GATE_ROWS
+    return ra_launch_status();
+}
+
+// ------------------------------------------------------------------ the two halves of a feed-forward
+template <typename S, typename T, int V>
+__global__ void gated_rows_kernel(const S* __restrict__ gu, long long ld_gu, T* __restrict__ out, int I, int kind, float limit,
+                                  float slope, long long total) {
+    const int per = I / V;
+    for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (long long)gridDim.x * blockDim.x) {
+        const long long t = i / per;
+        const int c = (int)(i - t * per) * V;
+        float a[V], b[V];
+        PrVec<S, V>::load(gu + t * ld_gu + c, a);
+        PrVec<S, V>::load(gu + t * ld_gu + I + c, b);
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            if (kind == 1) {
+                const float g = fminf(a[e], limit), u = fminf(fmaxf(b[e], -limit), limit);
+                a[e] = g / (1.0f + expf(-slope * g)) * (u + 1.0f);
+            } else {
+                a[e] = a[e] / (1.0f + expf(-a[e])) * b[e];
+            }
+        }
+        PrVec<T, V>::store(out + t * I + c, a);
+    }
+}
+
+extern "C" int ra_gated_rows(const void* gu, int gu_dtype, long long ld_gu, void* out, int T_tokens, int I, int kind,
+                             float limit, float slope, int dtype, void* stream) {
+    if (T_tokens <= 0) return RA_OK;
+    if (I < 1 || ld_gu < 2LL * I || kind < 0 || kind > 1 || (kind == 1 && !(limit > 0.f)) || gu == nullptr || out == nullptr ||
+        (gu_dtype != RA_DTYPE_F32 && gu_dtype != dtype))
+        return RA_ERR_ARG;
+    hipStream_t st = (hipStream_t)stream;
+    const bool vec = I % 4 == 0 && ld_gu % 4 == 0 && ((uintptr_t)gu & 15) == 0 && ((uintptr_t)out & 15) == 0;
+    const long long total = (long long)T_tokens * (I / (vec ? 4 : 1));
+    const unsigned blocks = (unsigned)std::min<long long>((total + 255) / 256, 65535LL * 16);
+#define GATED_ROWS(S_, T_)                                                                                           \
+    do {                                                                                                             \
+        if (vec) hipLaunchKernelGGL((gated_rows_kernel<S_, T_, 4>), dim3(blocks), dim3(256), 0, st, (const S_*)gu, ld_gu, \
+                                    (T_*)out, I, kind, limit, slope, total);                                         \
+        else hipLaunchKernelGGL((gated_rows_kernel<S_, T_, 1>), dim3(blocks), dim3(256), 0, st, (const S_*)gu, ld_gu, \
+                                (T_*)out, I, kind, limit, slope, total);                                             \
+    } while (0)
+    if (dtype == RA_DTYPE_F32) GATED_ROWS(float, float);
+    else if (dtype == RA_DTYPE_BF16 && gu_dtype == RA_DTYPE_BF16) GATED_ROWS(bf16, bf16);
+    else if (dtype == RA_DTYPE_BF16) GATED_ROWS(float, bf16);
+    else return RA_ERR_ARG;
+#undef GATED_ROWS
     return ra_launch_status();
 }

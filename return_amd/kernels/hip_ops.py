@@ -12,7 +12,7 @@ from typing import Optional
 
 import torch
 
-from ..parts.runtime import ScaledRows, Slabs
+from ..parts.runtime import RowSums, ScaledRows, Slabs
 from . import build as _build
 
 _F32, _BF16 = 0, 1
@@ -57,14 +57,16 @@ def _declare(lib):
         "ra_post_norm_mix": [P, L, I, P, P, P, F, P, P, F, P, I, I, I, P],
         "ra_heads_gate": [P, P, L, P, I, I, I, I, P],
         "ra_silu_mul_bias": [P, P, P, I, I, I, P],
-        "ra_latent_kv_prepare": [P, L, I, I, I, I, P, P, F, P, P, P, I, P, P, P, P, I, I, P],
+        "ra_latent_kv_prepare": [P, L, I, I, I, I, P, P, F, P, P, P, I, P, P, P, P, I, P, L, I, I, P, I, P],
         "ra_latent_q_prepare": [P, P, I, I, I, I, I, P, P, P, I, P, I, P],
         "ra_attention_latent_plain": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, I, I, P],
         "ra_attention_latent_plain_window": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, I, I, I, P],
         "ra_attention_latent_mfma_window_bf16": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P, I, P, I, P],
         "ra_add_rmsnorm_pair": [P, P, P, P, F, P, P, F, P, I, I, I, P],
         "ra_qkv_blend_prepare": [P, L, I, I, I, I, P, P, P, I, F, P, P, P, I, P, P, P, P, I, L, P, I, I, F, I, P],
-        "ra_clamped_mul": [P, L, P, I, I, F, F, I, P],
+        "ra_gated_rows": [P, I, L, P, I, I, I, F, F, I, P],
+        "ra_gate_rows": [P, L, P, L, I, I, I, P],
+        "ra_qkv_rows_prepare": [P, L, I, I, I, I, P, P, I, I, F, P, P, P, I, P, P, P, P, I, L, I, P],
         "ra_causal_conv_bias": [P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, P],
         "ra_scalar_rule": [P, L, P, L, P, L, P, P, P, P, I, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "ra_attention_latent_plain_fits": [I, I],
@@ -72,8 +74,8 @@ def _declare(lib):
         "ra_attention_latent_mfma_fits": [I, I, I],
         "ra_attention_latent_mfma_tile_tokens": [I],
         "ra_outer_rule": [P, L, P, L, P, L, P, F, P, F, P, P, P, P, P, I, I, I, I, I, I, I, P],
-        "ra_moe_route_law": [P, P, I, I, I, I, I, F, P, P, I, P],
-        "ra_moe_product_act": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, I, P],
+        "ra_moe_route_law": [P, L, P, I, I, I, I, I, F, P, P, I, P],
+        "ra_moe_product_act": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P, I, P],
         "ra_add_rmsnorm": [P, P, P, F, P, P, I, I, I, P],
         "ra_add_scaled_rmsnorm": [P, P, F, P, F, P, P, I, I, I, P],
         "ra_stream_pair_rows": [P, P, F, P, P, L, I, I, P],
@@ -87,7 +89,7 @@ def _declare(lib):
         "ra_moe_tile_rows": [I, I, I, I],
         "ra_moe_product": [P, P, P, P, P, P, I, I, I, I, I, I, I, P],
         "ra_moe_combine": [P, P, P, I, I, I, I, P],
-        "ra_moe_combine_extra": [P, P, P, I, I, I, P, P, L, I, P],
+        "ra_moe_combine_extra": [P, P, P, I, I, I, P, P, I, L, I, P],
         "ra_add_slabs_rmsnorm": [P, P, I, L, P, F, P, P, I, I, I, P],
         "ra_residual_add": [P, P, L, I, P],
         "ra_head_rmsnorm": [P, P, F, L, I, I, P],
@@ -114,7 +116,7 @@ def _declare(lib):
         "ra_channel_recurrence_chunk": [I],
         "ra_channel_recurrence_mfma": [I, I, I],
         "ra_layer_norm_add": [P, P, P, F, P, I, I, I, P],
-        "ra_layer_norm_rows": [P, P, F, P, P, I, I, I, P],
+        "ra_stream_layer_norm": [P, P, P, I, P, P, P, L, P, P, F, P, P, I, I, I, P],
         "ra_stream_rows": [P, P, L, I, P],
         "ra_softcap": [P, F, L, P],
         "ra_delta_rule_fits": [I, I],
@@ -183,7 +185,7 @@ class HipOps:
             self._library_fp32_out = False
         try:                                 # and the same for a batch of products
             a = torch.ones(2, 1, 8, dtype=torch.bfloat16, device=self.device)
-            self._library_bmm_fp32 = torch.bmm(a, a.transpose(1, 2), out_dtype=torch.float32).dtype == torch.float32
+            self._library_bmm_fp32 = torch.bmm(a, a.transpose(1, 2).contiguous(), out_dtype=torch.float32).dtype == torch.float32
         except (TypeError, RuntimeError):
             self._library_bmm_fp32 = False
         # whether the library's float32 product is a true 32-bit one (against a 64-bit product; operands
@@ -362,11 +364,18 @@ class HipOps:
         self._check(self.lib.ra_heads_gate(_ptr(o), _ptr(gate), ld, _ptr(out), T, Hn, Dv, _code(o.dtype), self._stream()),
                     "heads_gate")
 
-    def batched_product(self, a, b):
-        """[B, M, K] x [B, K, N] -> [B, M, N] in a's dtype, by the library (32-bit operands: a true 32-bit product)."""
-        if a.dim() != 3 or b.dim() != 3 or a.shape[0] != b.shape[0] or a.shape[2] != b.shape[1] or a.dtype != b.dtype:
+    def batched_product(self, a, b, out=None):
+        """[B, M, K] x [B, K, N] -> [B, M, N] in a's dtype, by the library (32-bit operands: a true 32-bit product). out:
+        where the result goes (rows of N elements side by side, apart by any distance: the rows of all b's batches may be
+        columns of the same wider rows); None: a new tensor."""
+        if a.dim() != 3 or b.dim() != 3 or a.shape[0] != b.shape[0] or a.shape[2] != b.shape[1] or a.dtype != b.dtype \
+                or not b.is_contiguous():
             raise KernelError(f"batched_product: {tuple(a.shape)} x {tuple(b.shape)}")
-        return torch.bmm(a, b)
+        if out is None:
+            return torch.bmm(a, b)
+        if tuple(out.shape) != (a.shape[0], a.shape[1], b.shape[2]) or out.dtype != a.dtype or (out.shape[2] > 1 and out.stride(2) != 1):
+            raise KernelError(f"batched_product: {tuple(a.shape)} x {tuple(b.shape)} into {tuple(out.shape)}, strides {out.stride()}")
+        return torch.bmm(a, b, out=out)
 
     def add_rmsnorm(self, h, delta, weight, eps, out, rows=None, delta_scale=1.0):
         """h += delta_scale * delta (in place, unless a row list is given); out = norm(h) * weight."""
@@ -594,17 +603,70 @@ class HipOps:
                                                  float(eps2), _ptr(out2), T, H, _code(out1.dtype), self._stream()),
                     "add_rmsnorm_pair")
 
-    def clamped_mul(self, gu, out, limit, slope=1.702):
-        """gu [T, >= 2 I] (gate columns first; possibly a column slice of wider rows) -> out [T, I] =
-        g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)."""
+    def gated_rows(self, gu, out, activation="silu", limit=0.0, slope=1.702):
+        """gu [T, >= 2 I] (gate columns first; possibly a column slice of wider rows; out's type or fp32) -> out [T, I] =
+        silu(gate) * up or, "clamped", g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)."""
         ld = self._want_rows(gu, "gate-up rows")
-        self._want(out, "activation output", gu.dtype, 2)
+        self._want(out, "activation output", dims=2)
         T, I = out.shape
-        if gu.shape[0] != T or gu.shape[1] < 2 * I or not limit > 0:
-            raise KernelError(f"clamped_mul: gu {tuple(gu.shape)}, out {tuple(out.shape)}, limit {limit}")
-        self._check(self.lib.ra_clamped_mul(_ptr(gu), ld, _ptr(out), T, I, float(limit), float(slope), _code(gu.dtype),
-                                            self._stream()), "clamped_mul")
+        if activation not in ("silu", "clamped") or (activation == "clamped" and not limit > 0):
+            raise KernelError(f"gated_rows: activation {activation!r} with limit {limit}")
+        if gu.shape[0] != T or gu.shape[1] < 2 * I or gu.dtype not in (out.dtype, torch.float32):
+            raise KernelError(f"gated_rows: gu {tuple(gu.shape)} {gu.dtype}, out {tuple(out.shape)} {out.dtype}")
+        self._check(self.lib.ra_gated_rows(_ptr(gu), _code(gu.dtype), ld, _ptr(out), T, I, 1 if activation == "clamped" else 0,
+                                           float(limit), float(slope), _code(out.dtype), self._stream()), "gated_rows")
         return out
+
+    def clamped_mul(self, gu, out, limit, slope=1.702):
+        return self.gated_rows(gu, out, "clamped", limit, slope)
+
+    def gate_rows(self, o, gate):
+        """o [T, N] *= sigmoid(gate) in place, element by element in 32-bit; both possibly column slices of wider rows."""
+        ld_o = self._want_rows(o, "rows to gate")
+        ld_g = self._want_rows(gate, "gates", o.dtype)
+        if gate.shape != o.shape:
+            raise KernelError(f"gate_rows: rows {tuple(o.shape)}, gates {tuple(gate.shape)}")
+        self._check(self.lib.ra_gate_rows(_ptr(o), ld_o, _ptr(gate), ld_g, o.shape[0], o.shape[1], _code(o.dtype),
+                                          self._stream()), "gate_rows")
+        return o
+
+    def qkv_rows_prepare(self, qkv, n_q, n_kv, D, w_q, w_k, q_size, k_size, eps, positions, cos, sin, rotary_dim, q_out,
+                         k_pool, v_pool, slot_mapping):
+        """q/k/v preparation of an attention whose norms run over the whole query and key projections: rows of qkv
+        (possibly a column slice of wider rows) are [n_q | n_kv | n_kv] heads of D; the query part is divided by
+        sqrt(sum of its squares / q_size + eps) and weighed (w_q fp32 [n_q D]), the key part by k_size likewise (w_k fp32
+        [n_kv D]; elements beyond a head's true width must be zeros), then the first rotary_dim elements of every q and k
+        head turn by the position (element i with i + rotary_dim / 2). q to q_out [T, n_q, D], k and v to the pools' rows
+        that slot_mapping names (pools None: nothing is written)."""
+        ld_qkv = self._want_rows(qkv, "qkv")
+        self._want(q_out, "q", qkv.dtype, 3)
+        self._want(positions, "positions", torch.int32, 1)
+        T, R = qkv.shape[0], int(rotary_dim)
+        if qkv.shape[1] != (n_q + 2 * n_kv) * D or tuple(q_out.shape) != (T, n_q, D) or positions.shape[0] != T \
+                or not 1 <= q_size <= n_q * D or not 1 <= k_size <= n_kv * D:
+            raise KernelError(f"qkv_rows_prepare: qkv {tuple(qkv.shape)}, q {tuple(q_out.shape)}, {T} tokens, norms over "
+                              f"{q_size} and {k_size}")
+        for w, n in ((w_q, n_q), (w_k, n_kv)):
+            self._want(w, "norm weight", torch.float32, 1)
+            if w.shape[0] != n * D:
+                raise KernelError(f"qkv_rows_prepare: norm weight {tuple(w.shape)} for {n} heads of {D}")
+        if R:
+            self._want(cos, "cos table", torch.float32, 2)
+            self._want(sin, "sin table", torch.float32, 2)
+            if R % 2 or R > D or cos.shape[1] != R // 2 or sin.shape != cos.shape:
+                raise KernelError(f"qkv_rows_prepare: rotary_dim {R}, tables {tuple(cos.shape)}, head size {D}")
+        P, pool_rows = 1, 0
+        if k_pool is not None:
+            self._want(slot_mapping, "slot mapping", torch.int32, 1)
+            if slot_mapping.shape[0] != T:
+                raise KernelError("qkv_rows_prepare: slot mapping does not match the token count")
+            pool_rows = self._pool_rows(k_pool, v_pool, n_kv, D, qkv.dtype)
+            P = k_pool.shape[2]
+        self._check(self.lib.ra_qkv_rows_prepare(
+            _ptr(qkv), ld_qkv, T, n_q, n_kv, D, _ptr(w_q), _ptr(w_k), int(q_size), int(k_size), float(eps), _ptr(positions),
+            _ptr(cos) if R else None, _ptr(sin) if R else None, R, _ptr(q_out), _ptr(k_pool), _ptr(v_pool),
+            _ptr(slot_mapping) if k_pool is not None else None, P, pool_rows, _code(qkv.dtype), self._stream()),
+            "qkv_rows_prepare")
 
     def qkv_blend_prepare(self, qkv, n_q, n_kv, D, bias, positions, cos, sin, rotary_dim, q_out, k_pool, v_pool,
                           slot_mapping, first=None, blend=None, w_q=None, w_k=None, norm_dim=None, eps=0.0):
@@ -824,19 +886,51 @@ class HipOps:
         self._check(self.lib.ra_layer_norm_add(_ptr(h), _ptr(y), _ptr(weight), float(eps), _ptr(out), T, H, _code(y.dtype),
                                                self._stream()), "layer_norm_add")
 
-    def layer_norm(self, h, weight, eps, out, rows=None):
-        """out[i] = (h[r] - mean) / sqrt(variance + eps) * weight with r = rows[i] (int32; None: r = i)."""
+    def layer_norm(self, h, weight, eps, out, rows=None, bias=None, first=None, second=None):
+        """out[i] = (g[r] - mean) / sqrt(variance + eps) * weight + bias with r = rows[i] (int32; None: r = i), where g is h
+        (fp32 [T, H]) plus, in 32-bit, first [T, H] and second (rows [T, H] or RowSums), each None or in out's type. Without
+        a list of rows h becomes g; with one it stays as it is."""
         self._want(h, "residual stream", torch.float32, 2)
         self._want(weight, "norm weight", torch.float32, 1)
         self._want(out, "norm output", dims=2)
-        M = h.shape[0]
+        T, H = h.shape
+        M = T
         if rows is not None:
             self._want(rows, "row list", torch.int32, 1)
             M = rows.shape[0]
-        if weight.shape[0] != h.shape[1] or tuple(out.shape) != (M, h.shape[1]):
+        if weight.shape[0] != H or tuple(out.shape) != (M, H):
             raise KernelError(f"layer_norm: h {tuple(h.shape)}, weight {tuple(weight.shape)}, out {tuple(out.shape)}")
-        self._check(self.lib.ra_layer_norm_rows(_ptr(h), _ptr(weight), float(eps), _ptr(out), _ptr(rows), M, h.shape[1],
-                                                _code(out.dtype), self._stream()), "layer_norm")
+        if bias is not None:
+            self._want(bias, "norm bias", torch.float32, 1)
+            if bias.shape[0] != H:
+                raise KernelError(f"layer_norm: bias {tuple(bias.shape)} for rows of {H}")
+        if first is not None:
+            self._want(first, "first delta", out.dtype, 2)
+            if first.shape != h.shape:
+                raise KernelError(f"layer_norm: first delta {tuple(first.shape)} for a stream {tuple(h.shape)}")
+        b, nb, wb, extra, logit, ld_logit = None, 1, None, None, None, 0
+        if isinstance(second, RowSums):
+            b, nb, wb, extra, logit = second.rows, second.count, second.weights, second.extra, second.logits
+            self._want(b, "rows to sum", out.dtype, 2)
+            if tuple(b.shape) != (T * nb, H):
+                raise KernelError(f"layer_norm: {tuple(b.shape)} rows for sums of {nb} into a stream {tuple(h.shape)}")
+            if wb is not None:
+                self._want(wb, "factors", torch.float32, 2)
+                if tuple(wb.shape) != (T, nb):
+                    raise KernelError(f"layer_norm: factors {tuple(wb.shape)} for {T} x {nb} rows")
+            if extra is not None:
+                self._want(extra, "further term", out.dtype, 2)
+                ld_logit = self._want_rows(logit, "gate logits of the further term", torch.float32)
+                if extra.shape != h.shape or tuple(logit.shape) != (T, 1):
+                    raise KernelError(f"layer_norm: further term {tuple(extra.shape)}, its logits {tuple(logit.shape)}")
+        elif second is not None:
+            b = second
+            self._want(b, "second delta", out.dtype, 2)
+            if b.shape != h.shape:
+                raise KernelError(f"layer_norm: second delta {tuple(b.shape)} for a stream {tuple(h.shape)}")
+        self._check(self.lib.ra_stream_layer_norm(_ptr(h), _ptr(first), _ptr(b), int(nb), _ptr(wb), _ptr(extra), _ptr(logit),
+                                                  ld_logit, _ptr(weight), _ptr(bias), float(eps), _ptr(out), _ptr(rows), M, H,
+                                                  _code(out.dtype), self._stream()), "stream_layer_norm")
 
     def stream_rows(self, h, out):
         """out = the rows of h (fp32) in out's type."""
@@ -1752,24 +1846,36 @@ class HipOps:
         _code(dtype)
 
     def latent_kv_prepare(self, z, Q, C, R, wq_norm, wkv_norm, eps, positions, cos, sin, rotary_dim, cq_out,
-                          k_pool, v_pool, slot_mapping):
-        """From the rows z = [a: Q | b: C | r: R | ...]: cq_out = rmsnorm(a) wq_norm; rmsnorm(b) wkv_norm to the value
-        pool's rows and r, its first rotary_dim elements turned by the position (element i with i + rotary_dim / 2),
-        to the key pool's rows that slot_mapping names (pools None: only cq_out)."""
+                          k_pool, v_pool, slot_mapping, q=None, qq_out=None):
+        """From the rows z = [a: Q | b: C | r: R | ...]: cq_out = rmsnorm(a) wq_norm (Q 0: no such part, both None);
+        rmsnorm(b) wkv_norm to the value pool's rows and r, its first rotary_dim elements turned by the position (element i
+        with i + rotary_dim / 2), to the key pool's rows that slot_mapping names (pools None: not written). With q (rows
+        [T, H (D + R)], possibly a column slice of wider rows) and qq_out [T, H, C + R] also latent_q_prepare's rotated
+        part, qq_out[t, h, C:] = q[t, h, D:] turned, by the same kernel."""
         ld = self._want_rows(z, "latent rows")
-        self._want(cq_out, "query latent", z.dtype, 2)
         self._want(positions, "positions", torch.int32, 1)
-        self._want(wq_norm, "query latent norm weight", torch.float32, 1)
         self._want(wkv_norm, "latent norm weight", torch.float32, 1)
         T, rot = z.shape[0], int(rotary_dim)
-        if z.shape[1] < Q + C + R or tuple(cq_out.shape) != (T, Q) or positions.shape[0] != T or wq_norm.shape[0] != Q \
-                or wkv_norm.shape[0] != C:
-            raise KernelError(f"latent_kv_prepare: z {tuple(z.shape)} for {Q} + {C} + {R}, cq {tuple(cq_out.shape)}")
+        if Q:
+            self._want(cq_out, "query latent", z.dtype, 2)
+            self._want(wq_norm, "query latent norm weight", torch.float32, 1)
+            if tuple(cq_out.shape) != (T, Q) or wq_norm.shape[0] != Q:
+                raise KernelError(f"latent_kv_prepare: cq {tuple(cq_out.shape)}, its norm {tuple(wq_norm.shape)} for {Q}")
+        if z.shape[1] < Q + C + R or positions.shape[0] != T or wkv_norm.shape[0] != C:
+            raise KernelError(f"latent_kv_prepare: z {tuple(z.shape)} for {Q} + {C} + {R}")
         if rot:
             self._want(cos, "cos table", torch.float32, 2)
             self._want(sin, "sin table", torch.float32, 2)
             if rot % 2 or rot > R or cos.shape[1] != rot // 2 or sin.shape != cos.shape:
                 raise KernelError(f"latent_kv_prepare: rotary_dim {rot}, tables {tuple(cos.shape)}, key part {R}")
+        ld_q, Hn, D = 0, 0, 0
+        if q is not None:
+            ld_q = self._want_rows(q, "query rows", z.dtype)
+            self._want(qq_out, "prepared q", z.dtype, 3)
+            Hn = qq_out.shape[1]
+            D = q.shape[1] // Hn - R
+            if qq_out.shape[0] != T or qq_out.shape[2] != C + R or D < 0 or tuple(q.shape) != (T, Hn * (D + R)):
+                raise KernelError(f"latent_kv_prepare: q {tuple(q.shape)}, prepared q {tuple(qq_out.shape)}")
         P = 1
         if k_pool is not None:
             self._want(slot_mapping, "slot mapping", torch.int32, 1)
@@ -1779,21 +1885,25 @@ class HipOps:
             P = k_pool.shape[2]
             k_pool = k_pool if R else None               # (no rotated part: the key pool's rows are empty)
         self._check(self.lib.ra_latent_kv_prepare(
-            _ptr(z), ld, T, int(Q), int(C), int(R), _ptr(wq_norm), _ptr(wkv_norm), float(eps), _ptr(positions),
-            _ptr(cos) if rot else None, _ptr(sin) if rot else None, rot, _ptr(cq_out), _ptr(k_pool), _ptr(v_pool),
-            _ptr(slot_mapping) if v_pool is not None else None, P, _code(z.dtype), self._stream()), "latent_kv_prepare")
+            _ptr(z), ld, T, int(Q), int(C), int(R), _ptr(wq_norm) if Q else None, _ptr(wkv_norm), float(eps), _ptr(positions),
+            _ptr(cos) if rot else None, _ptr(sin) if rot else None, rot, _ptr(cq_out) if Q else None, _ptr(k_pool), _ptr(v_pool),
+            _ptr(slot_mapping) if v_pool is not None else None, P, _ptr(q), ld_q, Hn, D, _ptr(qq_out) if q is not None else None,
+            _code(z.dtype), self._stream()), "latent_kv_prepare")
 
     def latent_q_prepare(self, q, q_lat, D, R, positions, cos, sin, rotary_dim, qq_out):
         """qq_out [T, H, C + R] = [q_lat[h, t] | q[t, h, D:] with its first rotary_dim elements turned]; q [T, H (D + R)],
-        q_lat [H, T, C]."""
+        q_lat [H, T, C] (None: the first C elements are there already)."""
         self._want(q, "q", dims=2)
-        self._want(q_lat, "q over the latent", q.dtype, 3)
         self._want(qq_out, "prepared q", q.dtype, 3)
         self._want(positions, "positions", torch.int32, 1)
         T, Hn, CR = qq_out.shape
         C, rot = CR - R, int(rotary_dim)
-        if tuple(q.shape) != (T, Hn * (D + R)) or tuple(q_lat.shape) != (Hn, T, C) or C < 1 or positions.shape[0] != T:
-            raise KernelError(f"latent_q_prepare: q {tuple(q.shape)}, q_lat {tuple(q_lat.shape)}, out {tuple(qq_out.shape)}")
+        if q_lat is not None:
+            self._want(q_lat, "q over the latent", q.dtype, 3)
+            if tuple(q_lat.shape) != (Hn, T, C):
+                raise KernelError(f"latent_q_prepare: q_lat {tuple(q_lat.shape)}, out {tuple(qq_out.shape)}")
+        if tuple(q.shape) != (T, Hn * (D + R)) or C < 1 or positions.shape[0] != T:
+            raise KernelError(f"latent_q_prepare: q {tuple(q.shape)}, out {tuple(qq_out.shape)}")
         if rot:
             self._want(cos, "cos table", torch.float32, 2)
             self._want(sin, "sin table", torch.float32, 2)
@@ -1877,10 +1987,12 @@ class HipOps:
     def moe_route(self, z, bias, top, groups, keep, norm_eps, law="sigmoid_groups"):
         """Router logits z [T, E] (32-bit) -> (ids int32 [T, top], weights fp32 [T, top]). law "softmax_top": the
         largest z + bias are taken and weighed by the softmax over them alone. law "softmax_groups": the choice is made
-        on s = softmax(z) over all experts, a group scores its largest s, the weights are the chosen s as they are."""
-        if law not in ("sigmoid_groups", "softmax_top", "softmax_groups"):
+        on s = softmax(z) over all experts, a group scores its largest s, the weights are the chosen s as they are. law
+        "sigmoid_raw": as "sigmoid_groups", but the weights are the chosen s as they are."""
+        laws = {"sigmoid_groups": 0, "softmax_top": 1, "softmax_groups": 2, "sigmoid_raw": 3}
+        if law not in laws:
             raise KernelError(f"moe_route: no router law {law!r}")
-        self._want(z, "router logits", torch.float32, 2)
+        ld_z = self._want_rows(z, "router logits", torch.float32)
         T, E = z.shape
         self.check_moe_sizes(E, top, groups, keep)
         if bias is not None:
@@ -1889,19 +2001,24 @@ class HipOps:
                 raise KernelError(f"moe_route: correction {tuple(bias.shape)} for {E} experts")
         ids = torch.empty(T, top, dtype=torch.int32, device=self.device)
         weights = torch.empty(T, top, dtype=torch.float32, device=self.device)
-        self._check(self.lib.ra_moe_route_law(_ptr(z), _ptr(bias), T, E, int(top), int(groups), int(keep), float(norm_eps),
+        self._check(self.lib.ra_moe_route_law(_ptr(z), ld_z, _ptr(bias), T, E, int(top), int(groups), int(keep), float(norm_eps),
                                               _ptr(ids), _ptr(weights),
-                                              {"sigmoid_groups": 0, "softmax_top": 1, "softmax_groups": 2}[law], self._stream()),
+                                              laws[law], self._stream()),
                     "moe_route")
         return ids, weights
 
     def moe_experts(self, x, ids, weights, w_gate_up, w_down, activation="silu", limit=0.0, slope=1.702, extra=None,
-                    extra_logits=None):
+                    extra_logits=None, weigh="output", combine=True):
         """sum_k weights[t, k] * down_e(silu(gate_e x_t) * up_e x_t), e = ids[t, k]; w_gate_up [E, 2I, H] (gate
         rows first), w_down [E, H, I]. The pairs are grouped by expert on the device. activation "clamped": an
         expert is down(g sigmoid(slope g) (u + 1)) with g = min(gate x, limit), u = clamp(up x, -limit, limit).
         extra [T, H] with extra_logits [T, 1] (possibly a column of wider rows): one more term of every token's sum,
-        extra[t] * sigmoid(extra_logits[t]), added last in the same 32-bit sum."""
+        extra[t] * sigmoid(extra_logits[t]), added last in the same 32-bit sum (extra_logits in x's type or fp32).
+        weigh "input": a weight multiplies what its expert reads, down_e(act(gate_e (w x), up_e (w x))), and the sum is a
+        plain one. combine False: the sum is not formed; returns RowSums (extra_logits must then be fp32) for whatever forms
+        the stream next."""
+        if weigh not in ("output", "input"):
+            raise KernelError(f"moe_experts: weigh {weigh!r}: 'output' or 'input'")
         if activation not in ("silu", "clamped") or (activation == "clamped" and not limit > 0):
             raise KernelError(f"moe_experts: activation {activation!r} with limit {limit}")
         act = 1 if activation == "clamped" else 0
@@ -1923,12 +2040,13 @@ class HipOps:
             raise KernelError("moe_experts: a further term needs its rows and its gate logits")
         if extra is not None:
             self._want(extra, "further term", x.dtype, 2)
-            ld_logits = self._want_rows(extra_logits, "gate logits of the further term", x.dtype)
+            ld_logits = self._want_rows(extra_logits, "gate logits of the further term")
+            if extra_logits.dtype not in (x.dtype, torch.float32) or (not combine and extra_logits.dtype != torch.float32):
+                raise KernelError(f"moe_experts: gate logits of the further term in {extra_logits.dtype}")
             if tuple(extra.shape) != (T, H) or tuple(extra_logits.shape) != (T, 1):
                 raise KernelError(f"moe_experts: further term {tuple(extra.shape)}, its logits {tuple(extra_logits.shape)}")
-        out = torch.empty(T, H, dtype=x.dtype, device=self.device)
         if n_pairs == 0:
-            return out
+            return torch.empty(T, H, dtype=x.dtype, device=self.device)
         mid = torch.empty(n_pairs, I, dtype=x.dtype, device=self.device)
         y = torch.empty(n_pairs, H, dtype=x.dtype, device=self.device)
 
@@ -1948,13 +2066,24 @@ class HipOps:
         down = up if rows_down == rows_up else plan(rows_down)
         order, tiles, meta, max_tiles, rows = up
         self._check(self.lib.ra_moe_product_act(_ptr(x), _ptr(w_gate_up), _ptr(mid), _ptr(order), _ptr(tiles), _ptr(meta),
-                                                max_tiles, rows, I, H, top, 1, act, float(limit), float(slope), code,
+                                                max_tiles, rows, I, H, top, 1, act, float(limit), float(slope),
+                                                _ptr(weights) if weigh == "input" else None, code,
                                                 self._stream()), "moe_product (gate-up)")
         order, tiles, meta, max_tiles, rows = down
         self._check(self.lib.ra_moe_product(_ptr(mid), _ptr(w_down), _ptr(y), _ptr(order), _ptr(tiles), _ptr(meta),
                                             max_tiles, rows, H, I, 1, 0, code, self._stream()), "moe_product (down)")
-        self._check(self.lib.ra_moe_combine_extra(_ptr(y), _ptr(weights), _ptr(out), T, top, H, _ptr(extra),
-                                                  _ptr(extra_logits), ld_logits, code, self._stream()), "moe_combine")
+        sums = RowSums(y, top, weights if weigh == "output" else None, extra, extra_logits)
+        return self.row_sums(sums) if combine else sums
+
+    def row_sums(self, sums):
+        """The rows [T, H] of RowSums (32-bit sums in their order, rounded to the rows' type)."""
+        y, top, extra = sums.rows, sums.count, sums.extra
+        T, H, code = y.shape[0] // top, y.shape[1], _code(y.dtype)
+        out = torch.empty(T, H, dtype=y.dtype, device=self.device)
+        logits_code = _code(sums.logits.dtype) if extra is not None else code
+        ld_logits = self._want_rows(sums.logits, "gate logits of the further term") if extra is not None else 0
+        self._check(self.lib.ra_moe_combine_extra(_ptr(y), _ptr(sums.weights), _ptr(out), T, top, H, _ptr(extra),
+                                                  _ptr(sums.logits), logits_code, ld_logits, code, self._stream()), "moe_combine")
         return out
 
     # ------------------------------------------------------------------ measurement

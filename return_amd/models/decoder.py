@@ -12,7 +12,7 @@ import torch
 
 from ..parts.block import BLOCKS
 from ..parts.registry import part_class
-from ..parts.runtime import Normed, StreamRows, unscaled
+from ..parts.runtime import Normed, StreamRows, enter_stream
 from ..parts.spec import ModelSpec
 
 
@@ -125,13 +125,8 @@ class Decoder:
             if call.pass_input is not None:
                 h, pending = self.pass_input.forward(h, pending, h_in, call.pass_input)
             if call.add_input:
-                if pending is not None:                   # what the part before left goes into the stream first
-                    delta, factor = unscaled(pending)
-                    if factor != 1.0:
-                        self.rt.ops.residual_add(h, delta, scale=factor)
-                    else:
-                        self.rt.ops.residual_add(h, pending)
-                    pending = None
+                enter_stream(self.rt.ops, h, pending)     # what the part before left goes into the stream first
+                pending = None
                 self.rt.ops.residual_add(h, h_in)
             view = None
             if call.cache is not None:
@@ -150,10 +145,8 @@ class Decoder:
                 post = None
                 if isinstance(pending, Normed):
                     post, pending = pending, None
-                if pending is not None:
-                    delta, factor = unscaled(pending)
-                    self.rt.ops.residual_add(h, delta, scale=factor)
-                    pending = None
+                enter_stream(self.rt.ops, h, pending)
+                pending = None
                 # the next call's first norm may be formed with the sum, if nothing comes between
                 nxt = self.schedule[i + 1] if i + 1 < len(self.schedule) else None
                 norm = None

@@ -181,7 +181,12 @@ class BlendAttention:
     With bias False there are no biases. With qk_norm_eps every head of q and k is divided by its root mean square
     (that eps inside the root) and weighed (roles q_norm, k_norm, [D] for all heads) before it turns. With sink the
     softmax's denominator also holds exp(sink[h]) (role sink, [Hq]): a key that has no value and is not scaled. With
-    fine_weights the softmax's weights enter the product with the values with 16 bits of mantissa in bfloat16.
+    fine_weights the softmax's weights enter the product with the values with 16 bits of mantissa in bfloat16; with
+    sink_one the denominator holds one more 1 (a key of score 0 without a value).
+    With row_norm_eps it is the whole query projection (all heads at once) that is divided by its root mean square and
+    weighed, and the whole key projection likewise (roles q_norm [Hq D], k_norm [Hkv D]), before the heads turn. With gate
+    the heads' results are multiplied element by element by sigmoid(W_g x) (role g_proj, [Hq Dv, W]) in front of the output
+    projection; W_g's rows ride in the first product.
     The blended v is what the cache keeps. The biases are added, the rotation is done and the values are blended in
     32-bit by one kernel that also writes the cache rows. The cache rows of keys and values have one width, the
     larger of D and Dv (in bfloat16 a multiple of 16, so that the matrix-core kernels take it): the stacked weight
@@ -191,8 +196,9 @@ class BlendAttention:
     of its own; take_products() gives up the stacked first weight and the output projection, and run() does what lies
     between the two, on a column slice of wider rows on either side.
     Parameters: hidden_size, num_heads, num_kv_heads, head_dim, value_dim (None: head_dim), scale (None: D^-1/2),
-    bias (True unless given), qk_norm_eps, sink, fine_weights, inner, window, position, value_rows (name of the model's shared part through which the first blending layer hands its
-    values on; None: this layer does not blend), first_of_blend (this layer is that first one).
+    bias (True unless given), qk_norm_eps, row_norm_eps, sink, sink_one, gate, fine_weights, inner, window, position,
+    value_rows (name of the model's shared part through which the first blending layer hands its values on; None: this
+    layer does not blend), first_of_blend (this layer is that first one).
     """
 
     @staticmethod
@@ -206,8 +212,12 @@ class BlendAttention:
             shapes["blend"] = ()
         if params.get("qk_norm_eps") is not None:
             shapes.update({"q_norm": (D,), "k_norm": (D,)})
+        if params.get("row_norm_eps") is not None:
+            shapes.update({"q_norm": (Hq * D,), "k_norm": (Hkv * D,)})
         if params.get("sink"):
             shapes["sink"] = (Hq,)
+        if params.get("gate"):
+            shapes["g_proj"] = (Hq * Dv, H)
         return shapes
 
     @staticmethod
@@ -257,6 +267,9 @@ class BlendAttention:
         rows = [padded("q_proj", self.n_q, self.d), padded("k_proj", self.n_kv, self.d), padded("v_proj", self.n_kv, self.dv)]
         self.inner = bool(params.get("inner"))
         note = (lambda w, **kw: w) if self.inner else rt.product
+        self.gated = bool(params.get("gate"))
+        if self.gated:
+            rows.append(padded("g_proj", self.n_q, self.dv))
         self.w_qkv = note(rt.matrix(torch.cat(rows, dim=0).contiguous()))
         self.bias = None
         if params.get("bias", True):
@@ -266,16 +279,25 @@ class BlendAttention:
         if params.get("qk_norm_eps") is not None:
             self.norms = dict(w_q=rt.vector32(padded("q_norm", 1, self.d)), w_k=rt.vector32(padded("k_norm", 1, self.d)),
                               norm_dim=self.d, eps=float(params["qk_norm_eps"]))
+        self.row_norms = None
+        if params.get("row_norm_eps") is not None:
+            if self.norms or self.bias is not None or self.value_rows is not None:
+                raise ValueError("norms over whole projections are built without biases, norms per head and blended values")
+            self.row_norms = (rt.vector32(padded("q_norm", self.n_q, self.d)), rt.vector32(padded("k_norm", self.n_kv, self.d)),
+                              self.n_q * self.d, self.n_kv * self.d, float(params["row_norm_eps"]))
         self.extras = {}
         if params.get("sink"):
             self.extras["sink_logit"] = rt.vector32(tensors["sink"])
+        elif params.get("sink_one"):
+            self.extras["sink"] = True
         if params.get("fine_weights"):
             self.extras["fine_weights"] = True
         o = tensors["o_proj"].reshape(W, self.n_q, self.dv)
         o_pad = torch.zeros(W, self.n_q, self.dp, dtype=o.dtype, device=o.device)
         o_pad[:, :, :self.dv] = o
-        self.w_o = note(rt.matrix(o_pad.reshape(W, self.n_q * self.dp).contiguous()), **({} if self.inner else {"residual": True}))
-        self.in_width, self.out_width = (self.n_q + 2 * self.n_kv) * self.dp, self.n_q * self.dp
+        self.w_o = note(rt.matrix(o_pad.reshape(W, self.n_q * self.dp).contiguous()), **({} if self.inner or self.gated else {"residual": True}))
+        self.qkv_width = (self.n_q + 2 * self.n_kv) * self.dp
+        self.in_width, self.out_width = self.qkv_width + (self.n_q * self.dp if self.gated else 0), self.n_q * self.dp
         if not self.inner:
             self.first_product = (self.w_qkv, False)      # (see PagedAttention)
             self.last_product = self.w_o
@@ -301,9 +323,11 @@ class BlendAttention:
         return project(o, self.w_o)
 
     def run(self, qkv, step, cache, write_cache, out, out_scale=1.0):
-        """From the first product's rows, [T, (Hq + 2 Hkv) * D] (columns of wider rows are fine), to the heads' results
-        side by side times out_scale in out, [T, Hq * D] (columns of wider rows too)."""
+        """From the first product's rows, [T, (Hq + 2 Hkv) * D (+ Hq * D gates)] (columns of wider rows are fine), to the
+        heads' results side by side times out_scale in out, [T, Hq * D] (columns of wider rows too)."""
         rt, ops = self.rt, self.rt.ops
+        gate = qkv[:, self.qkv_width:self.in_width] if self.gated else None
+        qkv = qkv[:, :self.qkv_width]
         T, Hq, Hkv, D = qkv.shape[0], self.n_q, self.n_kv, self.dp
         tables = step.groups[cache.group]
         cos, sin, rot = self.position.tables() if self.position is not None else (None, None, 0)
@@ -315,12 +339,17 @@ class BlendAttention:
             else:
                 first = self.value_rows.get(step)
         q = rt.empty(T, Hq, D)
-        ops.qkv_blend_prepare(qkv, Hq, Hkv, D, self.bias, step.positions, cos, sin, rot, q,
-                              cache.k_pool if write_cache else None, cache.v_pool if write_cache else None,
-                              tables.slot_mapping, first, self.blend, **self.norms)
+        pools = (cache.k_pool, cache.v_pool) if write_cache else (None, None)
+        if self.row_norms is not None:
+            ops.qkv_rows_prepare(qkv, Hq, Hkv, D, *self.row_norms, step.positions, cos, sin, rot, q, *pools, tables.slot_mapping)
+        else:
+            ops.qkv_blend_prepare(qkv, Hq, Hkv, D, self.bias, step.positions, cos, sin, rot, q, *pools, tables.slot_mapping,
+                                  first, self.blend, **self.norms)
         extras = self.extras if out_scale == 1.0 else dict(self.extras, out_scale=float(out_scale))
         ops.attention(q, out.view(T, Hq, D), cache.k_pool, cache.v_pool, step, cache.group, self.scale,
                       int(self.window) if self.window else 0, **extras)
+        if gate is not None:
+            ops.gate_rows(out, gate)
 
 
 register_part("mixer", "blend_attention", BlendAttention)
@@ -424,20 +453,27 @@ class LatentAttention:
     head. The products with W_uk and W_uv are moved to the query's side, where they cost one row per new token
     instead of one per key read:  q_h . (W_uk,h c) = (W_uk,h^T q_h) . c  and  sum_j p_j W_uv,h c_j = W_uv,h (sum_j p_j c_j),
     so every head reads the same rows [c | rot(k_r)] with a query of C + R elements, and one kernel serves
-    whole prompts, portions and single tokens.
+    whole prompts, portions and single tokens. Both products write where their result is wanted: into the first C elements
+    of every head's query, and (without a gate) into the heads' places side by side.
+    With direct_q there is no query latent: q = W_q x (role q), whose rows ride in the first product, and one kernel turns
+    q's rotated parts beside the token's key part.
+    A position encoding that pairs neighbours (2i with 2i + 1) is served by the order of rows: those of W_uq (or W_q) and
+    W_dkv that make the rotated parts are put into the order [0, 2, 4, ... | 1, 3, 5, ...] at load, the same for queries and
+    keys, so the scores are what they were and the kernels pair element i with i + rotary_dim / 2.
     Parameters: hidden_size, num_heads, head_dim (D), rot_dim (R; 0: no rotated part at all, the key pool's rows
     are empty), value_dim, q_rank, kv_rank, scale, eps, position (a rotary encoding of the model's over the R
     elements; None: none), sink, gate (each off unless true), window (w: position i reads j with 0 <= i - j < w;
-    None: every j <= i); q_rank None: what the stored tensors have.
+    None: every j <= i), direct_q; q_rank None: what the stored tensors have.
     """
 
     @staticmethod
     def tensor_shapes(params):
         W, H, D, R, Dv = (params["hidden_size"], params["num_heads"], params["head_dim"], params["rot_dim"],
                           params["value_dim"])
-        Q, C = params["q_rank"], params["kv_rank"]
-        shapes = {"dq": (Q, W), "dq_norm": (Q,), "uq": (H * (D + R), Q), "dkv": (C + R, W), "dkv_norm": (C,),
-                  "uk": (H * D, C), "uv": (H * Dv, C), "o": (W, H * Dv)}
+        Q, C = params.get("q_rank"), params["kv_rank"]
+        shapes = {"q": (H * (D + R), W)} if params.get("direct_q") else \
+            {"dq": (Q, W), "dq_norm": (Q,), "uq": (H * (D + R), Q)}
+        shapes.update({"dkv": (C + R, W), "dkv_norm": (C,), "uk": (H * D, C), "uv": (H * Dv, C), "o": (W, H * Dv)})
         if params.get("sink"):
             shapes["sink"] = (H,)
         if params.get("gate"):
@@ -456,8 +492,9 @@ class LatentAttention:
         self.rt = rt
         self.hidden = W = int(params["hidden_size"])
         self.H, self.D, self.R, self.Dv = (int(params[k]) for k in ("num_heads", "head_dim", "rot_dim", "value_dim"))
-        self.Q, self.C = int(tensors["dq"].shape[0]), int(params["kv_rank"])
-        if tensors["uq"].shape[1] != self.Q or tensors["dq_norm"].shape[0] != self.Q:
+        self.direct = bool(params.get("direct_q"))
+        self.Q, self.C = 0 if self.direct else int(tensors["dq"].shape[0]), int(params["kv_rank"])
+        if not self.direct and (tensors["uq"].shape[1] != self.Q or tensors["dq_norm"].shape[0] != self.Q):
             raise ValueError("the query latent's two maps and its norm differ in the latent's size")
         self.scale = float(params["scale"]) if params.get("scale") is not None else (self.D + self.R) ** -0.5
         self.eps = float(params["eps"])
@@ -470,8 +507,17 @@ class LatentAttention:
             rt.ops.check_attention_latent_sizes(self.H, self.C, self.R, rt.dtype)
         self.sink = rt.vector32(tensors["sink"]) if params.get("sink") else None
         self.window = int(params["window"]) if params.get("window") else None
-        # x goes into one product: [W_dq; W_dkv; W_g], rows filled up with zeros to a multiple of 16
-        rows = [rt.matrix(tensors["dq"]), rt.matrix(tensors["dkv"])]
+        # the order of the rotated rows (see above): of every head of q, and of the shared key part
+        w_q, w_dkv = rt.matrix(tensors["q" if self.direct else "uq"]), rt.matrix(tensors["dkv"])
+        if self.position is not None and getattr(self.position, "pairing", "half") == "interleaved":
+            n = self.position.tables()[2]
+            order = torch.cat([torch.arange(0, n, 2), torch.arange(1, n, 2), torch.arange(n, self.R)]).to(rt.device)
+            w_q = w_q.view(self.H, self.D + self.R, -1)
+            w_q = torch.cat([w_q[:, :self.D], w_q[:, self.D:][:, order]], dim=1).reshape(self.H * (self.D + self.R), -1).contiguous()
+            w_dkv = torch.cat([w_dkv[:self.C], w_dkv[self.C:][order]], dim=0).contiguous()
+        # x goes into one product: [W_q or W_dq; W_dkv; W_g], rows filled up with zeros to a multiple of 16
+        rows = [w_q if self.direct else rt.matrix(tensors["dq"]), w_dkv]
+        self.at_kv = rows[0].shape[0]                    # columns of the product's rows in front of [C | R]
         self.gated = bool(params.get("gate"))
         if self.gated:
             rows.append(rt.matrix(tensors["gate"]))
@@ -479,8 +525,10 @@ class LatentAttention:
         if pad:
             rows.append(torch.zeros(pad, W, dtype=rt.dtype, device=rt.device))
         self.w_in = rt.product(torch.cat(rows, dim=0).contiguous())
-        self.w_dq_norm, self.w_dkv_norm = rt.vector32(tensors["dq_norm"]), rt.vector32(tensors["dkv_norm"])
-        self.w_uq = rt.product(rt.matrix(tensors["uq"]))
+        self.w_dkv_norm = rt.vector32(tensors["dkv_norm"])
+        self.w_dq_norm = self.w_uq = None
+        if not self.direct:
+            self.w_dq_norm, self.w_uq = rt.vector32(tensors["dq_norm"]), rt.product(w_q)
         # per head: W_uk,h [D, C] (q's unrotated part times it gives the query over c) and W_uv,h^T [C, Dv]
         self.w_uk = rt.matrix(tensors["uk"]).view(self.H, self.D, self.C).contiguous()
         self.w_uv_t = rt.matrix(tensors["uv"]).view(self.H, self.Dv, self.C).transpose(1, 2).contiguous()
@@ -497,28 +545,37 @@ class LatentAttention:
 
     def forward(self, x, step, cache, write_cache=True):
         rt, ops = self.rt, self.rt.ops
-        T, H, D, R, C, Q = x.shape[0], self.H, self.D, self.R, self.C, self.Q
+        T, H, D, R, C, Q, Dv = x.shape[0], self.H, self.D, self.R, self.C, self.Q, self.Dv
         tables = step.groups[cache.group]
-        z = ops.linear(x, self.w_in)                                  # [T, Q | C + R | H | pad]
+        z = ops.linear(x, self.w_in)                                  # [T, H (D + R) or Q | C + R | H | pad]
         cos, sin, rot = self.position.tables() if self.position is not None else (None, None, 0)
-        cq = rt.empty(T, Q)
-        ops.latent_kv_prepare(z, Q, C, R, self.w_dq_norm, self.w_dkv_norm, self.eps, step.positions, cos, sin, rot, cq,
-                              cache.k_pool if write_cache else None, cache.v_pool if write_cache else None,
-                              tables.slot_mapping)
-        q = ops.linear(cq, self.w_uq)                                 # [T, H (D + R)]
-        q_flat = q.view(T, H, D + R)[:, :, :D].transpose(0, 1)        # [H, T, D], a view
-        q_lat = ops.batched_product(q_flat, self.w_uk)                # [H, T, C]
+        at, kv = self.at_kv, (cache.k_pool, cache.v_pool) if write_cache else (None, None)
         qq = rt.empty(T, H, C + R)
-        ops.latent_q_prepare(q, q_lat, D, R, step.positions, cos, sin, rot, qq)
+        if self.direct:
+            q = z[:, :at]                                             # [T, H (D + R)], columns of z
+            ops.latent_kv_prepare(z[:, at:at + C + R], 0, C, R, None, self.w_dkv_norm, self.eps, step.positions, cos, sin, rot,
+                                  None, *kv, tables.slot_mapping, q=q if R else None, qq_out=qq)
+        else:
+            cq = rt.empty(T, Q)
+            ops.latent_kv_prepare(z, Q, C, R, self.w_dq_norm, self.w_dkv_norm, self.eps, step.positions, cos, sin, rot, cq,
+                                  *kv, tables.slot_mapping)
+            q = ops.linear(cq, self.w_uq)                             # [T, H (D + R)]
+            if R:
+                ops.latent_q_prepare(q, None, D, R, step.positions, cos, sin, rot, qq)
+        q_flat = q.unflatten(1, (H, D + R))[:, :, :D].transpose(0, 1)          # [H, T, D], a view
+        ops.batched_product(q_flat, self.w_uk, out=qq.transpose(0, 1)[:, :, :C])
         o_lat = rt.empty(H, T, C)
         if self.window:
             ops.attention_latent(qq, o_lat, cache.k_pool, cache.v_pool, step, cache.group, self.scale, self.sink,
                                  window=self.window)
         else:
             ops.attention_latent(qq, o_lat, cache.k_pool, cache.v_pool, step, cache.group, self.scale, self.sink)
-        o = ops.batched_product(o_lat, self.w_uv_t)                   # [H, T, Dv]
-        y = rt.empty(T, H * self.Dv)
-        ops.heads_gate(o, z[:, Q + C + R:Q + C + R + H] if self.gated else None, y)
+        y = rt.empty(T, H * Dv)
+        if self.gated:
+            o = ops.batched_product(o_lat, self.w_uv_t)               # [H, T, Dv]
+            ops.heads_gate(o, z[:, at + C + R:at + C + R + H], y)
+        else:
+            ops.batched_product(o_lat, self.w_uv_t, out=y.view(T, H, Dv).transpose(0, 1))
         return ops.linear(y, self.w_o)
 
 

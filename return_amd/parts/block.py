@@ -20,7 +20,7 @@ from __future__ import annotations
 
 import inspect
 
-from .runtime import Normed, NormSink, Pair, ResidualSink, Scaled, StreamRows, unscaled
+from .runtime import Normed, NormSink, Pair, ResidualSink, Scaled, StreamRows, enter_stream
 
 
 _TAKES_SINK = {}
@@ -247,21 +247,24 @@ class PrePostNormBlock:
 
 
 class ParallelPreNormBlock:
-    """A layer whose two sublayers run side by side on the same stream, each behind a norm of its own, the
-    feed-forward optional:
+    """A layer whose two sublayers run side by side on the same stream, the feed-forward optional:
 
         h += mixer(mixer_norm(h)) + feed_forward(feed_forward_norm(h))
 
-    Parts by name: mixer_norm, mixer and, both or neither, feed_forward_norm + feed_forward. Both norms are formed in
-    one pass over the rows, which also adds what the layer before left pending; the layer's own two outputs are
-    handed on as a Pair for whatever forms the stream next."""
+    Parts by name: mixer_norm, mixer and, each optional, feed_forward and feed_forward_norm (not there: the feed-forward
+    reads what the mixer reads, one norm serves both). Two norms are formed in one pass over the rows, which also adds
+    what the layer before left pending; the layer's own two outputs are handed on as a Pair for whatever forms the stream
+    next, the feed-forward's as RowSums where the norm that follows forms such sums itself."""
 
     def __init__(self, spec, build):
         self.mixer_norm = build("mixer_norm")
         self.mixer = build("mixer")
         self.feed_forward = build("feed_forward") if "feed_forward" in spec.parts else None
-        self.feed_forward_norm = build("feed_forward_norm") if self.feed_forward is not None else None
-        self._plain = all(n is None or (hasattr(n, "weight") and hasattr(n, "eps") and getattr(n, "size", None))
+        self.feed_forward_norm = build("feed_forward_norm") if self.feed_forward is not None and \
+            "feed_forward_norm" in spec.parts else None
+        # the decoder tells a block that names its first norm what takes its output; no product forms that norm here
+        self.first_norm = self.mixer_norm
+        self._plain = not getattr(self.mixer_norm, "centered", False) and all(n is None or (hasattr(n, "weight") and hasattr(n, "eps") and getattr(n, "size", None))
                           for n in (self.mixer_norm, self.feed_forward_norm))
 
     def cache_spec(self):
@@ -270,11 +273,13 @@ class ParallelPreNormBlock:
     def step_needs(self):
         return self.mixer.step_needs() if hasattr(self.mixer, "step_needs") else {}
 
-    def forward(self, h, pending, step, cache, write_cache=True):
+    def forward(self, h, pending, step, cache, write_cache=True, after=None):
         rt = self.mixer_norm.rt
         if self.feed_forward is None:
             return h, self.mixer.forward(self.mixer_norm.forward(h, pending), step, cache, write_cache)
-        if self._plain and hasattr(rt.ops, "add_rmsnorm_pair") and (pending is None or isinstance(pending, Pair)
+        if self.feed_forward_norm is None:
+            x1 = x2 = self.mixer_norm.forward(h, pending)
+        elif self._plain and hasattr(rt.ops, "add_rmsnorm_pair") and (pending is None or isinstance(pending, Pair)
                                                                     or hasattr(pending, "dtype")):
             a, b = (pending.first, pending.second) if isinstance(pending, Pair) else (pending, None)
             x1, x2 = rt.empty(h.shape[0], h.shape[1]), rt.empty(h.shape[0], h.shape[1])
@@ -284,8 +289,9 @@ class ParallelPreNormBlock:
             x1 = self.mixer_norm.forward(h, pending)
             x2 = self.feed_forward_norm.forward(h, None)
         y = self.mixer.forward(x1, step, cache, write_cache)
-        f = self.feed_forward.forward(x2, step)
-        return h, Pair(y, f)
+        if getattr(self.feed_forward, "leaves_sums", False) and after is not None and getattr(after[0], "takes_row_sums", False):
+            return h, Pair(y, self.feed_forward.forward(x2, step, combine=False))
+        return h, Pair(y, self.feed_forward.forward(x2, step))
 
 
 class PostNormBlock:
@@ -326,12 +332,7 @@ class PostNormBlock:
         if isinstance(pending, StreamRows):
             x = pending.tensor
         else:
-            if isinstance(pending, Pair):
-                rt.ops.residual_add(h, pending.first)
-                pending = pending.second
-            delta, factor = unscaled(pending)
-            if delta is not None:
-                rt.ops.residual_add(h, delta, scale=factor)
+            enter_stream(rt.ops, h, pending)
             x = h
             if rt.dtype != h.dtype:
                 x = rt.empty(h.shape[0], h.shape[1])

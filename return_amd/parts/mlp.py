@@ -75,3 +75,36 @@ class SquaredReLU:
 
 
 register_part("feed_forward", "relu2", SquaredReLU)
+
+
+class ClampedGLU:
+    """Dense feed-forward with clamped halves, no biases: down(g sigmoid(slope g) (u + 1)) with g = min(gate(x), limit),
+    u = clamp(up(x), -limit, limit). Params hidden_size, intermediate_size, limit, slope (1.702 unless given)."""
+
+    @staticmethod
+    def tensor_shapes(params):
+        H, I = params["hidden_size"], params["intermediate_size"]
+        return {"gate_proj": (I, H), "up_proj": (I, H), "down_proj": (H, I)}
+
+    @staticmethod
+    def random_init(params, role):
+        return "matrix"
+
+    def __init__(self, params, tensors, rt, shared=None):
+        self.rt = rt
+        self.inter = int(params["intermediate_size"])
+        self.limit, self.slope = float(params["limit"]), float(params.get("slope", 1.702))
+        if not self.limit > 0:
+            raise ValueError(f"clamped feed-forward: limit {self.limit} must be positive")
+        self.w_gate_up = rt.product(torch.cat([rt.matrix(tensors["gate_proj"]), rt.matrix(tensors["up_proj"])],
+                                              dim=0).contiguous())
+        self.w_down = rt.product(rt.matrix(tensors["down_proj"]))
+
+    def forward(self, x, step=None):
+        ops = self.rt.ops
+        a = self.rt.empty(x.shape[0], self.inter)
+        ops.gated_rows(ops.linear(x, self.w_gate_up), a, "clamped", self.limit, self.slope)
+        return ops.linear(a, self.w_down)
+
+
+register_part("feed_forward", "clamped_glu", ClampedGLU)

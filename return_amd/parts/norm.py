@@ -8,8 +8,10 @@ is multiplied into the 32-bit weight when the part is built).
 """
 from __future__ import annotations
 
+import torch
+
 from .registry import register_part
-from .runtime import Pair, ScaledRows, StreamRows, unscaled
+from .runtime import Pair, RowSums, Scaled, ScaledRows, StreamRows, unscaled
 
 
 class RMSNorm:
@@ -27,7 +29,6 @@ class RMSNorm:
         # a weight stored as its distance from `offset`: drawn so that offset + w lies around one
 
         def draw(shape, gen):
-            import torch
             return (1.0 - offset) + 0.1 * torch.randn(*shape, generator=gen, dtype=torch.float32, device=gen.device)
         return draw
 
@@ -67,17 +68,24 @@ class RMSNorm:
 
 
 class LayerNorm:
-    """y = (x - mean) / sqrt(variance + eps) * w over the last axis, the variance the mean of the squared deviations; a
-    weight and no bias, all in 32-bit, rounded to the compute dtype at the end."""
+    """y = (x - mean) / sqrt(variance + eps) * w (+ b with params bias: role "bias") over the last axis, the variance the
+    mean of the squared deviations, all in 32-bit, rounded to the compute dtype at the end. What is pending, also two
+    outputs (Pair) and sums not yet formed (RowSums), is added into the stream by the same kernel."""
 
     centered = True             # (an arrangement that puts a norm behind a sublayer asks which kind it has)
+    takes_row_sums = True       # (a feed-forward in front may leave its sums to forward's delta)
 
     @staticmethod
     def tensor_shapes(params):
-        return {"weight": (params["size"],)}
+        shapes = {"weight": (params["size"],)}
+        if params.get("bias"):
+            shapes["bias"] = (params["size"],)
+        return shapes
 
     @staticmethod
     def random_init(params, role):
+        if role == "bias":
+            return lambda shape, gen: 0.1 * torch.randn(*shape, generator=gen, dtype=torch.float32, device=gen.device)
         return "norm"
 
     def __init__(self, params, tensors, rt, shared=None):
@@ -85,20 +93,26 @@ class LayerNorm:
         self.eps = float(params["eps"])
         self.rt = rt
         self.weight = rt.vector32(tensors["weight"])
+        self.bias = rt.vector32(tensors["bias"]) if params.get("bias") else None
 
     def forward(self, h, delta=None, out_rows=None):
-        """h (fp32 [T, size]) += delta in place; returns norm(h) (only rows out_rows, if given)."""
+        """h (fp32 [T, size]) += delta in place (not where only some rows are wanted: then h is left as it is); returns
+        norm(h) (only rows out_rows, if given)."""
         ops = self.rt.ops
+        first = second = None
         if isinstance(delta, StreamRows):                   # (nothing is left to add)
             delta = None
         if isinstance(delta, Pair):
-            ops.residual_add(h, delta.first)
-            delta = delta.second
-        delta, factor = unscaled(delta)
-        if delta is not None:
-            ops.residual_add(h, delta, scale=factor)
+            first, second = delta.first, delta.second
+        elif isinstance(delta, RowSums):
+            second = delta
+        elif isinstance(delta, Scaled):
+            ops.residual_add(h, delta.tensor, scale=delta.factor)
+        else:
+            first = delta
         out = self.rt.empty(h.shape[0] if out_rows is None else out_rows.shape[0], self.size)
-        ops.layer_norm(h, self.weight, self.eps, out, out_rows)
+        kw = {k: v for k, v in (("bias", self.bias), ("first", first), ("second", second)) if v is not None}
+        ops.layer_norm(h, self.weight, self.eps, out, out_rows, **kw)
         return out
 
 

@@ -30,6 +30,8 @@ Interfaces (``rt`` is the return_amd.parts.runtime.Runtime of the engine):
                 output projection), in_width / out_width their outer sizes; run(z, step, cache, write_cache, out,
                 out_scale) does what lies between them, z and out being columns of wider rows
   feed_forward  forward(x, step) -> y
+                optional: leaves_sums = True and forward(x, step, combine=True): asked with combine False, which an
+                arrangement does where the norm that follows has takes_row_sums = True, y may be RowSums
 
   Optional, for a mixer or feed-forward whose input goes into ONE product and whose output comes out
   of ONE (then the kernel set may finish the norms around the part inside those products, or form the
@@ -42,7 +44,8 @@ Interfaces (``rt`` is the return_amd.parts.runtime.Runtime of the engine):
                     sink.project(a, w) instead of ops.linear(a, w) (it may be ScaledRows or Slabs and
                     goes to the next norm as it is). A part without that parameter is never given one.
   and for a norm: weight, eps attributes (a plain RMS norm whose 1/rms a product can apply) and
-                takes_slabs = True if forward's delta may be Slabs.
+                takes_slabs = True if forward's delta may be Slabs; takes_row_sums = True if it may be RowSums,
+                alone or as a Pair's second.
   position      an object the mixer uses; rotary ones offer tables() -> (cos, sin, rotary_dim)
                 and every one offers apply(q, k, positions) in place on [T, heads, D].
                 One with more than one axis per token declares step_needs() ->

@@ -98,11 +98,39 @@ class Pair:
         return self.first.shape
 
 
+class RowSums:
+    """A part's output left as the rows whose sums it is: row t is sum_k weights[t, k] * rows[t * count + k] (weights None:
+    factors of one) + extra[t] * sigmoid(logits[t]) (extra None: no such term), k in order, in 32-bit. A layer norm that
+    adds the pending output into the stream forms the sums itself; the kernel set's row_sums forms them for anyone else."""
+    __slots__ = ("rows", "count", "weights", "extra", "logits")
+
+    def __init__(self, rows, count, weights=None, extra=None, logits=None):
+        self.rows, self.count, self.weights, self.extra, self.logits = rows, int(count), weights, extra, logits
+
+    @property
+    def shape(self):
+        return (self.rows.shape[0] // self.count, self.rows.shape[1])
+
+
 def unscaled(delta):
     """(rows, factor) of a pending output, Scaled or plain (None stays None)."""
     if isinstance(delta, Scaled):
         return delta.tensor, delta.factor
     return delta, 1.0
+
+
+def enter_stream(ops, h, pending):
+    """h += pending, whatever form the pending output has (None: nothing)."""
+    if pending is None or isinstance(pending, StreamRows):
+        return
+    if isinstance(pending, Pair):
+        enter_stream(ops, h, pending.first)
+        enter_stream(ops, h, pending.second)
+        return
+    if isinstance(pending, RowSums):
+        pending = ops.row_sums(pending)
+    delta, factor = unscaled(pending)
+    ops.residual_add(h, delta, scale=factor)
 
 
 class ResidualSink:

@@ -320,8 +320,8 @@ def test_the_stream_after_every_layer_is_the_plain_one(model):
     seen = []
     from return_amd.parts.runtime import Pair
     for i, block in enumerate(runner.model.blocks):
-        def wrapped(h, pending, step, cache, write_cache=True, _f=block.forward):
-            h, out = _f(h, pending, step, cache, write_cache)
+        def wrapped(h, pending, step, cache, write_cache=True, _f=block.forward, **kw):
+            h, out = _f(h, pending, step, cache, write_cache, **kw)
             total = h.clone()
             for part in ((out.first, out.second) if isinstance(out, Pair) else (out,)):
                 total += part.float()

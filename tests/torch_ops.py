@@ -10,7 +10,7 @@ from __future__ import annotations
 
 import torch
 
-from return_amd.parts.runtime import ScaledRows, Slabs
+from return_amd.parts.runtime import RowSums, ScaledRows, Slabs
 
 
 def _pool_rows(pool, pages, n):
@@ -265,7 +265,7 @@ class TorchOps:
                 c = c.masked_fill(~stay[:, :, None].expand(T, groups, per).reshape(T, E), float("-inf"))
             ids = c.topk(top, dim=-1).indices
             return ids.int(), s.gather(1, ids)
-        s = torch.sigmoid(z.float())
+        s = torch.sigmoid(z.float())                        # ("sigmoid_raw": the chosen s are the weights)
         c = s + (bias if bias is not None else 0.0)
         if groups > 1 and keep < groups:
             per = E // groups
@@ -275,31 +275,57 @@ class TorchOps:
             c = c.masked_fill(~stay[:, :, None].expand(T, groups, per).reshape(T, E), float("-inf"))
         ids = c.topk(top, dim=-1).indices
         w = s.gather(1, ids)
+        if law == "sigmoid_raw":
+            return ids.int(), w
         return ids.int(), w / (w.sum(-1, keepdim=True) + norm_eps)
 
     def moe_experts(self, x, ids, weights, w_gate_up, w_down, activation="silu", limit=0.0, slope=1.702, extra=None,
-                    extra_logits=None):
+                    extra_logits=None, weigh="output", combine=True):
         T, H = x.shape
-        I = w_gate_up.shape[1] // 2
-        out = torch.zeros(T, H, dtype=torch.float32, device=x.device)
+        I, top = w_gate_up.shape[1] // 2, ids.shape[1]
+        y = torch.empty(T * top, H, dtype=x.dtype, device=x.device)
         for t in range(T):
-            for k in range(ids.shape[1]):
+            for k in range(top):
                 e = int(ids[t, k])
-                gu = (x[t].float() @ w_gate_up[e].float().t()).to(x.dtype).float()
+                gu = x[t].float() @ w_gate_up[e].float().t()
+                if weigh == "input":
+                    gu = weights[t, k] * gu
+                gu = gu.to(x.dtype).float()
                 if activation == "clamped":
                     g, u = gu[:I].clamp(max=limit), gu[I:].clamp(-limit, limit)
                     a = (g * torch.sigmoid(slope * g) * (u + 1.0)).to(x.dtype)
                 else:
                     a = (gu[:I] * torch.sigmoid(gu[:I]) * gu[I:]).to(x.dtype)
-                out[t] += weights[t, k] * (a.float() @ w_down[e].float().t()).to(x.dtype).float()
-        if extra is not None:                               # one more term of every token's sum, behind its gate
-            out += extra.float() * torch.sigmoid(extra_logits.float())
-        return out.to(x.dtype)
+                y[t * top + k] = (a.float() @ w_down[e].float().t()).to(x.dtype)
+        sums = RowSums(y, top, weights if weigh == "output" else None, extra, extra_logits)
+        return self.row_sums(sums) if combine else sums
+
+    @staticmethod
+    def _row_sums32(s):
+        y = s.rows.float().view(-1, s.count, s.rows.shape[1])
+        v = (y if s.weights is None else y * s.weights[:, :, None]).sum(1)
+        if s.extra is not None:                             # one more term of every token's sum, behind its gate
+            v = v + s.extra.float() * torch.sigmoid(s.logits.float())
+        return v
+
+    def row_sums(self, sums):
+        return self._row_sums32(sums).to(sums.rows.dtype)
 
     def clamped_mul(self, gu, out, limit, slope=1.702):
-        """gu [T, >= 2 I] (gate columns first) -> out [T, I] = g sigmoid(slope g) (u + 1), g = min(gate, limit),
-        u = clamp(up, -limit, limit)."""
+        return self.gated_rows(gu, out, "clamped", limit, slope)
+
+    def gate_rows(self, o, gate):
+        o.copy_((o.float() * torch.sigmoid(gate.float())).to(o.dtype))
+        return o
+
+    def gated_rows(self, gu, out, activation="silu", limit=0.0, slope=1.702):
+        """gu [T, >= 2 I] (gate columns first) -> out [T, I] = silu(gate) up or, "clamped", g sigmoid(slope g) (u + 1),
+        g = min(gate, limit), u = clamp(up, -limit, limit)."""
         I = out.shape[1]
+        if activation == "silu":
+            g = gu[:, :I].float()
+            out.copy_((g * torch.sigmoid(g) * gu[:, I:2 * I].float()).to(out.dtype))
+            return out
         g, u = gu[:, :I].float().clamp(max=limit), gu[:, I:2 * I].float().clamp(-limit, limit)
         out.copy_((g * torch.sigmoid(slope * g) * (u + 1.0)).to(out.dtype))
         return out
@@ -343,6 +369,23 @@ class TorchOps:
         page, row = slot_mapping.long() // P, slot_mapping.long() % P
         k_pool[page, :, row] = k.to(k_pool.dtype)
         v_pool[page, :, row] = v.reshape(T, n_kv, D).to(v_pool.dtype)
+
+    def qkv_rows_prepare(self, qkv, n_q, n_kv, D, w_q, w_k, q_size, k_size, eps, positions, cos, sin, rotary_dim, q_out,
+                         k_pool, v_pool, slot_mapping):
+        """Norms over the whole query and key parts of a row (sums of squares over q_size and k_size true elements)."""
+        T, x = qkv.shape[0], qkv.float()
+
+        def part(a, n, w, size):
+            v = x[:, a:a + n * D]
+            v = v / torch.sqrt((v * v).sum(-1, keepdim=True) / size + eps) * w
+            return self._turn(v.reshape(T, n, D), positions, cos, sin, rotary_dim)
+        q_out.copy_(part(0, n_q, w_q, q_size).to(q_out.dtype))
+        if k_pool is None:
+            return
+        P = k_pool.shape[2]
+        page, row = slot_mapping.long() // P, slot_mapping.long() % P
+        k_pool[page, :, row] = part(n_q * D, n_kv, w_k, k_size).to(k_pool.dtype)
+        v_pool[page, :, row] = x[:, (n_q + n_kv) * D:].reshape(T, n_kv, D).to(v_pool.dtype)
 
     def scalar_rule(self, qkv, dt, a_log, dt_bias, skip, gate, norm_w, norm_groups, eps, state, step, out, H, G, D, V):
         """S <- exp(-exp(a_log) delta) S + delta k v^T, o = S^T q + skip v with delta = softplus(dt + dt_bias);
@@ -478,10 +521,17 @@ class TorchOps:
         if out is not None:
             out.copy_(h.to(out.dtype))
 
-    def layer_norm(self, h, weight, eps, out, rows=None):
-        v = h if rows is None else h[rows.long()]
+    def layer_norm(self, h, weight, eps, out, rows=None, bias=None, first=None, second=None):
+        v = h if first is None else h + first.float()
+        if second is not None:
+            v = v + (self._row_sums32(second) if isinstance(second, RowSums) else second.float())
+        if rows is None:
+            h.copy_(v)
+        else:
+            v = v[rows.long()]
         c = v - v.mean(-1, keepdim=True)
-        out.copy_((c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight).to(out.dtype))
+        c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight
+        out.copy_((c if bias is None else c + bias).to(out.dtype))
 
     def stream_rows(self, h, out):
         out.copy_(h.to(out.dtype))
@@ -530,15 +580,21 @@ class TorchOps:
         self.depth_mix(results, count, weights, out, norm_weight, norm_eps, normed)
 
     # ---- attention over a latent row per token
-    def batched_product(self, a, b):
-        """[B, M, K] x [B, K, N] -> [B, M, N], rounded to a's dtype."""
-        return torch.bmm(a.float(), b.float()).to(a.dtype)
+    def batched_product(self, a, b, out=None):
+        """[B, M, K] x [B, K, N] -> [B, M, N], rounded to a's dtype (into out, if given)."""
+        y = torch.bmm(a.float(), b.float()).to(a.dtype)
+        return y if out is None else out.copy_(y)
 
     def latent_kv_prepare(self, z, Q, C, R, wq_norm, wkv_norm, eps, positions, cos, sin, rotary_dim, cq_out,
-                          k_pool, v_pool, slot_mapping):
+                          k_pool, v_pool, slot_mapping, q=None, qq_out=None):
         def norm(x, w):
             return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w
-        cq_out.copy_(norm(z[:, :Q].float(), wq_norm).to(cq_out.dtype))
+        if Q:
+            cq_out.copy_(norm(z[:, :Q].float(), wq_norm).to(cq_out.dtype))
+        if q is not None:
+            T, H = qq_out.shape[:2]
+            part = q.reshape(T, H, -1)[:, :, q.shape[1] // H - R:].float()
+            qq_out[:, :, C:] = self._turn(part, positions, cos, sin, rotary_dim).to(qq_out.dtype)
         if k_pool is None:
             return
         c = norm(z[:, Q:Q + C].float(), wkv_norm)
@@ -562,8 +618,9 @@ class TorchOps:
 
     def latent_q_prepare(self, q, q_lat, D, R, positions, cos, sin, rotary_dim, qq_out):
         T, H = qq_out.shape[0], qq_out.shape[1]
-        C = q_lat.shape[2]
-        qq_out[:, :, :C] = q_lat.transpose(0, 1)
+        C = qq_out.shape[2] - R
+        if q_lat is not None:
+            qq_out[:, :, :C] = q_lat.transpose(0, 1)
         turned = self._turn(q.view(T, H, D + R)[:, :, D:].float(), positions, cos, sin, rotary_dim)
         qq_out[:, :, C:] = turned.to(qq_out.dtype)
 
