@@ -171,9 +171,9 @@ def measured_peaks(runner, dtype):
 PROFILE_KERNELS = True      # --no-kernels: no profiler pass of bench.py's own (for runs under another profiler)
 
 
-def kernel_split(run, steps):
+def kernel_split(run, steps, top_n=10):
     """Device time of `steps` calls of run() by kernel, from a profiler pass of its own (outside every
-    timed region; what rollout/utils/prof_graph.py:64-101 does for the reference's decode): the ten
+    timed region; what rollout/utils/prof_graph.py:64-101 does for the reference's decode): the top_n
     kernels that take the most time, in microseconds per call, the rest as "other", and the sum."""
     import re
     import torch
@@ -205,10 +205,10 @@ def kernel_split(run, steps):
         if not per:
             return {"error": "the profiler saw no kernels"}
         top = sorted(per.items(), key=lambda kv: -kv[1][1])
-        out = {name: {"us": round(us / steps, 1), "calls": round(calls / steps, 1)} for name, (calls, us) in top[:10]}
-        rest = sum(us for _, (_, us) in top[10:])
+        out = {name: {"us": round(us / steps, 1), "calls": round(calls / steps, 1)} for name, (calls, us) in top[:top_n]}
+        rest = sum(us for _, (_, us) in top[top_n:])
         if rest > 0:
-            out["other"] = {"us": round(rest / steps, 1), "calls": round(sum(c for _, (c, _) in top[10:]) / steps, 1)}
+            out["other"] = {"us": round(rest / steps, 1), "calls": round(sum(c for _, (c, _) in top[top_n:]) / steps, 1)}
         out["sum_us"] = round(sum(us for _, us in per.values()) / steps, 1)
         return out
     except Exception as error:          # a measurement beside the bench: its failure is reported, not raised
@@ -1236,11 +1236,159 @@ def mepolix(args):
             "measured": peaks, "designs": out}
 
 
+# The Mapalorn design beside the Fefulorn design at equal sizes: --workload mapalorn
+def mapalorn_shape(width, heads, head_dim, ff, vocab, kv_rank=512, rot_dim=64, experts=32, top=4):
+    """config.json of a Mapalorn model of seven layers and eight layer runs: three latent attentions to one attention, the
+    first layer with a dense feed-forward, the others with routed experts (each ff / top channels) and a shared expert of the
+    same width, the third layer gone through twice."""
+    latent = {"type": "latent_attention",
+              "mixer": {"heads": heads, "dim": head_dim, "rot_dim": rot_dim, "vdim": head_dim, "kv_rank": kv_rank,
+                        "scale": (head_dim + rot_dim) ** -0.5, "rot": {"base": 1e6, "dims": rot_dim}}}
+    attn = {"type": "attention",
+            "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+                      "rot": {"base": 1e6, "dims": head_dim}}}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff // top}}
+    layers = [dict(latent, mlp=dense)] + [dict(kind, mlp=moe) for kind in (latent, latent, attn, latent, latent, attn)]
+    return {"architecture": "Mapalorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers,
+            "loop": {"start": 2, "stop": 3, "times": 2}}
+
+
+def fefulorn_attention_shape(width, heads, head_dim, ff, vocab, **kw):
+    """The Fefulorn design with attention layers alone, in the order of mapalorn_shape's layer runs: the latent attention
+    and the attention with every key in their windows, routed experts and a shared one in every layer."""
+    base = fefulorn_shape(width=width, heads=heads, head_dim=head_dim, ff=ff, layers=8, vocab=vocab, **kw)
+    kinds = {layer["type"]: dict(layer, mixer=dict(layer["mixer"], mask={"size": 16384})) for layer in base["layers"]}
+    order = ["latent_attention"] * 4 + ["attention"] + ["latent_attention"] * 2 + ["attention"]
+    return dict(base, layers=[kinds[name] for name in order])
+
+
+def _mapalorn_runs(raw):
+    loop = raw.get("loop") or {"start": 0, "stop": len(raw["layers"]), "times": 1}
+    a, b = loop["start"], loop["stop"]
+    return raw["layers"][:a] + raw["layers"][a:b] * loop["times"] + raw["layers"][b:]
+
+
+def _mapalorn_mixer_weights(layer, W):
+    """Elements of a mixer's matrices."""
+    m = layer["mixer"]
+    H, D, V = m["heads"], m["dim"], m["vdim"]
+    if layer["type"] == "latent_attention":
+        return (H * (D + m["rot_dim"]) + m["kv_rank"] + m["rot_dim"]) * W + H * (D + V) * m["kv_rank"] + W * H * V
+    return (H * D + m["kv_heads"] * (D + V) + H * V) * W + W * H * V
+
+
+def mapalorn_bytes(raw, elt, batch, ctx):
+    """Bytes one decode step has to move: every matrix once a layer run (of the experts those that the step's tokens are
+    expected to choose, every token choosing `top` of them evenly), the latent rows, keys and values, the head."""
+    W = raw["width"]
+    total = raw["vocab"] * W * elt
+    for layer in _mapalorn_runs(raw):
+        m, mlp = layer["mixer"], layer["mlp"]
+        total += _mapalorn_mixer_weights(layer, W) * elt
+        row = m["kv_rank"] + m["rot_dim"] if layer["type"] == "latent_attention" else m["kv_heads"] * (m["dim"] + m["vdim"])
+        total += batch * ctx * row * elt
+        if mlp["kind"] == "dense":
+            total += 3 * W * mlp["ff"] * elt
+        else:
+            E, top = mlp["router"]["experts"], mlp["router"]["top"]
+            total += (E * W + E * (1.0 - (1.0 - top / E) ** batch) * 3 * W * mlp["expert"]["ff"] + (3 * mlp["shared"]["ff"] + 1) * W) * elt
+    return total
+
+
+def mapalorn_flops(raw, T):
+    """Operations of a prompt of T tokens on the matrix cores: (as the design states them, and with the latent attention in
+    the form that reads the latent rows themselves)."""
+    W = raw["width"]
+    lin = raw["vocab"] * W / T
+    attn = latent = 0.0
+    keys = T * (T + 1) / 2
+    for layer in _mapalorn_runs(raw):
+        m, mlp = layer["mixer"], layer["mlp"]
+        lin += _mapalorn_mixer_weights(layer, W)
+        R = m.get("rot_dim", 0)
+        stated = keys * m["heads"] * 2.0 * (m["dim"] + R + m["vdim"])
+        attn += stated
+        latent += keys * m["heads"] * 2.0 * (2 * m["kv_rank"] + R) if layer["type"] == "latent_attention" else stated
+        lin += 3 * W * mlp["ff"] if mlp["kind"] == "dense" else \
+            mlp["router"]["experts"] * W + mlp["router"]["top"] * 3 * W * mlp["expert"]["ff"] + (3 * mlp["shared"]["ff"] + 1) * W
+    return 2.0 * T * lin + attn, 2.0 * T * lin + latent
+
+
+def mapalorn(args):
+    """Prefill of 2,048 tokens and decode at batch 1, 8 and 64 over 2,048-token prefixes of the Mapalorn design at two sizes
+    that resemble a model's layers (eight layer runs, random weights), each beside the Fefulorn design with attention layers
+    alone (the closest one here: sublayers side by side, latent attention and attention, experts with a shared one) with the
+    same width, heads, expert and latent sizes and number of layer runs, through the same engine; the step's time by kernel
+    for both. value: Mapalorn decode tok/s at batch 8 on the larger size."""
+    import torch
+    from return_amd.engine.runner import StepEntry
+    elt = 2 if args.dtype == "bfloat16" else 4
+    vocab = 32000
+    sizes = {"w2048": dict(width=2048, heads=16, head_dim=128, ff=8192),
+             "w4096": dict(width=4096, heads=32, head_dim=128, ff=12288)}
+    k, w = max(8, min(args.steps, 32)), min(args.warmup, 4)
+    out, peaks = {}, None
+    for tag, sz in sizes.items():
+        raws = {"mapalorn": (mapalorn_shape(vocab=vocab, **sz), mapalorn_flops, mapalorn_bytes),
+                "fefulorn": (fefulorn_attention_shape(vocab=vocab, **sz), fefulorn_flops, fefulorn_bytes)}
+        for design, (raw, flops_of, bytes_of) in raws.items():
+            cfg, runner = build_runner(0, args.dtype, 64, raw=raw, std=0.02, use_graphs=not args.no_graphs,
+                                       tune_products=not args.no_tune, defer_norms=not args.no_defer_norms)
+            if peaks is None:
+                peaks = measured_peaks(runner, args.dtype)
+            rec = {}
+            toks = [(7 * i + 3) % vocab for i in range(PREFILL_TOKENS)]
+
+            def prompt():
+                runner.add_request("p")
+                runner.step([StepEntry("p", toks, [PREFILL_TOKENS - 1])])
+                runner.free_request("p")
+            prompt()
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            for _ in range(3):
+                prompt()
+            torch.cuda.synchronize()
+            secs = (time.perf_counter() - t0) / 3
+            stated, as_run = flops_of(raw, PREFILL_TOKENS)[:2]
+            rec["prefill_2048"] = prefill_record(cfg, args.dtype, PREFILL_TOKENS, secs, peaks=peaks, flops=stated)
+            rec["prefill_2048"]["GFLOP_in_latent_form"] = round(as_run / 1e9, 1)
+            rec["prefill_2048"]["kernels"] = kernel_split(prompt, 2, 20)
+            for b in (1, 8, 64):
+                ids = seat_requests(runner, b, CONTEXT)
+                secs = decode_steps(runner, ids, k, w, vocab)
+                ms = secs / k * 1e3
+                point = {"tok_s": round(b * k / secs, 1), "ms_per_step": round(ms, 4)}
+                got = bytes_of(raw, elt, b, CONTEXT + w + (k + 1) // 2) / (ms * 1e-3) / 1e9
+                point.update({"bound": "hbm", "achieved": round(got, 1), "frac": round(got / PEAK_HBM_GBS, 4),
+                              "frac_of_measured": round(got / peaks["read_GBs"], 4)})
+
+                def one_step():
+                    t = runner.decode_launch(ids, None, [0.0] * b, [0] * b, [1.0] * b, [0.0] * b, feed_rows=list(range(b)))
+                    runner.decode_collect(t)
+                point["kernels"] = kernel_split(one_step, 4, 20)
+                release(runner, ids)
+                rec[f"decode_b{b}"] = point
+            out[f"{design}_{tag}"] = rec
+            print(f"bench.py: {design} {tag} measured", file=sys.stderr, flush=True)
+            del runner
+            torch.cuda.empty_cache()
+    head = out["mapalorn_w4096"]["decode_b8"]
+    return {"metric": "decode tok/s (Mapalorn design, width 4096, 8 layer runs, random weights)", "value": head["tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": k, "warmup": w, "ms_per_step": head["ms_per_step"],
+            "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic",
+            "config": {"model": "Mapalorn and Fefulorn designs at equal sizes", "layer_runs": 8, "vocab": vocab,
+                       "sizes": sizes, "global_batch": 8, "seq_len": CONTEXT, "parallelism": "single GPU"},
+            "measured": peaks, "designs": out}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--workload", default="decode_8b",
                     choices=["decode_8b", "continuous_4b", "long_32b", "contexts_8b", "products_8b", "decode_4b",
-                             "decode_32b", "kofipel", "rupezen", "safilorn", "fefulorn", "mepolix"],
+                             "decode_32b", "kofipel", "rupezen", "safilorn", "fefulorn", "mepolix", "mapalorn"],
                     help="decode_8b: the headline run; the others: the 4B and 32B shapes with their own "
                          "workloads (one JSON line each, other fields)")
     ap.add_argument("--gpus", type=int, default=1)
@@ -1274,7 +1422,9 @@ def main():
         return 1
     if args.workload != "decode_8b":
         print(json.dumps({"continuous_4b": continuous_4b, "long_32b": long_32b,
-                          "contexts_8b": contexts_8b, "products_8b": products_8b, "kofipel": kofipel, "rupezen": rupezen, "safilorn": safilorn, "fefulorn": fefulorn, "mepolix": mepolix,
+                          "contexts_8b": contexts_8b, "products_8b": products_8b, "kofipel": kofipel, "rupezen": rupezen, "safilorn": safilorn, "fefulorn": fefulorn,
+                          "mepolix": mepolix,
+                          "mapalorn": mapalorn,
                           "decode_4b": lambda a: decode_shape(a, QWEN3_4B, "Qwen3-4B", 0.02),
                           "decode_32b": lambda a: decode_shape(a, QWEN3_32B, "Qwen3-32B", 0.01)}[args.workload](args)))
         return 0

@@ -29,30 +29,73 @@
 #include "common.h"
 
 // ------------------------------------------------------------------ preparation
-template <typename T>
-__global__ __launch_bounds__(256) void latent_kv_prepare_kernel(
+__device__ __forceinline__ void lat_load4(const float* p, float (&v)[4]) {
+    const float4 t = *reinterpret_cast<const float4*>(p);
+    v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
+}
+__device__ __forceinline__ void lat_load4(const bf16* p, float (&v)[4]) {
+    const uint2 t = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u);
+    v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
+}
+
+__device__ __forceinline__ void lat_store4(float* p, const float (&v)[4]) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+__device__ __forceinline__ void lat_store4(bf16* p, const float (&v)[4]) {
+    uint2 t;
+    t.x = (uint32_t)f2bf_bits(v[0]) | ((uint32_t)f2bf_bits(v[1]) << 16);
+    t.y = (uint32_t)f2bf_bits(v[2]) | ((uint32_t)f2bf_bits(v[3]) << 16);
+    *reinterpret_cast<uint2*>(p) = t;
+}
+
+// V 4: the whole of R turns, four pairs a thread at a time (R a multiple of eight); V 1: element by element
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void latent_kv_prepare_kernel(
     const T* __restrict__ z, long long ld_z, int Q, int C, int R, const float* __restrict__ wq,
     const float* __restrict__ wc, float eps, const int* __restrict__ positions, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, int rot, T* __restrict__ cq_out, T* __restrict__ k_pool, T* __restrict__ v_pool,
     const int* __restrict__ slot_mapping, int P, const T* __restrict__ q, long long ld_q, int Hn, int D,
     T* __restrict__ qq) {
     __shared__ float scratch[16];
-    const int t = blockIdx.x, tid = threadIdx.x;
+    const int t = blockIdx.x, tid = threadIdx.x, nt = blockDim.x;
     const T* zr = z + (size_t)t * ld_z;
     float ss = 0.f;
     if (Q > 0) {
-        for (int i = tid; i < Q; i += 256) {
+        for (int i = tid; i < Q; i += nt) {
             const float a = to_f(zr[i]);
             ss = fmaf(a, a, ss);
         }
         const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)Q + eps);
-        for (int i = tid; i < Q; i += 256) cq_out[(size_t)t * Q + i] = from_f<T>(to_f(zr[i]) * rq * wq[i]);
+        for (int i = tid; i < Q; i += nt) cq_out[(size_t)t * Q + i] = from_f<T>(to_f(zr[i]) * rq * wq[i]);
     }
     if (q != nullptr) {
         const int half = rot >> 1, pos = positions[t];
         const T* qr = q + (size_t)t * ld_q + D;
         T* dst = qq + (size_t)t * Hn * (C + R) + C;
-        for (int j = tid; j < Hn * R; j += 256) {
+        if constexpr (V == 4) {
+            const int per = half / 4;
+            const float* cr = cos_t + (size_t)pos * half;
+            const float* sr = sin_t + (size_t)pos * half;
+            for (int j = tid; j < Hn * per; j += nt) {
+                const int h = j / per, i = (j - h * per) * 4;
+                const T* src = qr + (size_t)h * (D + R) + i;
+                T* to = dst + (size_t)h * (C + R) + i;
+                float u[4], v[4], cs[4], sn[4], a[4], b[4];
+                lat_load4(src, u);
+                lat_load4(src + half, v);
+                lat_load4(cr + i, cs);
+                lat_load4(sr + i, sn);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    a[e] = u[e] * cs[e] - v[e] * sn[e];
+                    b[e] = v[e] * cs[e] + u[e] * sn[e];
+                }
+                lat_store4(to, a);
+                lat_store4(to + half, b);
+            }
+        } else
+        for (int j = tid; j < Hn * R; j += nt) {
             const int h = j / R, i = j - h * R;
             const T* src = qr + (size_t)h * (D + R);
             float v = to_f(src[i]);
@@ -67,7 +110,7 @@ __global__ __launch_bounds__(256) void latent_kv_prepare_kernel(
     }
     if (v_pool == nullptr) return;
     ss = 0.f;
-    for (int i = tid; i < C; i += 256) {
+    for (int i = tid; i < C; i += nt) {
         const float a = to_f(zr[Q + i]);
         ss = fmaf(a, a, ss);
     }
@@ -75,10 +118,10 @@ __global__ __launch_bounds__(256) void latent_kv_prepare_kernel(
     const int slot = slot_mapping[t];
     if (slot < 0) return;
     T* vr = v_pool + ra_cache_offset(slot, 0, 1, P, C);
-    for (int i = tid; i < C; i += 256) vr[i] = from_f<T>(to_f(zr[Q + i]) * rc * wc[i]);
+    for (int i = tid; i < C; i += nt) vr[i] = from_f<T>(to_f(zr[Q + i]) * rc * wc[i]);
     T* kr = k_pool + ra_cache_offset(slot, 0, 1, P, R);
     const int half = rot >> 1, pos = positions[t];
-    for (int i = tid; i < R; i += 256) {
+    for (int i = tid; i < R; i += nt) {
         float v = to_f(zr[Q + C + i]);
         if (i < rot) {
             const int f = i < half ? i : i - half;
@@ -101,17 +144,19 @@ extern "C" int ra_latent_kv_prepare(const void* z, long long ld_z, int T_tokens,
         (v_pool != nullptr && R > 0 && k_pool == nullptr) || (Q > 0 && (wq == nullptr || cq_out == nullptr)) ||
         (q != nullptr && (Hn < 1 || D < 0 || ld_q < (long long)Hn * (D + R) || qq == nullptr || (long long)Hn * R > 0x7fffffffLL)))
         return RA_ERR_ARG;
+    if (dtype != RA_DTYPE_F32 && dtype != RA_DTYPE_BF16) return RA_ERR_ARG;
     hipStream_t st = (hipStream_t)stream;
-    if (dtype == RA_DTYPE_F32)
-        hipLaunchKernelGGL(latent_kv_prepare_kernel<float>, dim3(T_tokens), dim3(256), 0, st, (const float*)z, ld_z, Q, C, R,
-                           wq, wc, eps, positions, cos_t, sin_t, rot, (float*)cq_out, (float*)k_pool, (float*)v_pool,
-                           slot_mapping, P, (const float*)q, ld_q, Hn, D, (float*)qq);
-    else if (dtype == RA_DTYPE_BF16)
-        hipLaunchKernelGGL(latent_kv_prepare_kernel<bf16>, dim3(T_tokens), dim3(256), 0, st, (const bf16*)z, ld_z, Q, C, R,
-                           wq, wc, eps, positions, cos_t, sin_t, rot, (bf16*)cq_out, (bf16*)k_pool, (bf16*)v_pool,
-                           slot_mapping, P, (const bf16*)q, ld_q, Hn, D, (bf16*)qq);
-    else
-        return RA_ERR_ARG;
+    const auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    const bool vec = q != nullptr && rot == R && R % 8 == 0 && R > 0 && D % 4 == 0 && C % 4 == 0 && ld_q % 4 == 0 && aligned(q) &&
+                     aligned(qq) && aligned(cos_t) && aligned(sin_t);
+    const int threads = T_tokens <= 256 && (long long)Hn * R + Q + C > 1024 ? 1024 : 256;      // few tokens: fewer rounds of reads
+#define LAT_PREPARE(T_, V_)                                                                                              \
+    hipLaunchKernelGGL((latent_kv_prepare_kernel<T_, V_>), dim3(T_tokens), dim3(threads), 0, st, (const T_*)z, ld_z, Q, C, R, wq, \
+                       wc, eps, positions, cos_t, sin_t, rot, (T_*)cq_out, (T_*)k_pool, (T_*)v_pool, slot_mapping, P,    \
+                       (const T_*)q, ld_q, Hn, D, (T_*)qq)
+    if (dtype == RA_DTYPE_F32) { if (vec) LAT_PREPARE(float, 4); else LAT_PREPARE(float, 1); }
+    else { if (vec) LAT_PREPARE(bf16, 4); else LAT_PREPARE(bf16, 1); }
+#undef LAT_PREPARE
     return ra_launch_status();
 }
 
@@ -163,16 +208,6 @@ extern "C" int ra_latent_q_prepare(const void* q, const void* q_lat, int T_token
 // ------------------------------------------------------------------ the plain kernel
 #define LAT_MAX_ACC 8       // C <= 64 * 8
 #define LAT_BLOCK 64
-
-__device__ __forceinline__ void lat_load4(const float* p, float (&v)[4]) {
-    const float4 t = *reinterpret_cast<const float4*>(p);
-    v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
-}
-__device__ __forceinline__ void lat_load4(const bf16* p, float (&v)[4]) {
-    const uint2 t = *reinterpret_cast<const uint2*>(p);
-    v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u);
-    v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
-}
 
 template <typename T, int QR, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void attn_latent_plain_kernel(

@@ -381,12 +381,14 @@ extern "C" int ra_attention_latent_mfma_tile_tokens(int Hn) {
 }
 
 // The sums of a tile's splits into its output rows: the splits' maxima, sums and unnormed rows are merged in split
-// order, the sink's term joins the denominator. One wave per (tile, head); the tile's one token is row cu_q[request].
-__global__ __launch_bounds__(64) void attn_latent_merge_kernel(const float* __restrict__ part, bf16* __restrict__ out,
-                                                               const int* __restrict__ tiles, const int* __restrict__ cu_q,
-                                                               int T_rows, int Hn, int C, int n_splits, float scale,
-                                                               const float* __restrict__ sink) {
-    const int tile = blockIdx.x / Hn, head = blockIdx.x % Hn, lane = threadIdx.x;
+// order, the sink's term joins the denominator. One workgroup per (tile, head); its waves take equal runs of the splits
+// that hold anything, whose sums are added in wave order; the tile's one token is row cu_q[request].
+#define LAT_MERGE_WAVES 4
+__global__ __launch_bounds__(64 * LAT_MERGE_WAVES) void attn_latent_merge_kernel(
+    const float* __restrict__ part, bf16* __restrict__ out, const int* __restrict__ tiles, const int* __restrict__ cu_q,
+    int T_rows, int Hn, int C, int n_splits, float scale, const float* __restrict__ sink) {
+    __shared__ float sums[LAT_MERGE_WAVES][512 + 1];
+    const int tile = blockIdx.x / Hn, head = blockIdx.x % Hn, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const float scale2 = scale * LAT_LOG2E;
     const float* pp = part + (size_t)blockIdx.x * n_splits * (C + 2);
     const int token_row = cu_q[tiles[2 * tile]] + tiles[2 * tile + 1];
@@ -398,32 +400,47 @@ __global__ __launch_bounds__(64) void attn_latent_merge_kernel(const float* __re
     const float M2 = (m_all == -INFINITY) ? -INFINITY : m_all * scale2;
     const float s2 = sink != nullptr ? sink[head] * LAT_LOG2E : -INFINITY;
     const float top = fmaxf(M2, s2);
-    // weight of split sp's sums under the common maximum `top`
+    // weight of split sp's sums under the common maximum `top`; splits beyond the last that holds anything are not read
     const float my_w = (my_m == -INFINITY || top == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(my_m * scale2 - top);
+    const unsigned long long held = __ballot(my_m != -INFINITY);
+    const int used = held == 0 ? 0 : 64 - __builtin_clzll(held);
+    const int per = (used + LAT_MERGE_WAVES - 1) / LAT_MERGE_WAVES;
+    const int first = wave * per, last = min(used, first + per);
     float l = 0.f, a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};       // elements lane, lane + 64, ... (C <= 512)
-    for (int s0 = 0; s0 < n_splits; s0 += 4) {           // four splits' rows asked for at once, added in split order
+    for (int s0 = first; s0 < last; s0 += 4) {           // four splits' rows asked for at once, added in split order
         float raw[4][8];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const float* pm = pp + (size_t)min(s0 + j, n_splits - 1) * (C + 2) + 2;
+            const float* pm = pp + (size_t)min(s0 + j, last - 1) * (C + 2) + 2;
 #pragma unroll
             for (int i = 0; i < 8; ++i) raw[j][i] = lane + 64 * i < C ? pm[lane + 64 * i] : 0.f;
         }
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            if (s0 + j >= n_splits) break;
+            if (s0 + j >= last) break;
             const float wgt = __shfl(my_w, s0 + j, 64);
             l = fmaf(__shfl(my_l, s0 + j, 64), wgt, l);
 #pragma unroll
             for (int i = 0; i < 8; ++i) a[i] = fmaf(raw[j][i], wgt, a[i]);
         }
     }
-    if (sink != nullptr && top != -INFINITY) l += __builtin_amdgcn_exp2f(s2 - top);
-    const float f = l > 0.f ? 1.0f / l : 0.f;
-    bf16* op = out + ((size_t)head * T_rows + token_row) * C;
 #pragma unroll
     for (int i = 0; i < 8; ++i)
-        if (lane + 64 * i < C) op[lane + 64 * i] = from_f<bf16>(a[i] * f);
+        if (lane + 64 * i < C) sums[wave][lane + 64 * i] = a[i];
+    if (lane == 0) sums[wave][512] = l;
+    __syncthreads();
+    float den = 0.f;
+#pragma unroll
+    for (int w = 0; w < LAT_MERGE_WAVES; ++w) den += sums[w][512];
+    if (sink != nullptr && top != -INFINITY) den += __builtin_amdgcn_exp2f(s2 - top);
+    const float f = den > 0.f ? 1.0f / den : 0.f;
+    bf16* op = out + ((size_t)head * T_rows + token_row) * C;
+    for (int e = threadIdx.x; e < C; e += 64 * LAT_MERGE_WAVES) {
+        float v = 0.f;
+#pragma unroll
+        for (int w = 0; w < LAT_MERGE_WAVES; ++w) v += sums[w][e];
+        op[e] = from_f<bf16>(v * f);
+    }
 }
 
 // floats of the buffer that n_splits > 1 needs for n_tiles one-token tiles
@@ -486,7 +503,7 @@ extern "C" int ra_attention_latent_mfma_window_bf16(const void* qq, void* out, c
 #undef LAT_GO
     if (rc != RA_OK) return rc;
     if (n_splits > 1)
-        hipLaunchKernelGGL(attn_latent_merge_kernel, dim3(n_tiles * Hn), dim3(64), 0, st, part, (bf16*)out, tiles, cu_q,
+        hipLaunchKernelGGL(attn_latent_merge_kernel, dim3(n_tiles * Hn), dim3(64 * LAT_MERGE_WAVES), 0, st, part, (bf16*)out, tiles, cu_q,
                            T_rows, Hn, C, n_splits, scale, sink);
     return ra_launch_status();
 }

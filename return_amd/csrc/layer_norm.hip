@@ -127,7 +127,8 @@ __device__ __forceinline__ float ln_terms(const LnTerms<T>& d, size_t r, int H, 
     return v;
 }
 
-template <typename T, bool VEC>
+// G > 0: groups of four neighbours a thread (H a multiple of four, at most 4 G threads); G 0: element by element
+template <typename T, int G>
 __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restrict__ h, const int* __restrict__ rows,
                                                                  const LnTerms<T> d, const float* __restrict__ w,
                                                                  const float* __restrict__ bias, float eps,
@@ -140,10 +141,10 @@ __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restri
     const bool adds = d.a != nullptr || d.b != nullptr;
     const bool keep = adds && rows == nullptr;
     const float gate = d.extra != nullptr ? 1.0f / (1.0f + expf(-d.logit[r * d.ld_logit])) : 0.f;
-    if constexpr (VEC) {
-        float v[LN_G][4], av[LN_G][4], sv[LN_G][4], ev[LN_G][4], wv[LN_G][4], bv[LN_G][4];
+    if constexpr (G > 0) {
+        float v[G][4], av[G][4], sv[G][4], ev[G][4], wv[G][4], bv[G][4];
 #pragma unroll
-        for (int g = 0; g < LN_G; ++g) {
+        for (int g = 0; g < G; ++g) {
             const int c = (threadIdx.x + g * nt) * 4;
 #pragma unroll
             for (int e = 0; e < 4; ++e) v[g][e] = av[g][e] = sv[g][e] = ev[g][e] = wv[g][e] = bv[g][e] = 0.f;
@@ -156,24 +157,32 @@ __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restri
             }
         }
         if (d.b != nullptr) {
-            for (int k = 0; k < d.nb; ++k) {
-                const float f = d.wb != nullptr ? d.wb[r * d.nb + k] : 1.0f;
-                float t[LN_G][4];
+            // several rows at a time, all their reads asked for before the first sum (a row beyond the last counts nothing)
+            constexpr int KU = 4 / G;
+            for (int k0 = 0; k0 < d.nb; k0 += KU) {
+                float t[KU][G][4], f[KU];
 #pragma unroll
-                for (int g = 0; g < LN_G; ++g) {
-                    const int c = (threadIdx.x + g * nt) * 4;
-                    t[g][0] = t[g][1] = t[g][2] = t[g][3] = 0.f;
-                    if (c < H) ln_load4(d.b + (r * d.nb + k) * H + c, t[g]);
+                for (int u = 0; u < KU; ++u) {
+                    const int k = min(k0 + u, d.nb - 1);
+                    f[u] = k0 + u >= d.nb ? 0.f : d.wb != nullptr ? d.wb[r * d.nb + k] : 1.0f;
+#pragma unroll
+                    for (int g = 0; g < G; ++g) {
+                        const int c = (threadIdx.x + g * nt) * 4;
+                        t[u][g][0] = t[u][g][1] = t[u][g][2] = t[u][g][3] = 0.f;
+                        if (c < H && k0 + u < d.nb) ln_load4(d.b + (r * d.nb + k) * H + c, t[u][g]);
+                    }
                 }
 #pragma unroll
-                for (int g = 0; g < LN_G; ++g)
+                for (int u = 0; u < KU; ++u)
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) sv[g][e] = fmaf(f, t[g][e], sv[g][e]);
+                    for (int g = 0; g < G; ++g)
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) sv[g][e] = fmaf(f[u], t[u][g][e], sv[g][e]);
             }
         }
         float sum = 0.f;
 #pragma unroll
-        for (int g = 0; g < LN_G; ++g) {
+        for (int g = 0; g < G; ++g) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 if (d.extra != nullptr) sv[g][e] = fmaf(ev[g][e], gate, sv[g][e]);
@@ -183,7 +192,7 @@ __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restri
         }
         if (keep) {
 #pragma unroll
-            for (int g = 0; g < LN_G; ++g) {
+            for (int g = 0; g < G; ++g) {
                 const int c = (threadIdx.x + g * nt) * 4;
                 if (c < H) ln_store4(hr + c, v[g]);
             }
@@ -191,7 +200,7 @@ __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restri
         const float mean = block_sum(sum, scratch) / (float)H;
         float ss = 0.f;
 #pragma unroll
-        for (int g = 0; g < LN_G; ++g) {
+        for (int g = 0; g < G; ++g) {
             const bool in = (threadIdx.x + g * nt) * 4 < H;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
@@ -201,7 +210,7 @@ __global__ __launch_bounds__(1024) void stream_layer_norm_kernel(float* __restri
         }
         const float rstd = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
 #pragma unroll
-        for (int g = 0; g < LN_G; ++g) {
+        for (int g = 0; g < G; ++g) {
             const int c = (threadIdx.x + g * nt) * 4;
             if (c < H) {
 #pragma unroll
@@ -267,19 +276,23 @@ extern "C" int ra_stream_layer_norm(float* h, const void* a, const void* b, int 
         return RA_ERR_ARG;
     hipStream_t st = (hipStream_t)stream;
     auto al = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
-    const bool vec = H % 4 == 0 && H <= 4 * LN_G * 1024 && al(h) && al(a) && al(b) && al(extra) && al(w) && al(bias) && al(out);
-    // (a row of up to 4,096 elements by 256 threads; longer rows by as many as keep it in registers)
-    const int threads = H <= 4 * LN_G * 256 ? 256 : H <= 4 * LN_G * 512 ? 512 : 1024;
-#define LN_STREAM(T_, V_)                                                                                             \
+    const bool vec = H % 4 == 0 && H <= 16 * 1024 && al(h) && al(a) && al(b) && al(extra) && al(w) && al(bias) && al(out);
+    // few rows: one group of four neighbours a thread, so that all of a row is on its way at once; many rows: 256 threads
+    // with as many groups as the row has; rows beyond 4,096 elements: four groups a thread
+    const int groups = rows <= 256 && H <= 4096 ? 1 : H <= 1024 ? 1 : H <= 2048 ? 2 : 4;
+    const int threads = groups == 4 ? (H <= 4096 ? 256 : H <= 8192 ? 512 : 1024) : std::max(64, (H / (4 * groups) + 63) / 64 * 64);
+#define LN_STREAM(T_, G_)                                                                                             \
     do {                                                                                                              \
         const LnTerms<T_> d = {(const T_*)a, (const T_*)b, nb, wb, (const T_*)extra, logit, ld_logit};                \
-        hipLaunchKernelGGL((stream_layer_norm_kernel<T_, V_>), dim3(rows), dim3(threads), 0, st, h, row_ids, d, w, bias, eps, \
+        hipLaunchKernelGGL((stream_layer_norm_kernel<T_, G_>), dim3(rows), dim3(threads), 0, st, h, row_ids, d, w, bias, eps, \
                            (T_*)out, H);                                                                              \
     } while (0)
     if (dtype == RA_DTYPE_F32) {
-        if (vec) LN_STREAM(float, true); else LN_STREAM(float, false);
+        if (!vec) LN_STREAM(float, 0); else if (groups == 1) LN_STREAM(float, 1); else if (groups == 2) LN_STREAM(float, 2);
+        else LN_STREAM(float, 4);
     } else if (dtype == RA_DTYPE_BF16) {
-        if (vec) LN_STREAM(bf16, true); else LN_STREAM(bf16, false);
+        if (!vec) LN_STREAM(bf16, 0); else if (groups == 1) LN_STREAM(bf16, 1); else if (groups == 2) LN_STREAM(bf16, 2);
+        else LN_STREAM(bf16, 4);
     } else {
         return RA_ERR_ARG;
     }

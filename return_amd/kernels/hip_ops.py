@@ -1822,9 +1822,9 @@ class HipOps:
             _ptr(q), _ptr(out), _ptr(k_pool), _ptr(v_pool), *tabs, None, 0, step.n_seqs, T, n_q, n_kv, D2 // 2, Dv, P,
             *consts, _code(q.dtype), self._stream()), "attention_diff_plain")
 
-    def _diff_decode_splits(self, step, n_heads, window, chunk):
+    def _diff_decode_splits(self, step, n_heads, window, chunk, per_cu=8, least=4):
         """Workgroups that share the keys of a request that brings one token: enough of them to fill the chip
-        (about eight a CU), at least four blocks of 64 keys each. Decided by the step's class (the batch size and
+        (about `per_cu` a CU), at least `least` blocks of 64 keys each. Decided by the step's class (the batch size and
         context bucket of the graph that serves or would serve it) where the runner names one, so that a step run
         eagerly and its replay from a graph sum in the same order."""
         rule = getattr(step, "decode_rule", None)
@@ -1835,8 +1835,8 @@ class HipOps:
         if chunk > 0:
             keys = min(keys, chunk)
         blocks = -(-max(int(keys), 1) // 64)
-        want = -(-8 * self.cu_count // max(1, n * n_heads))
-        return int(max(1, min(64, want, blocks // 4)))
+        want = -(-per_cu * self.cu_count // max(1, n * n_heads))
+        return int(max(1, min(64, want, blocks // least)))
 
     # ------------------------------------------------------------------ attention over a latent row per token
     def check_attention_latent_sizes(self, n_heads, C, R, dtype):
@@ -1954,7 +1954,12 @@ class HipOps:
                     tiles = self._unit_tiles[:step.n_decode]
                 else:
                     tiles = torch.stack([step.decode_segs, torch.zeros_like(step.decode_segs)], dim=1).contiguous()
-                lists.append((tiles, self._diff_decode_splits(step, 1, window, 0)))
+                # A block of 64 keys is 6.7 µs of one workgroup's time whatever the heads, and a workgroup's tile of long
+                # rows fills half a CU's LDS: one workgroup a CU, down to one block each (measured with rows of 512 + 64
+                # at 16 and 32 heads: 2,048 keys, batch 1 23 µs against 39 with four blocks at least, batch 8 26 against
+                # 40; batch 64 73 with one workgroup a CU against 80 with two and 93 with four; 8,192 keys 38 against 121,
+                # 50 against 124, 266 against 277)
+                lists.append((tiles, self._diff_decode_splits(step, 1, window, 0, 1 if C + R >= 320 else 2, 1)))
             for tiles, splits in lists:
                 part = None
                 if splits > 1:
